@@ -29,7 +29,8 @@ template <typename T>
 __global__ __launch_bounds__(GEN_THREADS) void paged_attention_generic_kernel(
     const T* __restrict__ q, long q_stride, T* __restrict__ out, long out_stride, const T* __restrict__ k_pages,
     const T* __restrict__ v_pages, const int* __restrict__ block_tables, int bt_width, const int* __restrict__ seg,
-    const int* __restrict__ pos, int nh, int nkv, int d, int ps, float scale, int window, float softcap) {
+    const int* __restrict__ pos, int nh, int nkv, int d, int ps, float scale, int window, float softcap,
+    const float* __restrict__ bias) {
   extern __shared__ float smem[];
   float* sq = smem;                       // [d] query, pre-scaled
   float* sp = sq + d;                     // [256] scores, then probabilities
@@ -43,6 +44,8 @@ __global__ __launch_bounds__(GEN_THREADS) void paged_attention_generic_kernel(
   const int lo = first_visible_key(p, window);
   const int g = h / (nh / nkv);
   const int* bt = block_tables + (long)s * bt_width;
+
+  const float r1 = bias ? bias[h] : 0.f, r2 = bias ? bias[nh + h] : 0.f;
 
   for (int i = tid; i < d; i += GEN_THREADS) sq[i] = to_f32<T>(q[(long)t * q_stride + h * d + i]) * scale;
 
@@ -67,6 +70,7 @@ __global__ __launch_bounds__(GEN_THREADS) void paged_attention_generic_kernel(
                sq[i + 3] * to_f32<T>(kr[i + 3]);
       }
       sc = softcap > 0.f ? softcap * tanhf(dot / softcap) : dot;   // scores bounded by cap tanh(s / cap)
+      if (bias) sc -= r1 * log1pf(r2 * (float)(p - j));            // what the distance takes off
     }
     const float cmax = block_max(sc, red);
     const float m_new = fmaxf(m, cmax);
@@ -114,11 +118,13 @@ __global__ __launch_bounds__(GEN_THREADS) void paged_attention_generic_kernel(
 }
 
 // ``softcap`` c > 0: a score s (after the scale) becomes c tanh(s / c) before the softmax; 0: scores as they are.
-extern "C" int lmsf_paged_attention_generic_capped(const void* q, long q_stride, void* out, long out_stride,
+// ``bias`` float32 [2, nh] or null: r1_h ln(1 + r2_h (i - j)) comes off the score of query i and key j (r2 >= 0),
+// after the cap.
+extern "C" int lmsf_paged_attention_generic_biased(const void* q, long q_stride, void* out, long out_stride,
                                                    const void* k_pages, const void* v_pages, long num_pages,
                                                    const int* block_tables, int bt_width, const int* seg,
                                                    const int* pos, int n_tokens, int nh, int nkv, int d, int ps,
-                                                   float scale, int window, float softcap, int dtype,
+                                                   float scale, int window, float softcap, const float* bias, int dtype,
                                                    hipStream_t stream) {
   LMSF_CHECK(softcap >= 0.f, "paged_attention: the soft cap must be >= 0, got %g", (double)softcap);
   LMSF_CHECK(q && out && k_pages && v_pages && block_tables && seg && pos, "paged_attention: null pointer");
@@ -135,11 +141,11 @@ extern "C" int lmsf_paged_attention_generic_capped(const void* q, long q_stride,
   if (dtype == LMSF_F32)
     hipLaunchKernelGGL((paged_attention_generic_kernel<float>), grid, block, smem, stream, (const float*)q, q_stride,
                        (float*)out, out_stride, (const float*)k_pages, (const float*)v_pages, block_tables, bt_width,
-                       seg, pos, nh, nkv, d, ps, scale, window, softcap);
+                       seg, pos, nh, nkv, d, ps, scale, window, softcap, bias);
   else
     hipLaunchKernelGGL((paged_attention_generic_kernel<bf16_t>), grid, block, smem, stream, (const bf16_t*)q, q_stride,
                        (bf16_t*)out, out_stride, (const bf16_t*)k_pages, (const bf16_t*)v_pages, block_tables,
-                       bt_width, seg, pos, nh, nkv, d, ps, scale, window, softcap);
+                       bt_width, seg, pos, nh, nkv, d, ps, scale, window, softcap, bias);
   LMSF_LAUNCH_CHECK("paged_attention_generic");
   return 0;
 }
@@ -149,7 +155,7 @@ extern "C" int lmsf_paged_attention_generic(const void* q, long q_stride, void* 
                                             const int* block_tables, int bt_width, const int* seg, const int* pos,
                                             int n_tokens, int nh, int nkv, int d, int ps, float scale, int window,
                                             int dtype, hipStream_t stream) {
-  return lmsf_paged_attention_generic_capped(q, q_stride, out, out_stride, k_pages, v_pages, num_pages, block_tables,
-                                             bt_width, seg, pos, n_tokens, nh, nkv, d, ps, scale, window, 0.f, dtype,
-                                             stream);
+  return lmsf_paged_attention_generic_biased(q, q_stride, out, out_stride, k_pages, v_pages, num_pages, block_tables,
+                                             bt_width, seg, pos, n_tokens, nh, nkv, d, ps, scale, window, 0.f, nullptr,
+                                             dtype, stream);
 }

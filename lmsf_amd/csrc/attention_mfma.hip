@@ -113,16 +113,28 @@ __device__ __forceinline__ float capped_score(float r, float cap_raw) {
   return cap_raw * (1.f - 2.f * __builtin_amdgcn_rcpf(e + 1.f));
 }
 
+// What a distance takes off a score (BIAS): r1_h ln(1 + r2_h (i - j)), the head's numbers from ``bias`` [2, nh] (the r1
+// of all heads, then their r2), after the cap. Raw scores are multiplied by scale log2 e later, and r1 ln x * log2 e is
+// r1 log2 x: a raw score loses (r1 / scale_log2) log2(1 + r2 (i - j)), with the hardware's logarithm.
+struct DistanceBias {
+  float b1, r2;
+  __device__ __forceinline__ void load(const float* __restrict__ bias, int nh, int head, float scale_log2) {
+    b1 = bias[head] / scale_log2;
+    r2 = bias[nh + head];
+  }
+  // (keys behind the query are masked by the caller: any finite number)
+  __device__ __forceinline__ float off(int diff) const { return b1 * __builtin_amdgcn_logf(fmaf(r2, (float)max(diff, 0), 1.f)); }
+};
 
 // One workgroup of 4 waves per (tile, kv head, block of HB heads of its group). Wave w owns the rows
 // (w * NQB + j) * 16 + c, j < NQB, c = lane % 16; row r is token r / HB of the tile and head r % HB of
 // the block. tiles[2 i], tiles[2 i + 1]: first flat token and number of tokens of tile i.
-template <int DPAD, int NQB, int WP = 1>
+template <int DPAD, int NQB, int WP = 1, bool BIAS = false>
 __global__ __launch_bounds__(256) void attn_prefill_mfma_kernel(
     const bf16_t* __restrict__ q, long q_stride, bf16_t* __restrict__ out, long out_stride,
     const bf16_t* __restrict__ k_pages, const bf16_t* __restrict__ v_pages, const int* __restrict__ block_tables,
     int btw, const int* __restrict__ tiles, const int* __restrict__ seg, const int* __restrict__ pos, int nh, int nkv,
-    int d, int ps, float scale_log2, float cap_raw, int window, int HB, int n_hb) {
+    int d, int ps, float scale_log2, float cap_raw, int window, int HB, int n_hb, const float* __restrict__ bias) {
   constexpr int DS = DPAD / 32, DV = DPAD / 16;
   const int tile = blockIdx.x;
   const int kvh = blockIdx.y / n_hb, hb = blockIdx.y - kvh * n_hb;
@@ -134,6 +146,7 @@ __global__ __launch_bounds__(256) void attn_prefill_mfma_kernel(
   G.bt = block_tables + (long)seg[t0] * btw;
 
   int rpos[NQB], rlo[NQB];
+  DistanceBias db[NQB];
   long qoff[NQB], ooff[NQB];
   int wmax = -1, wlo = INT_MAX;
 #pragma unroll
@@ -146,6 +159,7 @@ __global__ __launch_bounds__(256) void attn_prefill_mfma_kernel(
     rpos[j] = p;
     rlo[j] = p >= 0 ? first_visible_key(p, window) : 0;
     const int head = kvh * n_rep + (valid ? hin : 0);
+    if constexpr (BIAS) db[j].load(bias, nh, head, scale_log2);
     qoff[j] = (long)tok * q_stride + (long)head * d;
     ooff[j] = (long)tok * out_stride + (long)head * d;
     wmax = max(wmax, p);
@@ -221,6 +235,7 @@ __global__ __launch_bounds__(256) void attn_prefill_mfma_kernel(
         for (int i = 0; i < 4; ++i) {
           const int key = kbase + b * 16 + g * 4 + i;
           const bool ok = key <= rpos[j] && key >= rlo[j];
+          if constexpr (BIAS) st[b][j][i] -= db[j].off(rpos[j] - key);
           const float x = ok ? st[b][j][i] * scale_log2 : -INFINITY;
           sv[b * 4 + i] = x;
           mx = fmaxf(mx, x);
@@ -353,12 +368,13 @@ __device__ __forceinline__ unsigned lds_address(const void* p) {
 #define PREFILL_BT_CAP 2048
 #define PREFILL_BT_CAP_SMALL 64
 #define PREFILL_BT_PAD 8
-template <int DPAD, int NQB, int STAGES, int NW, int WP = 1>
+template <int DPAD, int NQB, int STAGES, int NW, int WP = 1, bool BIAS = false>
 __global__ __launch_bounds__(NW * 64, (NW == 8 ? 4 : 1)) void attn_prefill_dma_kernel(
     const bf16_t* __restrict__ q, long q_stride, bf16_t* __restrict__ out, long out_stride,
     const bf16_t* __restrict__ k_pages, const bf16_t* __restrict__ v_pages, const int* __restrict__ block_tables,
     int btw, const int* __restrict__ tiles, const int* __restrict__ seg, const int* __restrict__ pos, int nh, int nkv,
-    int d, int ps_log2, float scale_log2, float cap_raw, int window, int HB, int n_hb, int bt_cap, int n_cus) {
+    int d, int ps_log2, float scale_log2, float cap_raw, int window, int HB, int n_hb, int bt_cap, int n_cus,
+    const float* __restrict__ bias) {
   constexpr int DS = DPAD / 32, DV = DPAD / 16;
   constexpr int PR = DPAD / 8;                   // 16-byte pieces per K row
   constexpr bool PR_POW2 = (PR & (PR - 1)) == 0;
@@ -399,6 +415,7 @@ __global__ __launch_bounds__(NW * 64, (NW == 8 ? 4 : 1)) void attn_prefill_dma_k
   for (int i = tid; i < min(n_blk, bt_cap) + PREFILL_BT_PAD; i += NW * 64) lds_bt[i] = bt[blk0 + min(i, n_blk - 1)];
 
   int rpos[NQB], rlo[NQB];
+  DistanceBias db[NQB];
   long qoff[NQB], ooff[NQB];
   int wmax = -1, wlo = INT_MAX, wminpos = INT_MAX, wmaxlo = 0;
 #pragma unroll
@@ -411,6 +428,7 @@ __global__ __launch_bounds__(NW * 64, (NW == 8 ? 4 : 1)) void attn_prefill_dma_k
     rpos[j] = p;
     rlo[j] = p >= 0 ? first_visible_key(p, window) : 0;
     const int head = kvh * n_rep + (valid ? hin : 0);
+    if constexpr (BIAS) db[j].load(bias, nh, head, scale_log2);
     qoff[j] = (long)tok * q_stride + (long)head * d;
     ooff[j] = (long)tok * out_stride + (long)head * d;
     wmax = max(wmax, p);
@@ -609,6 +627,10 @@ __global__ __launch_bounds__(NW * 64, (NW == 8 ? 4 : 1)) void attn_prefill_dma_k
 #pragma unroll
           for (int e = 0; e < 8; ++e) r[e] = capped_score(r[e], cap_raw);
         }
+        if constexpr (BIAS) {
+#pragma unroll
+          for (int e = 0; e < 8; ++e) r[e] -= db[j].off(rpos[j] - (kbase + g * 8 + e));
+        }
         if (need_mask) {
 #pragma unroll
           for (int e = 0; e < 8; ++e) {
@@ -688,11 +710,12 @@ __global__ __launch_bounds__(NW * 64, (NW == 8 ? 4 : 1)) void attn_prefill_dma_k
 }
 
 
-template <int DPAD, int WP>
+template <int DPAD, int WP, bool BIAS>
 static int launch_prefill_dma(dim3 grid, hipStream_t stream, const bf16_t* q, long q_stride, bf16_t* out,
                               long out_stride, const bf16_t* k_pages, const bf16_t* v_pages, const int* block_tables,
                               int btw, const int* tiles, const int* seg, const int* pos, int nh, int nkv, int d, int ps,
-                              float scale_log2, float cap_raw, int window, int HB, int n_hb, int bt_cap) {
+                              float scale_log2, float cap_raw, int window, int HB, int n_hb, int bt_cap,
+                              const float* bias) {
   int ps_log2 = 0;
   while ((1 << ps_log2) < ps) ++ps_log2;
   // four stages of a head size of 128 and the table are 72 KB: two workgroups share a compute unit's LDS,
@@ -703,7 +726,7 @@ static int launch_prefill_dma(dim3 grid, hipStream_t stream, const bf16_t* q, lo
   // waves on every SIMD, which hide each other's waits.
   constexpr int NW = (DPAD == 64 || DPAD == 128) ? 8 : 4;
   const size_t smem = (size_t)STAGES * 4 * 32 * DPAD + (PREFILL_BT_CAP + PREFILL_BT_PAD) * sizeof(int);
-  auto kernel = attn_prefill_dma_kernel<DPAD, 8 / NW, STAGES, NW, WP>;
+  auto kernel = attn_prefill_dma_kernel<DPAD, 8 / NW, STAGES, NW, WP, BIAS>;
   static bool configured = false;   // per instantiation
   if (!configured) {
     hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel),
@@ -716,7 +739,7 @@ static int launch_prefill_dma(dim3 grid, hipStream_t stream, const bf16_t* q, lo
   }
   hipLaunchKernelGGL(kernel, dim3(grid.x * grid.y), dim3(NW * 64), smem, stream, q, q_stride, out, out_stride, k_pages,
                      v_pages, block_tables, btw, tiles, seg, pos, nh, nkv, d, ps_log2, scale_log2, cap_raw, window, HB, n_hb,
-                     bt_cap, lmsf_compute_units());
+                     bt_cap, lmsf_compute_units(), bias);
   return 0;
 }
 
@@ -761,13 +784,14 @@ static int launch_prefill_dma(dim3 grid, hipStream_t stream, const bf16_t* q, lo
 // V page holds and every line is asked for twice: continuous batching at 32 kv heads with pages of 32 tokens 3,580 ->
 // 3,710 generated tokens/s (pages of 16: 3,830), with pages of 64 3,030 -> 3,290; 8 tokens of 8,000 keys at 8 kv heads
 // with pages of 64 1,520 -> 1,770 tokens/s. Pages of 8 and 16 tokens stay with the other dealing (measured above).
-template <int DPAD, bool FULL, bool ROW8, int WP = 1>
+template <int DPAD, bool FULL, bool ROW8, int WP = 1, bool BIAS = false>
 __global__ __launch_bounds__(256) void attn_decode_mfma_kernel(
     const bf16_t* __restrict__ q, long q_stride, const bf16_t* __restrict__ k_pages,
     const bf16_t* __restrict__ v_pages, const int* __restrict__ block_tables, int btw,
     const int* __restrict__ tok_idx, const int* __restrict__ seg, const int* __restrict__ pos, int nh, int nkv, int d,
     int ps, float scale_log2, float cap_raw, int window, int HB, int n_hb, int chunk, int n_splits, float* __restrict__ part_o,
-    float* __restrict__ part_ml, bf16_t* __restrict__ out, long out_stride, int heads_first) {
+    float* __restrict__ part_ml, bf16_t* __restrict__ out, long out_stride, int heads_first,
+    const float* __restrict__ bias) {
   constexpr int DS = DPAD / 32, DV = DPAD / 16;
   extern __shared__ float lds_f[];
   // (heads_first: the heads of a token are started together, the tokens in the order of tok_idx, so that a
@@ -791,6 +815,8 @@ __global__ __launch_bounds__(256) void attn_decode_mfma_kernel(
   const int hin = hb * HB + c;
   const bool valid = c < HB && hin < n_rep;
   const int head = kvh * n_rep + (valid ? hin : 0);
+  DistanceBias db;
+  if constexpr (BIAS) db.load(bias, nh, head, scale_log2);
   Frag8 qf[DS];
 #pragma unroll
   for (int s = 0; s < DS; ++s) {
@@ -871,6 +897,7 @@ __global__ __launch_bounds__(256) void attn_decode_mfma_kernel(
       for (int i = 0; i < 4; ++i) {
         const int key = ROW8 ? kbase + 8 * g + 4 * b + i : kbase + b * 16 + g * 4 + i;
         const bool ok = valid && key <= p && key >= lo && key < c1;
+        if constexpr (BIAS) a[i] -= db.off(p - key);
         const float x = ok ? a[i] * scale_log2 : -INFINITY;
         sv[b * 4 + i] = x;
         mx = fmaxf(mx, x);
@@ -1091,12 +1118,13 @@ extern "C" int lmsf_attention_tile_tokens(int nh, int nkv) {
 // LDS where the page size allows it (the default); 1: every wave fetches them itself; 2: as 0 with a window of 64
 // entries of the block table in LDS instead of 2,048, so that it moves at contexts that a test can afford.
 // ``softcap`` c > 0: a scaled score s becomes c tanh(s / c) before the softmax; 0: scores as they are.
-extern "C" int lmsf_paged_attention_prefill_mfma_capped(const void* q, long q_stride, void* out, long out_stride,
+// ``bias`` float32 [2, nh] or null: r1_h ln(1 + r2_h (i - j)) comes off the score of query i and key j (r2 >= 0).
+extern "C" int lmsf_paged_attention_prefill_mfma_biased(const void* q, long q_stride, void* out, long out_stride,
                                                         const void* k_pages, const void* v_pages, long num_pages,
                                                         const int* block_tables, int btw, const int* tiles,
                                                         int n_tiles, const int* seg, const int* pos, int nh, int nkv,
                                                         int d, int ps, float scale, int window, float softcap,
-                                                        int variant, hipStream_t stream) {
+                                                        const float* bias, int variant, hipStream_t stream) {
   LMSF_CHECK(softcap >= 0.f, "paged_attention_prefill: the soft cap must be >= 0, got %g", (double)softcap);
   const float cap_raw = softcap > 0.f ? softcap / scale : 0.f;
   if (int rc = check_common("paged_attention_prefill", q, out, k_pages, v_pages, block_tables, seg, pos, q_stride,
@@ -1118,8 +1146,10 @@ extern "C" int lmsf_paged_attention_prefill_mfma_capped(const void* q, long q_st
     int rc = 0;
 #define LDS_ARGS                                                                                                    \
   grid, stream, (const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)k_pages, (const bf16_t*)v_pages, \
-      block_tables, btw, tiles, seg, pos, nh, nkv, d, ps, scale_log2, cap_raw, window, HB, n_hb, bt_cap
-#define LAUNCH_LDS(DP) rc = wp3 ? launch_prefill_dma<DP, 3>(LDS_ARGS) : launch_prefill_dma<DP, 1>(LDS_ARGS)
+      block_tables, btw, tiles, seg, pos, nh, nkv, d, ps, scale_log2, cap_raw, window, HB, n_hb, bt_cap, bias
+#define LAUNCH_LDS(DP)                                                                                               \
+  rc = bias ? (wp3 ? launch_prefill_dma<DP, 3, true>(LDS_ARGS) : launch_prefill_dma<DP, 1, true>(LDS_ARGS))          \
+            : (wp3 ? launch_prefill_dma<DP, 3, false>(LDS_ARGS) : launch_prefill_dma<DP, 1, false>(LDS_ARGS))
     switch (dpad) {
       case 32: LAUNCH_LDS(32); break;
       case 64: LAUNCH_LDS(64); break;
@@ -1136,14 +1166,16 @@ extern "C" int lmsf_paged_attention_prefill_mfma_capped(const void* q, long q_st
     LMSF_LAUNCH_CHECK("paged_attention_prefill");
     return 0;
   }
-#define LAUNCH_W(DP, W)                                                                                             \
-  hipLaunchKernelGGL((attn_prefill_mfma_kernel<DP, PREFILL_NQB, W>), grid, block, 0, stream, (const bf16_t*)q,      \
+#define LAUNCH_W(DP, W, B)                                                                                          \
+  hipLaunchKernelGGL((attn_prefill_mfma_kernel<DP, PREFILL_NQB, W, B>), grid, block, 0, stream, (const bf16_t*)q,   \
                      q_stride, (bf16_t*)out, out_stride, (const bf16_t*)k_pages, (const bf16_t*)v_pages,            \
-                     block_tables, btw, tiles, seg, pos, nh, nkv, d, ps, scale_log2, cap_raw, window, HB, n_hb)
-#define LAUNCH(DP)                \
-  do {                            \
-    if (wp3) LAUNCH_W(DP, 3);     \
-    else LAUNCH_W(DP, 1);         \
+                     block_tables, btw, tiles, seg, pos, nh, nkv, d, ps, scale_log2, cap_raw, window, HB, n_hb, bias)
+#define LAUNCH(DP)                           \
+  do {                                       \
+    if (bias && wp3) LAUNCH_W(DP, 3, true);  \
+    else if (bias) LAUNCH_W(DP, 1, true);    \
+    else if (wp3) LAUNCH_W(DP, 3, false);    \
+    else LAUNCH_W(DP, 1, false);             \
   } while (0)
   switch (dpad) {
     case 32: LAUNCH(32); break;
@@ -1161,14 +1193,14 @@ extern "C" int lmsf_paged_attention_prefill_mfma_capped(const void* q, long q_st
   return 0;
 }
 
-template <int DPAD, bool FULL, bool ROW8, int WP>
+template <int DPAD, bool FULL, bool ROW8, int WP, bool BIAS>
 static int launch_decode(dim3 grid, hipStream_t stream, const bf16_t* q, long q_stride, const bf16_t* k_pages,
                          const bf16_t* v_pages, const int* block_tables, int btw, const int* tok_idx, const int* seg,
                          const int* pos, int nh, int nkv, int d, int ps, float scale_log2, float cap_raw, int window, int HB, int n_hb,
                          int chunk, int n_splits, float* part_o, float* part_ml, bf16_t* out, long out_stride,
-                         int heads_first) {
+                         int heads_first, const float* bias) {
   const size_t smem = (size_t)(4 * 16 * (DPAD + 4) + 128) * sizeof(float);
-  auto kernel = attn_decode_mfma_kernel<DPAD, FULL, ROW8, WP>;
+  auto kernel = attn_decode_mfma_kernel<DPAD, FULL, ROW8, WP, BIAS>;
   static bool configured = false;   // per instantiation
   if (!configured) {
     hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel),
@@ -1181,7 +1213,7 @@ static int launch_decode(dim3 grid, hipStream_t stream, const bf16_t* q, long q_
   }
   hipLaunchKernelGGL(kernel, grid, dim3(256), smem, stream, q, q_stride, k_pages, v_pages, block_tables, btw, tok_idx,
                      seg, pos, nh, nkv, d, ps, scale_log2, cap_raw, window, HB, n_hb, chunk, n_splits, part_o, part_ml, out,
-                     out_stride, heads_first);
+                     out_stride, heads_first, bias);
   return 0;
 }
 
@@ -1196,12 +1228,14 @@ extern "C" long lmsf_attention_decode_scratch_floats(int n, int nh, int d, int n
 // n_splits * chunk must cover the longest context. scratch: lmsf_attention_decode_scratch_floats floats
 // (not touched with n_splits == 1). seg null: token i is the only token of request i (row i of the block tables),
 // as in a step of single tokens.
-extern "C" int lmsf_paged_attention_decode_mfma_capped(const void* q, long q_stride, void* out, long out_stride,
+// ``bias``: as for the prefill kernels.
+extern "C" int lmsf_paged_attention_decode_mfma_biased(const void* q, long q_stride, void* out, long out_stride,
                                                        const void* k_pages, const void* v_pages, long num_pages,
                                                        const int* block_tables, int btw, const int* tok_idx, int n,
                                                        const int* seg, const int* pos, int nh, int nkv, int d, int ps,
-                                                       float scale, int window, float softcap, int chunk, int n_splits,
-                                                       float* scratch, int order, hipStream_t stream) {
+                                                       float scale, int window, float softcap, const float* bias,
+                                                       int chunk, int n_splits, float* scratch, int order,
+                                                       hipStream_t stream) {
   LMSF_CHECK(softcap >= 0.f && scale > 0.f, "paged_attention_decode: the soft cap must be >= 0 and the scale positive");
   const float cap_raw = softcap > 0.f ? softcap / scale : 0.f;
   if (int rc = check_common("paged_attention_decode", q, out, k_pages, v_pages, block_tables, seg ? seg : pos, pos,
@@ -1231,15 +1265,17 @@ extern "C" int lmsf_paged_attention_decode_mfma_capped(const void* q, long q_str
 #define DECODE_ARGS                                                                                                 \
   grid, stream, (const bf16_t*)q, q_stride, (const bf16_t*)k_pages, (const bf16_t*)v_pages, block_tables, btw, tok_idx, \
       seg, pos, nh, nkv, d, ps, scale_log2, cap_raw, window, HB, n_hb, chunk, n_splits, part_o, part_ml, (bf16_t*)out,       \
-      out_stride, heads_first
+      out_stride, heads_first, bias
   const bool row8 = ps % 32 == 0;   // (needs pages of a multiple of 8 tokens; chosen from 32 on)
-#define LAUNCH_W(DP, W)                                                                                       \
-  rc = d == DP ? (row8 ? launch_decode<DP, true, true, W>(DECODE_ARGS) : launch_decode<DP, true, false, W>(DECODE_ARGS)) \
-               : (row8 ? launch_decode<DP, false, true, W>(DECODE_ARGS) : launch_decode<DP, false, false, W>(DECODE_ARGS))
-#define LAUNCH(DP)                \
-  do {                            \
-    if (wp3) LAUNCH_W(DP, 3);     \
-    else LAUNCH_W(DP, 1);         \
+#define LAUNCH_W(DP, W, B)                                                                                       \
+  rc = d == DP ? (row8 ? launch_decode<DP, true, true, W, B>(DECODE_ARGS) : launch_decode<DP, true, false, W, B>(DECODE_ARGS)) \
+               : (row8 ? launch_decode<DP, false, true, W, B>(DECODE_ARGS) : launch_decode<DP, false, false, W, B>(DECODE_ARGS))
+#define LAUNCH(DP)                           \
+  do {                                       \
+    if (bias && wp3) LAUNCH_W(DP, 3, true);  \
+    else if (bias) LAUNCH_W(DP, 1, true);    \
+    else if (wp3) LAUNCH_W(DP, 3, false);    \
+    else LAUNCH_W(DP, 1, false);             \
   } while (0)
   switch (dpad) {
     case 32: LAUNCH(32); break;
@@ -1272,9 +1308,9 @@ extern "C" int lmsf_paged_attention_prefill_mfma(const void* q, long q_stride, v
                                                  const int* block_tables, int btw, const int* tiles, int n_tiles,
                                                  const int* seg, const int* pos, int nh, int nkv, int d, int ps,
                                                  float scale, int window, int variant, hipStream_t stream) {
-  return lmsf_paged_attention_prefill_mfma_capped(q, q_stride, out, out_stride, k_pages, v_pages, num_pages,
+  return lmsf_paged_attention_prefill_mfma_biased(q, q_stride, out, out_stride, k_pages, v_pages, num_pages,
                                                   block_tables, btw, tiles, n_tiles, seg, pos, nh, nkv, d, ps, scale,
-                                                  window, 0.f, variant, stream);
+                                                  window, 0.f, nullptr, variant, stream);
 }
 
 extern "C" int lmsf_paged_attention_decode_mfma(const void* q, long q_stride, void* out, long out_stride,
@@ -1283,7 +1319,7 @@ extern "C" int lmsf_paged_attention_decode_mfma(const void* q, long q_stride, vo
                                                 const int* seg, const int* pos, int nh, int nkv, int d, int ps,
                                                 float scale, int window, int chunk, int n_splits, float* scratch,
                                                 int order, hipStream_t stream) {
-  return lmsf_paged_attention_decode_mfma_capped(q, q_stride, out, out_stride, k_pages, v_pages, num_pages,
+  return lmsf_paged_attention_decode_mfma_biased(q, q_stride, out, out_stride, k_pages, v_pages, num_pages,
                                                  block_tables, btw, tok_idx, n, seg, pos, nh, nkv, d, ps, scale,
-                                                 window, 0.f, chunk, n_splits, scratch, order, stream);
+                                                 window, 0.f, nullptr, chunk, n_splits, scratch, order, stream);
 }

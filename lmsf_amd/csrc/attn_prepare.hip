@@ -15,6 +15,7 @@
 
 // Per token and head, in this order, each step optional:
 //   q, k <- x / sqrt(mean(x^2) + eps) over the head's dim entries                  (unit_norm)
+//   q, k <- times a weight over the head's dim entries, shared by the heads        (wq, wk != null)
 //   q, k <- rotation of the first ``rot`` entries, pairs (i, i + rot/2), by the position's angles (table != null)
 //   q    <- q (1 + temp_coef ln(floor((p + 1) / temp_every) + 1))                  (temp_every > 0)
 // q goes to q_out [N, H * D]; k to the token's slot of k_pages [pages, G, ps, D], v to v_pages [pages, G, D, ps]
@@ -24,8 +25,8 @@ __global__ __launch_bounds__(256) void attn_prepare_kernel(
     const T* __restrict__ q, long q_stride, const T* __restrict__ k, long k_stride, const T* __restrict__ v,
     long v_stride, const int* __restrict__ positions, const float* __restrict__ table, int rot, int max_pos,
     const int* __restrict__ slots, T* __restrict__ q_out, long qo_stride, T* __restrict__ k_pages,
-    T* __restrict__ v_pages, int H, int G, int dim, int vdim, int D, int ps, int unit_norm, float eps, float temp_coef,
-    int temp_every) {
+    T* __restrict__ v_pages, int H, int G, int dim, int vdim, int D, int ps, int unit_norm, float eps,
+    const float* __restrict__ wq, const float* __restrict__ wk, float temp_coef, int temp_every) {
   const int t = blockIdx.x;
   const int wave = threadIdx.x / LMSF_WAVE, lane = threadIdx.x % LMSF_WAVE;
   const int p = positions[t];
@@ -52,15 +53,18 @@ __global__ __launch_bounds__(256) void attn_prepare_kernel(
         inv = 1.f / sqrtf(ss / (float)dim + eps);
       }
       const float mul = is_q ? temp : 1.f;
+      const float* w = is_q ? wq : wk;
       T* dst = is_q ? q_out + (long)t * qo_stride + (long)head * D
                     : k_pages + (((long)page * G + head) * ps + off) * D;
       for (int e = lane; e < D; e += LMSF_WAVE) {
         float x = 0.f;
         if (e < dim) {
           x = to_f32<T>(src[e]) * inv;
+          if (w) x *= w[e];
           if (cs && e < rot) {
             const bool first = e < half;
-            const float other = to_f32<T>(src[first ? e + half : e - half]) * inv;
+            float other = to_f32<T>(src[first ? e + half : e - half]) * inv;
+            if (w) other *= w[first ? e + half : e - half];
             const float c = cs[first ? e : e - half], sn = cs[half + (first ? e : e - half)];
             float a, b;
             if (first) rope_rotate(x, other, c, sn, &a, &b); else rope_rotate(other, x, c, sn, &b, &a);
@@ -84,8 +88,8 @@ extern "C" int lmsf_attn_prepare(const void* q, long q_stride, const void* k, lo
                                  long v_stride, int dtype, const int* positions, const float* table, int rot,
                                  int max_pos, const int* slots, void* q_out, long qo_stride, void* k_pages,
                                  void* v_pages, long num_pages, int n_tokens, int H, int G, int dim, int vdim, int D,
-                                 int ps, int unit_norm, float eps, float temp_coef, int temp_every,
-                                 hipStream_t stream) {
+                                 int ps, int unit_norm, float eps, const float* wq, const float* wk, float temp_coef,
+                                 int temp_every, hipStream_t stream) {
   LMSF_CHECK(q && k && v && positions && q_out, "attn_prepare: null pointer");
   LMSF_CHECK(dtype == LMSF_F32 || dtype == LMSF_BF16, "attn_prepare: unknown dtype code %d", dtype);
   LMSF_CHECK(H > 0 && G > 0 && H % G == 0 && dim > 0 && vdim > 0 && D >= dim && D >= vdim,
@@ -104,12 +108,12 @@ extern "C" int lmsf_attn_prepare(const void* q, long q_stride, const void* k, lo
     hipLaunchKernelGGL((attn_prepare_kernel<float>), grid, dim3(256), 0, stream, (const float*)q, q_stride,
                        (const float*)k, k_stride, (const float*)v, v_stride, positions, table, rot, max_pos, slots,
                        (float*)q_out, qo_stride, (float*)k_pages, (float*)v_pages, H, G, dim, vdim, D, ps, unit_norm, eps,
-                       temp_coef, temp_every);
+                       wq, wk, temp_coef, temp_every);
   else
     hipLaunchKernelGGL((attn_prepare_kernel<bf16_t>), grid, dim3(256), 0, stream, (const bf16_t*)q, q_stride,
                        (const bf16_t*)k, k_stride, (const bf16_t*)v, v_stride, positions, table, rot, max_pos, slots,
                        (bf16_t*)q_out, qo_stride, (bf16_t*)k_pages, (bf16_t*)v_pages, H, G, dim, vdim, D, ps, unit_norm,
-                       eps, temp_coef, temp_every);
+                       eps, wq, wk, temp_coef, temp_every);
   LMSF_LAUNCH_CHECK("attn_prepare");
   return 0;
 }

@@ -1,11 +1,11 @@
-// The gated delta rule with one decay per head and key channel, a matrix memory S [dim, vdim] per head and request:
+// The gated delta rule with a decay per head and key channel or per head, a matrix memory S [dim, vdim] per head and request:
 //
 //   S <- diag(g_t) S;   u = beta_t (v_t - S^T k_t);   S <- S + k_t u^T;   o_t = S^T q_t
 //
 // (the read-out sees the token's own write). What enters the recurrence is made here, in float32, from the
 // projections' results: q and k are made unit vectors per head, x / sqrt(sum x^2 + unit_eps), q times q_scale;
 // beta = sigmoid(b); g = exp(-exp(A_log_h) softplus(a + dt_bias)), one factor per head and key channel, acting on the
-// rows of S. H value heads and G query/key heads (head h reads q/k head h / (H / G)). S lives in the request's state
+// rows of S; or one factor per head (``a`` [N, H], dt_bias [H]: the same product with equal factors). H value heads and G query/key heads (head h reads q/k head h / (H / G)). S lives in the request's state
 // slot in float32 and is read once and written once a step.
 //
 // The columns of S are independent of one another: column j only ever needs k, q, g, beta and v_j. Token by token a
@@ -91,7 +91,7 @@ __global__ __launch_bounds__(256) void gated_delta_prepare_kernel(
     const float* __restrict__ dt_bias, const float* __restrict__ a_log, const float* __restrict__ b, long b_stride,
     const int* __restrict__ seg_of, const int* __restrict__ seg_starts, float* __restrict__ prep,
     float* __restrict__ vals, int n_tokens, long chunk_rows, long val_rows, int H, int G, int dim, int vdim, int RPL,
-    float q_scale, float unit_eps) {
+    float q_scale, float unit_eps, int a_head, int a_entry) {
   const long w = (long)blockIdx.x * (256 / LMSF_WAVE) + threadIdx.x / LMSF_WAVE;
   const int lane = threadIdx.x % LMSF_WAVE;
   if (w >= (long)n_tokens * H) return;
@@ -132,7 +132,8 @@ __global__ __launch_bounds__(256) void gated_delta_prepare_kernel(
       if (m < nt && i < dim) {
         k[m] = to_f32<T>(qkv[(long)(t + m) * stride + k_at + gh * dim + i]) * ik[m];
         q[m] = to_f32<T>(qkv[(long)(t + m) * stride + q_at + gh * dim + i]) * iq[m];
-        lg[m] = -rate * softplus_f32(a[(long)(t + m) * a_stride + h * dim + i] + dt_bias[h * dim + i]);
+        const int at = h * a_head + i * a_entry;       // (dim, 1): a factor per key entry; (1, 0): one a head
+        lg[m] = -rate * softplus_f32(a[(long)(t + m) * a_stride + at] + dt_bias[at]);
       }
     }
     // every exponent is a sum of the logarithms it spans, added up directly (not a difference of running sums)
@@ -381,7 +382,8 @@ static int launch_delta_recurrence(dim3 grid, hipStream_t stream, const float* p
 }
 
 // qkv: the (convolved, activated) q [N, G dim], k [N, G dim], v [N, H vdim] as columns q_at, k_at, v_at of one buffer
-// of ``dtype`` with row stride ``stride``; a: float32 [N, H dim] before bias and softplus; dt_bias float32 [H dim];
+// of ``dtype`` with row stride ``stride``; a: float32 [N, H dim] before bias and softplus; dt_bias float32 [H dim]
+// (``per_head``: [N, H] and [H], one decay a head);
 // a_log float32 [H]; b: float32 [N, >= H] before the sigmoid; state float32 [slots, >= lmsf_gated_delta_state_floats];
 // seg_of [N], seg_starts [S + 1], slots [S]: the step's segments; longest: the most tokens a segment holds, if the caller
 // knows (0: not known); scratch: lmsf_gated_delta_scratch_floats floats,
@@ -391,7 +393,7 @@ extern "C" int lmsf_gated_delta(const void* qkv, int dtype, long stride, int q_a
                                 long b_stride, float* state, long state_stride, const int* seg_of,
                                 const int* seg_starts, const int* slots, float* scratch, float* out, long out_stride,
                                 int n_tokens, int n_segments, int longest, int H, int G, int dim, int vdim,
-                                float q_scale, float unit_eps, hipStream_t stream) {
+                                float q_scale, float unit_eps, int per_head, hipStream_t stream) {
   LMSF_CHECK(qkv && a && dt_bias && a_log && b && state && seg_of && seg_starts && slots && out && scratch,
              "gated_delta: null pointer");
   LMSF_CHECK(dtype == LMSF_F32 || dtype == LMSF_BF16, "gated_delta: unknown dtype code %d", dtype);
@@ -399,7 +401,7 @@ extern "C" int lmsf_gated_delta(const void* qkv, int dtype, long stride, int q_a
              "gated_delta: heads %d over %d key heads, keys of %d (at most 256) and values of %d entries", H, G, dim, vdim);
   const int n_cb = (vdim + DELTA_COLS - 1) / DELTA_COLS;
   LMSF_CHECK(H <= 65535 && n_cb <= 65535, "gated_delta: too many heads or columns");
-  LMSF_CHECK(a_stride >= (long)H * dim && b_stride >= H && out_stride >= (long)H * vdim &&
+  LMSF_CHECK(a_stride >= (long)H * (per_head ? 1 : dim) && b_stride >= H && out_stride >= (long)H * vdim &&
                  state_stride >= lmsf_gated_delta_state_floats(H, dim, vdim) && q_at >= 0 && k_at >= 0 && v_at >= 0,
              "gated_delta: strides too small");
   LMSF_CHECK(lmsf_aligned16(scratch), "gated_delta: the scratch must be 16-byte aligned");
@@ -412,7 +414,8 @@ extern "C" int lmsf_gated_delta(const void* qkv, int dtype, long stride, int q_a
 #define DELTA_PREP(T)                                                                                               \
   hipLaunchKernelGGL((gated_delta_prepare_kernel<T>), g1, dim3(256), 0, stream, (const T*)qkv, stride, q_at, k_at,   \
                      v_at, a, a_stride, dt_bias, a_log, b, b_stride, seg_of, seg_starts, prep, vals, n_tokens,      \
-                     chunk_rows, val_rows, H, G, dim, vdim, RPL, q_scale, unit_eps)
+                     chunk_rows, val_rows, H, G, dim, vdim, RPL, q_scale, unit_eps, per_head ? 1 : dim,              \
+                     per_head ? 0 : 1)
   if (dtype == LMSF_F32) DELTA_PREP(float);
   else DELTA_PREP(bf16_t);
 #undef DELTA_PREP

@@ -26,6 +26,30 @@ int lmsf_paged_attention_decode_mfma(const void* q, long q_stride, void* out, lo
     const int* pos, int nh, int nkv, int d, int ps, float scale, int window, int chunk, int n_splits, float* scratch,
     int order, hipStream_t stream);
 
+int lmsf_paged_attention_prefill_mfma_biased(const void* q, long q_stride, void* out, long out_stride, const void*
+    k_pages, const void* v_pages, long num_pages, const int* block_tables, int btw, const int* tiles, int n_tiles,
+    const int* seg, const int* pos, int nh, int nkv, int d, int ps, float scale, int window, float softcap, const
+    float* bias, int variant, hipStream_t stream);
+int lmsf_paged_attention_decode_mfma_biased(const void* q, long q_stride, void* out, long out_stride, const void*
+    k_pages, const void* v_pages, long num_pages, const int* block_tables, int btw, const int* tok_idx, int n, const
+    int* seg, const int* pos, int nh, int nkv, int d, int ps, float scale, int window, float softcap, const float*
+    bias, int chunk, int n_splits, float* scratch, int order, hipStream_t stream);
+
+// token_extras.hip
+int lmsf_position_embedding(const int* ids, const int* pos, const void* table, const void* places, int dtype, float
+    scale, float* out, void* cast, int n_tokens, int V, int P, int W, int* bad_flag, hipStream_t stream);
+
+// linear_recurrence.hip
+long lmsf_linear_recurrence_entry_floats(int C);
+int lmsf_linear_recurrence_gates(const void* u, int dtype, long u_stride, const void* Wr, const float* br, const void*
+    Wi, const float* bi, const float* rate, float* a, float* b, int n_tokens, int C, int c, hipStream_t stream);
+int lmsf_linear_recurrence_step(const void* u, int dtype, long u_stride, const void* Wr, const float* br, const void*
+    Wi, const float* bi, const float* rate, const void* y, long y_stride, float* state, long state_stride, const int*
+    seg_of, const int* slots, void* out, long out_stride, int n_tokens, int C, int c, hipStream_t stream);
+int lmsf_linear_recurrence_scan(const float* a, const float* b, const void* y, int dtype, long y_stride, float* state,
+    long state_stride, const int* seg_starts, const int* slots, void* out, long out_stride, int n_tokens, int
+    n_segments, int C, int chunk, int max_chunks, const int* scratch_base, float* scratch, hipStream_t stream);
+
 // group_norm.hip
 int lmsf_group_norm(const void* branch, int branch_dtype, long branch_stride, const float* wb, float* residual,
     float* hist, long hist_stride, int hist_index, const float* mix, const float* wn, void* out, int out_dtype,
@@ -57,7 +81,8 @@ int lmsf_table_moe_grouped(int dtype, int n_tokens, int top, int E, int F, int W
 int lmsf_attn_prepare(const void* q, long q_stride, const void* k, long k_stride, const void* v, long v_stride, int
     dtype, const int* positions, const float* table, int rot, int max_pos, const int* slots, void* q_out, long
     qo_stride, void* k_pages, void* v_pages, long num_pages, int n_tokens, int H, int G, int dim, int vdim, int D, int
-    ps, int unit_norm, float eps, float temp_coef, int temp_every, hipStream_t stream);
+    ps, int unit_norm, float eps, const float* wq, const float* wk, float temp_coef, int temp_every, hipStream_t
+    stream);
 int lmsf_head_gate(const void* x, int dtype, long x_stride, int x_head, const void* gate, long gate_stride, void* out,
     long out_stride, int n_tokens, int H, int dv, hipStream_t stream);
 int lmsf_rms_pair(const void* a, long a_stride, const void* b, long b_stride, int dtype, const float* wa, const float*

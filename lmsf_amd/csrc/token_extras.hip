@@ -4,6 +4,7 @@
 //   mod buckets, the last row (number ``buckets``) for a request's first token. The previous id of a segment's
 //   first token is the last id of the request's step before, kept per state slot in ``prev_state`` (a second tiny
 //   kernel brings it up to date, so that nothing is written that another workgroup of the first still reads).
+// - An embedding with a learned vector per position: x = table[id] * scale + places[position].
 // - Two float32 rows laid side by side as one row of the run's type (the operand of a product over both).
 // - act(z) * table[id, at .. at + dim): a gate times a slice of a per-token table, act the tanh form of GELU.
 // - relu(z)^2, elementwise.
@@ -68,6 +69,46 @@ extern "C" int lmsf_hashed_pair_embedding(const int* ids, const int* pos, const 
   hipLaunchKernelGGL(last_token_kernel, dim3((n_segments + 63) / 64), dim3(64), 0, stream, ids, seg_starts,
                      state_slots, prev_state, n_segments);
   LMSF_LAUNCH_CHECK("hashed_pair_embedding");
+  return 0;
+}
+
+// ---------------------------------------------------------------- a learned vector per position
+
+template <typename T>
+__global__ __launch_bounds__(256) void position_embedding_kernel(const int* __restrict__ ids, const int* __restrict__ pos,
+                                                                 const T* __restrict__ table, const T* __restrict__ places,
+                                                                 float scale, float* __restrict__ out, T* __restrict__ cast,
+                                                                 int V, int P, int W, int* __restrict__ bad_flag) {
+  const long t = blockIdx.x;
+  const int id = ids[t];
+  const bool ok = id >= 0 && id < V;
+  if (!ok && threadIdx.x == 0 && bad_flag) atomicOr(bad_flag, 1);
+  const T* a = table + (long)(ok ? id : 0) * W;
+  const T* b = places + (long)min(max(pos[t], 0), P - 1) * W;
+  for (int i = threadIdx.x; i < W; i += 256) {
+    const float x = ok ? to_f32<T>(a[i]) * scale + to_f32<T>(b[i]) : 0.f;
+    out[t * W + i] = x;
+    if (cast) cast[t * W + i] = from_f32<T>(x);
+  }
+}
+
+// out float32 [n_tokens, W] = table[id] * scale + places[position]; cast (may be null): the same rounded to ``dtype``.
+// table [V, W], places [P, W] of ``dtype``. An id outside [0, V) gives a row of zeros and raises the flag; positions are
+// below P (the engine's longest request is no longer than that).
+extern "C" int lmsf_position_embedding(const int* ids, const int* pos, const void* table, const void* places, int dtype,
+                                       float scale, float* out, void* cast, int n_tokens, int V, int P, int W,
+                                       int* bad_flag, hipStream_t stream) {
+  LMSF_CHECK(ids && pos && table && places && out, "position_embedding: null pointer");
+  LMSF_CHECK(dtype == LMSF_F32 || dtype == LMSF_BF16, "position_embedding: unknown dtype code %d", dtype);
+  LMSF_CHECK(V > 0 && P > 0 && W > 0, "position_embedding: bad sizes");
+  if (n_tokens <= 0) return 0;
+  if (dtype == LMSF_F32)
+    hipLaunchKernelGGL((position_embedding_kernel<float>), dim3(n_tokens), dim3(256), 0, stream, ids, pos,
+                       (const float*)table, (const float*)places, scale, out, (float*)cast, V, P, W, bad_flag);
+  else
+    hipLaunchKernelGGL((position_embedding_kernel<bf16_t>), dim3(n_tokens), dim3(256), 0, stream, ids, pos,
+                       (const bf16_t*)table, (const bf16_t*)places, scale, out, (bf16_t*)cast, V, P, W, bad_flag);
+  LMSF_LAUNCH_CHECK("position_embedding");
   return 0;
 }
 

@@ -31,7 +31,6 @@ l<i>.side.{gate, proj, norm}, l<i>.mix.{q, k, v, q.norm, k.norm, g, o} or l<i>.m
 A_log, a1, a2, dt_bias, g1, g2, norm, o}, l<i>.mlp.{up, down} or l<i>.mlp.{router, e<k>.{up, down}}.
 """
 import json
-import os
 from dataclasses import dataclass
 from typing import Any, Dict, List, Optional, Tuple
 
@@ -55,21 +54,6 @@ def _need(d: Any, key: str, where: str, kind=(int,), positive: bool = True, at_l
     elif positive and not v > 0:
         raise ConfigError("config.json: %s.%s must be > 0, is %r" % (where, key, v))
     return v
-
-
-def _header_shapes(folder: str) -> Dict[str, Tuple[int, ...]]:
-    """Names and shapes of a folder's checkpoint tensors, from the files' headers alone."""
-    from ..weights.loader import list_weight_files
-    from ..weights.safetensors_io import SafetensorsFile
-    shapes: Dict[str, Tuple[int, ...]] = {}
-    for path in list_weight_files(folder):
-        f = SafetensorsFile(path)
-        try:
-            for name, e in f.entries.items():
-                shapes[name] = tuple(e.shape)
-        finally:
-            f.close()
-    return shapes
 
 
 @dataclass(frozen=True)
@@ -103,8 +87,9 @@ class MurulornConfig(ArchConfig):
                    and not ("decay_rank" in layer["mixer"] and "gate_rank" in layer["mixer"])]
         if not lacking:
             return d
+        from ..weights.loader import header_shapes
         try:
-            shapes = _header_shapes(folder)
+            shapes = header_shapes(folder)
         except Exception:  # noqa: BLE001 - no checkpoint (random weights): the defaults stand
             return d
         d = json.loads(json.dumps(d))

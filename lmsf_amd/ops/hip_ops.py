@@ -141,11 +141,14 @@ class HipOps:
             raise ValueError("embedding table must be contiguous [V, H]")
         n, (V, H) = ids.numel(), table.shape
         out = torch.empty((n, H), dtype=torch.float32, device=table.device)
-        if self._bad_flag is None or self._bad_flag.device != table.device:
-            self._bad_flag = torch.zeros(1, dtype=torch.int32, device=table.device)
         self._check(self.lib.lmsf_embedding(_ptr(ids), _ptr(table), _code(table.dtype), _ptr(out), n, H, V,
-                                            float(scale), _ptr(self._bad_flag), self._stream()))
+                                            float(scale), _ptr(self._bad_token_flag(table.device)), self._stream()))
         return out
+
+    def _bad_token_flag(self, device: torch.device) -> torch.Tensor:
+        if self._bad_flag is None or self._bad_flag.device != device:
+            self._bad_flag = torch.zeros(1, dtype=torch.int32, device=device)
+        return self._bad_flag
 
     def patch_tokens(self, ids: torch.Tensor, src: torch.Tensor, prev: torch.Tensor) -> None:
         """ids[i] = prev[src[i]] where src[i] >= 0 (all int32, on the device): a step launched ahead takes the
@@ -436,13 +439,15 @@ class HipOps:
     def paged_attention(self, q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,
                         block_tables: torch.Tensor, seg: torch.Tensor, pos: torch.Tensor, nh: int, nkv: int, d: int,
                         scale: float, window: int = 0, batch=None, kernel: Optional[str] = None,
-                        chunk: int = 0, weights_f32: bool = False, softcap: float = 0.0) -> torch.Tensor:
+                        chunk: int = 0, weights_f32: bool = False, softcap: float = 0.0,
+                        distance_bias: Optional[torch.Tensor] = None) -> torch.Tensor:
         """Attention of every query token over the cached keys of its request: those at positions up to its own,
         within the last ``window`` positions if a window is given, or within its own chunk of ``chunk`` positions
         (chunks counted from position 0 of the request) if a chunk size is given. ``weights_f32``: in a bfloat16 run
         the softmax weights enter the product with the values in full float32 (as three bfloat16 parts on the
         matrix cores) instead of rounded to bfloat16; scores, maxima and sums are float32 either way. ``softcap``
-        c > 0: a scaled score s enters the softmax as c tanh(s / c).
+        c > 0: a scaled score s enters the softmax as c tanh(s / c). ``distance_bias`` (float32 [2, nh], rows r1 and
+        r2 >= 0): r1_h ln(1 + r2_h (i - j)) comes off the score of query i and key j, after the cap.
 
         ``q`` is [N, >= nh*d] with unit column stride (it may be the fused QKV buffer, of which the
         first nh*d columns are read). ``k_pages`` [pages, nkv, page_size, d], ``v_pages``
@@ -466,6 +471,10 @@ class HipOps:
         self._i32(block_tables, "block_tables")
         self._i32(seg, "seg", N)
         self._i32(pos, "pos", N)
+        if distance_bias is not None:
+            self._dev(distance_bias)
+            self._f32_vec(distance_bias, 2 * nh, "paged_attention: distance_bias")
+        bias = _ptr(distance_bias)
         out = torch.empty((N, nh * d), dtype=q.dtype, device=q.device)
         if N == 0:
             return out
@@ -479,18 +488,18 @@ class HipOps:
             raise ValueError("the matrix-core attention kernels need bfloat16, a head size that is a multiple of 16 "
                              "up to 256, a page size that is a multiple of 4, 16-byte aligned query rows and a positive scale")
         if kernel == "generic" or not fast_ok:
-            self._check(self.lib.lmsf_paged_attention_generic_capped(
+            self._check(self.lib.lmsf_paged_attention_generic_biased(
                 _ptr(q), q.stride(0), _ptr(out), out.stride(0), _ptr(k_pages), _ptr(v_pages), num_pages,
                 _ptr(block_tables), block_tables.shape[1], _ptr(seg), _ptr(pos), N, nh, nkv, d, ps, float(scale),
-                int(window or 0), float(softcap), _code(q.dtype), self._stream()))
+                int(window or 0), float(softcap), bias, _code(q.dtype), self._stream()))
             return out
         plan = self._attention_plan(batch, seg, pos, nh, nkv)
         exact = self.ATTENTION_WEIGHTS_F32 if weights_f32 else 0
         common = (_ptr(k_pages), _ptr(v_pages), num_pages, _ptr(block_tables), block_tables.shape[1])
         if plan.tiles is not None:
-            self._check(self.lib.lmsf_paged_attention_prefill_mfma_capped(
+            self._check(self.lib.lmsf_paged_attention_prefill_mfma_biased(
                 _ptr(q), q.stride(0), _ptr(out), out.stride(0), *common, _ptr(plan.tiles), plan.n_tiles,
-                _ptr(seg), _ptr(pos), nh, nkv, d, ps, float(scale), int(window or 0), float(softcap),
+                _ptr(seg), _ptr(pos), nh, nkv, d, ps, float(scale), int(window or 0), float(softcap), bias,
                 self.prefill_attention_variant + exact, self._stream()))
         if plan.n_single:
             c_chunk, c_splits = ctypes.c_int(0), ctypes.c_int(0)
@@ -499,10 +508,10 @@ class HipOps:
             chunk, n_splits = c_chunk.value, c_splits.value
             floats = self.lib.lmsf_attention_decode_scratch_floats(plan.n_single, nh, d, n_splits)
             scratch = torch.empty(floats if n_splits > 1 else 1, dtype=torch.float32, device=q.device)
-            self._check(self.lib.lmsf_paged_attention_decode_mfma_capped(
+            self._check(self.lib.lmsf_paged_attention_decode_mfma_biased(
                 _ptr(q), q.stride(0), _ptr(out), out.stride(0), *common, _ptr(plan.single_tokens), plan.n_single,
                 None if plan.token_is_request else _ptr(seg), _ptr(pos), nh, nkv, d, ps, float(scale),
-                int(window or 0), float(softcap), chunk, n_splits, _ptr(scratch), self.decode_attention_order + exact,
+                int(window or 0), float(softcap), bias, chunk, n_splits, _ptr(scratch), self.decode_attention_order + exact,
                 self._stream()))
         return out
 
@@ -847,6 +856,24 @@ class HipOps:
             int(mul_cur), self._stream()))
         return (out, kept) if keep else out
 
+    def position_embedding(self, ids: torch.Tensor, positions: torch.Tensor, table: torch.Tensor, places: torch.Tensor,
+                           scale: float = 1.0):
+        """float32 [N, W] = table[id] * scale + places[position], and the same rounded to the tables' dtype."""
+        self._dev(ids, positions, table, places)
+        if table.dim() != 2 or places.dim() != 2 or places.shape[1] != table.shape[1] or table.dtype != places.dtype \
+                or not table.is_contiguous() or not places.is_contiguous():
+            raise ValueError("position_embedding: table [V, W] and places [P, W] of one dtype are needed")
+        N = ids.numel()
+        self._i32(ids, "token_ids", N)
+        self._i32(positions, "positions", N)
+        V, W = table.shape
+        out = torch.empty((N, W), dtype=torch.float32, device=table.device)
+        cast = torch.empty((N, W), dtype=table.dtype, device=table.device)
+        self._check(self.lib.lmsf_position_embedding(
+            _ptr(ids), _ptr(positions), _ptr(table), _ptr(places), _code(table.dtype), float(scale), _ptr(out), _ptr(cast),
+            N, V, places.shape[0], W, _ptr(self._bad_token_flag(table.device)), self._stream()))
+        return out, cast
+
     def concat_rows(self, a: torch.Tensor, b: torch.Tensor, out_dtype: torch.dtype) -> torch.Tensor:
         """[a | b] row by row in ``out_dtype``; a, b contiguous float32 [N, Wa], [N, Wb]."""
         self._dev(a, b)
@@ -966,22 +993,24 @@ class HipOps:
 
     def gated_delta(self, qkv: torch.Tensor, q_at: int, k_at: int, v_at: int, a: torch.Tensor, dt_bias: torch.Tensor,
                     a_log: torch.Tensor, b: torch.Tensor, state: torch.Tensor, batch, heads: int, kv_heads: int,
-                    dim: int, vdim: int, q_scale: float, unit_eps: float = 1e-6) -> torch.Tensor:
+                    dim: int, vdim: int, q_scale: float, unit_eps: float = 1e-6, per_head: bool = False) -> torch.Tensor:
         """The gated delta rule over each request's tokens, the memory S [heads, dim, vdim] carried in ``state``
         (float32 [slots, >= gated_delta_state_floats], laid out [heads, ceil(vdim / 4), dim, 4]): S <- diag(g) S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q, with
         q, k the unit vectors of columns q_at, k_at of ``qkv`` (kv_heads heads of dim; q times q_scale), v its columns
         from v_at (heads of vdim), beta = sigmoid(b [N, >= heads]) and g = exp(-exp(a_log [heads]) softplus(a + dt_bias))
-        (``a`` float32 [N, heads * dim]). Returns the heads' o as float32 [N, heads * vdim]."""
+        (``a`` float32 [N, heads * dim]; ``per_head``: ``a`` [N, heads] and dt_bias [heads], one decay a head). Returns
+        the heads' o as float32 [N, heads * vdim]."""
+        decays = heads if per_head else heads * dim
         self._dev(qkv, a, dt_bias, a_log, b)
         N = qkv.shape[0]
         need = max(q_at + kv_heads * dim, k_at + kv_heads * dim, v_at + heads * vdim)
         if qkv.dim() != 2 or qkv.stride(1) != 1 or qkv.shape[1] < need:
             raise ValueError("gated_delta: qkv must be [N, >= %d] with unit column stride" % need)
-        if a.dtype != torch.float32 or a.dim() != 2 or a.shape[0] != N or a.shape[1] < heads * dim or a.stride(1) != 1:
-            raise ValueError("gated_delta: a must be float32 [%d, >= %d]" % (N, heads * dim))
+        if a.dtype != torch.float32 or a.dim() != 2 or a.shape[0] != N or a.shape[1] < decays or a.stride(1) != 1:
+            raise ValueError("gated_delta: a must be float32 [%d, >= %d]" % (N, decays))
         if b.dtype != torch.float32 or b.dim() != 2 or b.shape[0] != N or b.shape[1] < heads or b.stride(1) != 1:
             raise ValueError("gated_delta: b must be float32 [%d, >= %d]" % (N, heads))
-        self._f32_vec(dt_bias, heads * dim, "gated_delta: dt_bias")
+        self._f32_vec(dt_bias, decays, "gated_delta: dt_bias")
         self._f32_vec(a_log, heads, "gated_delta: a_log")
         if heads % kv_heads or dim > 256:
             raise ValueError("gated_delta: %d heads over %d key heads, keys of %d entries (at most 256)" % (heads, kv_heads, dim))
@@ -995,7 +1024,7 @@ class HipOps:
             _ptr(dt_bias), _ptr(a_log), _ptr(b), b.stride(0), _ptr(state), state.stride(0), _ptr(seg_of), _ptr(seg_starts),
             _ptr(slots), _ptr(scratch), _ptr(out), out.stride(0), N, S,
             1 if (getattr(batch, "all_single", False) and S == N) else 0, int(heads), int(kv_heads), int(dim), int(vdim), float(q_scale),
-            float(unit_eps), self._stream()))
+            float(unit_eps), 1 if per_head else 0, self._stream()))
         return out
 
     def head_rms_gate(self, raw: torch.Tensor, heads: int, vdim: int, eps: float, weight: Optional[torch.Tensor],
@@ -1264,6 +1293,51 @@ class HipOps:
             aux[key] = plan
         return plan
 
+    linear_recurrence_chunk_tokens = 32    # tokens of a chunk of the linear recurrence's chunked form
+
+    def linear_recurrence(self, u: torch.Tensor, wr: torch.Tensor, br: torch.Tensor, wi: torch.Tensor, bi: torch.Tensor,
+                          rate: torch.Tensor, y: torch.Tensor, state: torch.Tensor, batch) -> torch.Tensor:
+        """The real-gated linear recurrence over each request's tokens, a number per channel carried in ``state``
+        (float32 [slots, >= C]): with r = sigmoid(Wr u + br), i = sigmoid(Wi u + bi) block by block, log a = -rate r and
+        S <- a S + sqrt(1 - a^2) i u, returns S * gelu_tanh(y), [N, C] in u's dtype. ``u`` [N, C], ``y`` [N, >= C];
+        ``wr``, ``wi`` [blocks, C / blocks, C / blocks] of u's dtype; ``br``, ``bi``, ``rate`` float32 [C]."""
+        self._dev(u, wr, br, wi, bi, rate, y)
+        N, C = u.shape
+        if wr.dim() != 3 or wr.shape[1] != wr.shape[2] or wr.shape[0] * wr.shape[1] != C or wi.shape != wr.shape \
+                or wr.dtype != u.dtype or wi.dtype != u.dtype or not wr.is_contiguous() or not wi.is_contiguous():
+            raise ValueError("linear_recurrence: the gates' matrices must be contiguous [blocks, C / blocks, C / blocks] of "
+                             "u's dtype")
+        if u.stride(1) != 1 or y.dim() != 2 or y.shape[0] != N or y.shape[1] < C or y.stride(1) != 1 or y.dtype != u.dtype:
+            raise ValueError("linear_recurrence: u and y must be [%d, %d] of one dtype with unit column stride" % (N, C))
+        for t, name in ((br, "br"), (bi, "bi"), (rate, "rate")):
+            self._f32_vec(t, C, "linear_recurrence: " + name)
+        self._state_view(state, C, "linear_recurrence")
+        seg_of, seg_starts, slots, S = self._segments(batch, N)
+        c = wr.shape[1]
+        out = torch.empty((N, C), dtype=u.dtype, device=u.device)
+        if getattr(batch, "all_single", False) and S == N:
+            self._check(self.lib.lmsf_linear_recurrence_step(
+                _ptr(u), _code(u.dtype), u.stride(0), _ptr(wr), _ptr(br), _ptr(wi), _ptr(bi), _ptr(rate), _ptr(y),
+                y.stride(0), _ptr(state), state.stride(0), _ptr(seg_of), _ptr(slots), _ptr(out), out.stride(0), N, C, c,
+                self._stream()))
+            return out
+        a = torch.empty((N, C), dtype=torch.float32, device=u.device)
+        b = torch.empty((N, C), dtype=torch.float32, device=u.device)
+        self._check(self.lib.lmsf_linear_recurrence_gates(
+            _ptr(u), _code(u.dtype), u.stride(0), _ptr(wr), _ptr(br), _ptr(wi), _ptr(bi), _ptr(rate), _ptr(a), _ptr(b), N, C,
+            c, self._stream()))
+        chunk, most, bases, scratch = self.linear_recurrence_chunk_tokens, 1, None, None
+        plan = self._chunk_plan(batch, chunk)
+        if plan is not None:
+            bases, entries, most = plan
+            scratch = torch.empty(entries * self.lib.lmsf_linear_recurrence_entry_floats(C), dtype=torch.float32,
+                                  device=u.device)
+        self._check(self.lib.lmsf_linear_recurrence_scan(
+            _ptr(a), _ptr(b), _ptr(y), _code(u.dtype), y.stride(0), _ptr(state), state.stride(0), _ptr(seg_starts),
+            _ptr(slots), _ptr(out), out.stride(0), N, S, C, int(chunk), int(most), _ptr(bases), _ptr(scratch),
+            self._stream()))
+        return out
+
     def mlstm_state_floats(self, heads: int, dim: int, vdim: int) -> int:
         return int(self.lib.lmsf_mlstm_state_floats(heads, dim, vdim))
 
@@ -1330,9 +1404,11 @@ class HipOps:
     def attn_prepare(self, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, heads: int, kv_heads: int, dim: int,
                      vdim: int, padded: int, positions: torch.Tensor, slots: Optional[torch.Tensor],
                      k_pages: Optional[torch.Tensor], v_pages: Optional[torch.Tensor], table: Optional[torch.Tensor] = None,
-                     unit_norm_eps: Optional[float] = None, temp_coef: float = 0.0, temp_every: int = 0) -> torch.Tensor:
+                     unit_norm_eps: Optional[float] = None, temp_coef: float = 0.0, temp_every: int = 0,
+                     q_weight: Optional[torch.Tensor] = None, k_weight: Optional[torch.Tensor] = None) -> torch.Tensor:
         """Readies projected queries, keys and values for ``paged_attention`` at head size ``padded``: q and k are
-        (each step optional) divided by their root mean square over the head (``unit_norm_eps``), rotated by the
+        (each step optional) divided by their root mean square over the head (``unit_norm_eps``), multiplied by a weight
+        over the head's entries (``q_weight``, ``k_weight`` float32 [dim]), rotated by the
         position over the first table.shape[1] entries in pairs (i, i + rot/2) (``table`` float32 [max_pos, rot] =
         [cos | sin]), q is multiplied by 1 + temp_coef ln(floor((p + 1) / temp_every) + 1); k and v go to the
         tokens' slots of the pages, everything padded with zeros to ``padded`` entries a head. q [N, heads * dim],
@@ -1343,6 +1419,10 @@ class HipOps:
             if t.dim() != 2 or t.shape[0] != N or t.shape[1] < w or t.stride(1) != 1 or t.dtype != q.dtype:
                 raise ValueError("attn_prepare: %s must be [%d, >= %d] of q's dtype with unit column stride" % (name, N, w))
         self._i32(positions, "positions", N)
+        for w, name in ((q_weight, "q_weight"), (k_weight, "k_weight")):
+            if w is not None:
+                self._dev(w)
+                self._f32_vec(w, dim, "attn_prepare: " + name)
         rot = max_pos = 0
         if table is not None:
             if table.dtype != torch.float32 or table.dim() != 2 or not table.is_contiguous() or table.shape[1] > dim \
@@ -1366,7 +1446,8 @@ class HipOps:
             _ptr(q), q.stride(0), _ptr(k), k.stride(0), _ptr(v), v.stride(0), _code(q.dtype), _ptr(positions), _ptr(table),
             rot, max_pos, _ptr(slots), _ptr(out), out.stride(0), _ptr(k_pages), _ptr(v_pages), num_pages, N, int(heads),
             int(kv_heads), int(dim), int(vdim), int(padded), ps, 0 if unit_norm_eps is None else 1,
-            float(unit_norm_eps or 0.0), float(temp_coef), int(temp_every), self._stream()))
+            float(unit_norm_eps or 0.0), _ptr(q_weight), _ptr(k_weight), float(temp_coef), int(temp_every),
+            self._stream()))
         return out
 
     def head_gate(self, x: torch.Tensor, x_head: int, heads: int, vdim: int, gate: Optional[torch.Tensor] = None) -> torch.Tensor:

@@ -10,7 +10,7 @@ from typing import Optional
 from ..csrc import build as _build
 from .dispatch import ProductShape, Route, Tunables
 
-ABI_VERSION = 34
+ABI_VERSION = 35
 
 _lib: Optional[ctypes.CDLL] = None
 _lib_path: Optional[str] = None
@@ -39,14 +39,21 @@ _SIGNATURES = {
     "lmsf_paged_attention_decode_mfma": (c_int, [_P, c_long, _P, c_long, _P, _P, c_long, _P, c_int, _P, c_int, _P, _P,
                                                  c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_int, _P, c_int,
                                                  _P]),
-    "lmsf_paged_attention_generic_capped": (c_int, [_P, c_long, _P, c_long, _P, _P, c_long, _P, c_int, _P, _P, c_int,
-                                                    c_int, c_int, c_int, c_int, c_float, c_int, c_float, c_int, _P]),
-    "lmsf_paged_attention_prefill_mfma_capped": (c_int, [_P, c_long, _P, c_long, _P, _P, c_long, _P, c_int, _P, c_int, _P,
-                                                         _P, c_int, c_int, c_int, c_int, c_float, c_int, c_float, c_int,
-                                                         _P]),
-    "lmsf_paged_attention_decode_mfma_capped": (c_int, [_P, c_long, _P, c_long, _P, _P, c_long, _P, c_int, _P, c_int, _P,
-                                                        _P, c_int, c_int, c_int, c_int, c_float, c_int, c_float, c_int,
+    "lmsf_paged_attention_generic_biased": (c_int, [_P, c_long, _P, c_long, _P, _P, c_long, _P, c_int, _P, _P, c_int,
+                                                    c_int, c_int, c_int, c_int, c_float, c_int, c_float, _P, c_int, _P]),
+    "lmsf_paged_attention_prefill_mfma_biased": (c_int, [_P, c_long, _P, c_long, _P, _P, c_long, _P, c_int, _P, c_int, _P,
+                                                         _P, c_int, c_int, c_int, c_int, c_float, c_int, c_float, _P,
+                                                         c_int, _P]),
+    "lmsf_paged_attention_decode_mfma_biased": (c_int, [_P, c_long, _P, c_long, _P, _P, c_long, _P, c_int, _P, c_int, _P,
+                                                        _P, c_int, c_int, c_int, c_int, c_float, c_int, c_float, _P, c_int,
                                                         c_int, _P, c_int, _P]),
+    "lmsf_position_embedding": (c_int, [_P, _P, _P, _P, c_int, c_float, _P, _P, c_int, c_int, c_int, c_int, _P, _P]),
+    "lmsf_linear_recurrence_entry_floats": (c_long, [c_int]),
+    "lmsf_linear_recurrence_gates": (c_int, [_P, c_int, c_long, _P, _P, _P, _P, _P, _P, _P, c_int, c_int, c_int, _P]),
+    "lmsf_linear_recurrence_step": (c_int, [_P, c_int, c_long, _P, _P, _P, _P, _P, _P, c_long, _P, c_long, _P, _P, _P, c_long,
+                                            c_int, c_int, c_int, _P]),
+    "lmsf_linear_recurrence_scan": (c_int, [_P, _P, _P, c_int, c_long, _P, c_long, _P, _P, _P, c_long, c_int, c_int, c_int,
+                                            c_int, c_int, _P, _P, _P]),
     "lmsf_hashed_pair_embedding": (c_int, [_P, _P, _P, _P, _P, _P, _P, _P, c_int, _P, _P, c_int, c_int, c_int, c_int,
                                            c_int, c_long, c_long, _P]),
     "lmsf_concat_rows": (c_int, [_P, _P, _P, c_int, c_int, c_int, c_int, _P]),
@@ -60,7 +67,8 @@ _SIGNATURES = {
     "lmsf_gated_delta_state_floats": (c_long, [c_int, c_int, c_int]),
     "lmsf_gated_delta_scratch_floats": (c_long, [c_int, c_int, c_int, c_int, c_int]),
     "lmsf_gated_delta": (c_int, [_P, c_int, c_long, c_int, c_int, c_int, _P, c_long, _P, _P, _P, c_long, _P, c_long, _P, _P,
-                                 _P, _P, _P, c_long, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, _P]),
+                                 _P, _P, _P, c_long, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float,
+                                 c_int, _P]),
     "lmsf_head_rms_gate": (c_int, [_P, c_long, _P, _P, c_long, c_int, _P, c_long, c_int, c_int, c_int, c_int, c_float, _P]),
     "lmsf_table_moe_act": (c_int, [_P, c_int, c_long, _P, _P, _P, _P, c_int, c_int, c_int, c_float, _P, c_long, _P, _P, _P,
                                    c_int, _P, _P, c_long, c_int, c_int, c_int, _P, _P, _P]),
@@ -104,8 +112,8 @@ _SIGNATURES = {
     "lmsf_mlstm_chunk_entry_floats": (c_long, [c_int, c_int, c_int]),
     "lmsf_mlstm_state_floats": (c_long, [c_int, c_int, c_int]),
     "lmsf_attn_prepare": (c_int, [_P, c_long, _P, c_long, _P, c_long, c_int, _P, _P, c_int, c_int, _P, _P, c_long, _P, _P,
-                                  c_long, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_int,
-                                  _P]),
+                                  c_long, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, _P, _P, c_float,
+                                  c_int, _P]),
     "lmsf_head_gate": (c_int, [_P, c_int, c_long, c_int, _P, c_long, _P, c_long, c_int, c_int, c_int, _P]),
     "lmsf_rms_pair": (c_int, [_P, c_long, _P, c_long, c_int, _P, _P, _P, c_int, c_int, c_float, c_float, _P]),
     "lmsf_gated_act": (c_int, [_P, _P, c_int, c_int, c_int, c_long, c_int, _P]),

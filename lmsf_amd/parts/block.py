@@ -351,3 +351,53 @@ class SandwichBlock(Block):
         else:
             self._close(n["post_mixer"], a, residual, ctx)
         return None
+
+
+@register_part("block", "output_norm")
+class OutputNormBlock(Block):
+    """A norm on each sublayer's output alone, the sublayers reading the stream as it is:
+
+        x += norm_a(mixer(x));   x += norm_b(ffn(x))
+
+    (without a feed-forward only the first). The stream is float32; a sublayer gets it rounded to the run's type. Every
+    addition with its norm is one kernel, which also hands on the new stream in the run's type: to the feed-forward, or
+    in ``ctx.aux["stream_rounded"]`` to the block that always follows (``link_next``). Nothing is left to add when the
+    block returns. The reference's only arrangement is the pre-norm one
+    (core/src/model_executor/models/llama/llama.rs:286-340)."""
+
+    graph_safe = True
+    recordable = False
+
+    ROLES = ("post_mixer",)          # and "post_ffn" where there is a feed-forward
+
+    def __init__(self, prefix: str, rt: Runtime, mixer, feed_forward, norms):
+        super().__init__(prefix, rt, mixer, feed_forward, norms)
+        self.has_ffn = not getattr(feed_forward, "absent", False)
+        if self.has_ffn and "post_ffn" not in norms:
+            raise ValueError("block %s needs the norm post_ffn behind its feed-forward" % prefix)
+        self._ffn_takes_ids = bool(getattr(feed_forward, "needs_token_ids", False))
+        self.hands_on = False        # whether the block that always follows reads the stream rounded
+
+    def link_next(self, following: Block) -> None:
+        self.hands_on = isinstance(following, OutputNormBlock)
+
+    def _add(self, norm, branch: torch.Tensor, residual: torch.Tensor, want: bool) -> Optional[torch.Tensor]:
+        """stream += norm(branch); with ``want`` the new stream in the run's type."""
+        # (no weight behind the sum: the kernel hands back the new stream itself)
+        return self.rt.ops.group_norm(x=branch, x_weight=norm.weight, residual=residual, groups=norm.groups,
+                                      x_eps=norm.eps, out_dtype=self.rt.dtype, want_out=want)
+
+    def forward(self, branch: Optional[torch.Tensor], residual: torch.Tensor, ctx, binding: CacheBinding):
+        if branch is not None:
+            raise ValueError("output_norm takes no branch that is still to be added")
+        x = ctx.aux.pop("stream_rounded", None)
+        if x is None:
+            x = self.rt.ops.group_norm(residual=residual, out_dtype=self.rt.dtype)
+        a = self.mixer.forward(x, ctx, binding)
+        x = self._add(self.norms["post_mixer"], a, residual, self.has_ffn or self.hands_on)
+        if self.has_ffn:
+            f = self.feed_forward.forward(x, token_ids=ctx.token_ids) if self._ffn_takes_ids else self.feed_forward.forward(x)
+            x = self._add(self.norms["post_ffn"], f, residual, self.hands_on)
+        if self.hands_on:
+            ctx.aux["stream_rounded"] = x
+        return None

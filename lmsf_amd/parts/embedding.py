@@ -94,6 +94,48 @@ class HashedPairEmbedding(Part):
         return x
 
 
+@register_part("embedding", "positioned_embedding")
+class PositionedEmbedding(Part):
+    """x = scale * table[id] + places[position]: a learned vector per position beside the token's row; the sum is
+    float32. The same rounded to the run's type is left in ``ctx.aux["stream_rounded"]`` for a block whose sublayer
+    reads the stream as it is. The reference's embedding is the plain row gather
+    (core/src/model_executor/layers/vocab_parallel_embedding.rs:28-38)."""
+
+    graph_safe = True
+    recordable = False
+    needs_context = True
+
+    def __init__(self, prefix: str, rt: Runtime, vocab_size: int, hidden_size: int, positions: int, scale: float = 1.0,
+                 position_name: str = "pos", weight_name: str = ""):
+        super().__init__(prefix, rt)
+        self.vocab_size, self.hidden_size, self.positions = int(vocab_size), int(hidden_size), int(positions)
+        self.scale = float(scale)
+        if rt.max_positions > self.positions:
+            raise ValueError("%s: requests of up to %d tokens, but vectors for %d positions"
+                             % (position_name, rt.max_positions, self.positions))
+        self.weight_name = "%s.%s" % (prefix, weight_name) if weight_name else prefix
+        self.position_name = str(position_name)
+        self.weight: Optional[torch.Tensor] = None
+        self.places: Optional[torch.Tensor] = None
+
+    def checkpoint_tensors(self) -> Dict[str, TensorDecl]:
+        return {self.weight_name: TensorDecl((self.vocab_size, self.hidden_size)),
+                self.position_name: TensorDecl((self.positions, self.hidden_size))}
+
+    def load_weights(self, fetch: Callable[[str], torch.Tensor]) -> None:
+        self.weight = fetch(self.weight_name).contiguous()
+        self.places = fetch(self.position_name).to(self.weight.dtype).contiguous()
+
+    def tensors(self):
+        return [t for t in (self.weight, self.places) if t is not None]
+
+    def forward_step(self, ctx) -> torch.Tensor:
+        """The step's tokens -> float32 [N, H]."""
+        x, rounded = self.rt.ops.position_embedding(ctx.token_ids, ctx.positions, self.weight, self.places, self.scale)
+        ctx.aux["stream_rounded"] = rounded
+        return x
+
+
 @register_part("head", "lm_head")
 class LMHead(Part):
     """``weight_name`` is the full checkpoint name of the [V, H] matrix: the head's own, or the

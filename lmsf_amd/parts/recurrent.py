@@ -1,11 +1,11 @@
-"""Mixers whose memory of a request is a state of fixed size: the selective scan and a matrix memory with
-exponential gates, and the short causal convolution that both they and some attention layers put behind a
+"""Mixers whose memory of a request is a state of fixed size: the selective scan, a matrix memory with
+exponential gates and a gated linear recurrence, and the short causal convolution that both they and some attention layers put behind a
 projection.
 
 A request's state is one row of float32 numbers in the engine's state slots (``StateSpec``); a mixer says how
 many it needs and gets ``binding.state`` [slots, that many]. The engine clears a row when a request takes it, so
 "zeros before the sequence's start" and "the state starts at zero" need no code here. Everything that enters a
-recurrence is float32 (csrc/recurrent.hip); the projections run in the run's dtype. The reference has no mixer
+recurrence is float32 (csrc/recurrent.hip, csrc/linear_recurrence.hip); the projections run in the run's dtype. The reference has no mixer
 with state (its only one is attention over a paged cache, core/src/model_executor/layers/attention.rs:91-231).
 """
 from typing import Callable, Dict, Optional, Sequence, Tuple
@@ -164,4 +164,65 @@ class MatrixMemory(Mixer):
         o = ops.mlstm(p[:, :H * d], p[:, H * d:2 * H * d], p[:, 2 * H * d:2 * H * d + H * dv], gates,
                       p[:, 2 * H * d + H * dv:], self.norm.weight, binding.state, ctx, H, d, dv, d ** -0.5, self.cap,
                       self.eps)
+        return self.o.forward(o)
+
+
+@register_part("mixer", "gated_linear_recurrence")
+class GatedLinearRecurrence(Mixer):
+    """Griffin's recurrent block with a real-gated linear recurrence. Two branches of C = ``width`` channels,
+    y = gelu_tanh(W_y h + b_y) and u = conv(W_x h + b_x) + b_c (no activation). u is cut into ``blocks`` equal parts, each
+    with its own square matrices: r = sigmoid(W_r u + b_r), i = sigmoid(W_i u + b_i). log a = -decay * r * softplus(lam);
+    S <- a S + sqrt(1 - a^2) i u; out = W_o (S * y). State of a request: S [C] and the convolution's last taps - 1 inputs."""
+
+    graph_safe = True
+    recordable = False
+
+    def __init__(self, prefix: str, rt: Runtime, hidden_size: int, width: int, blocks: int, conv: int, decay: float = 8.0,
+                 names: Optional[Dict[str, str]] = None):
+        super().__init__(prefix, rt)
+        self.C, self.blocks, self.taps, self.decay = int(width), int(blocks), int(conv), float(decay)
+        if self.blocks < 1 or self.C % self.blocks:
+            raise ValueError("%s: %d channels do not split into %d blocks" % (prefix, self.C, self.blocks))
+        nm = dict(y="y", x="x", bias="b", conv="conv", conv_bias="conv.b", r="ra", r_bias="ra.b", i="ri", i_bias="ri.b",
+                  lam="lam", out="o")
+        nm.update(names or {})
+        self.proj = FusedLinear(prefix, rt, hidden_size, [(nm["y"], self.C), (nm["x"], self.C)], bias=True,
+                                bare_names=True, bias_name=nm["bias"])
+        self.conv = ShortConv(prefix, rt, [(nm["conv"], self.C)], self.taps, bias_name=nm["conv_bias"])
+        self.o = Linear(prefix, rt, nm["out"], self.C, hidden_size, bare_names=True)
+        self.names = {k: "%s.%s" % (prefix, nm[k]) for k in ("r", "r_bias", "i", "i_bias", "lam")}
+        self.wr: Optional[torch.Tensor] = None       # [blocks, C / blocks, C / blocks]
+        self.wi: Optional[torch.Tensor] = None
+        self.br: Optional[torch.Tensor] = None       # float32 [C]
+        self.bi: Optional[torch.Tensor] = None
+        self.rate: Optional[torch.Tensor] = None     # float32 [C]: decay * softplus(lam)
+
+    def children(self):
+        return [self.proj, self.conv, self.o]
+
+    def checkpoint_tensors(self) -> Dict[str, TensorDecl]:
+        c = self.C // self.blocks
+        nm = self.names
+        return {nm["r"]: TensorDecl((self.blocks, c, c)), nm["i"]: TensorDecl((self.blocks, c, c)),
+                nm["r_bias"]: TensorDecl((self.blocks, c), init="zeros", keeps_float32=True),
+                nm["i_bias"]: TensorDecl((self.blocks, c), init="zeros", keeps_float32=True),
+                nm["lam"]: TensorDecl((self.C,), init="const:-2.0", keeps_float32=True)}
+
+    def load_weights(self, fetch: Callable[[str], torch.Tensor]) -> None:
+        nm = self.names
+        self.wr, self.wi = (fetch(nm[k]).to(self.rt.dtype).contiguous() for k in ("r", "i"))
+        self.br, self.bi = (fetch(nm[k]).to(torch.float32).reshape(-1).contiguous() for k in ("r_bias", "i_bias"))
+        self.rate = (self.decay * torch.nn.functional.softplus(fetch(nm["lam"]).to(torch.float32))).contiguous()
+
+    def tensors(self):
+        return [t for t in (self.wr, self.wi, self.br, self.bi, self.rate) if t is not None]
+
+    def state_spec(self) -> Optional[StateSpec]:
+        return StateSpec((self.C + self.conv.state_floats,), torch.float32)
+
+    def forward(self, h: torch.Tensor, ctx, binding: CacheBinding) -> torch.Tensor:
+        st = binding.state
+        p = self.proj.forward(h)                                                # [N, y | x]
+        u = self.conv.forward(p[:, self.C:], ctx, st[:, self.C:] if self.taps > 1 else None)
+        o = self.rt.ops.linear_recurrence(u, self.wr, self.br, self.wi, self.bi, self.rate, p[:, :self.C], st, ctx)
         return self.o.forward(o)

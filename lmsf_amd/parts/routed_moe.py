@@ -5,7 +5,7 @@ feed-forward y_e(x) = Wd_e (silu(Wg_e x) * (Wu_e x)) without biases. Options: ``
 ``groups`` / ``keep_groups``: the experts form equal groups of neighbours, a group's score is its best expert's, and
 only experts of the best ``keep_groups`` groups can be chosen; ``gated`` False: experts of one matrix in,
 y_e(x) = Wd_e relu(Wu_e x)^2; ``weight_on`` "output": a weight multiplies what its expert returns. The weights are the chosen scores (divided by
-their sum with ``renormalize``). A weight multiplies what its expert is given, not what it returns: the layer's
+their sum with ``renormalize``; with softmax scores that is the softmax over the chosen experts' logits alone). A weight multiplies what its expert is given, not what it returns: the layer's
 result is sum_e y_e(s_e h). An expert that every token runs (``shared``) is added, multiplied by sigmoid(w_sg . h), one
 number a token, where ``shared_gate`` names that vector.
 

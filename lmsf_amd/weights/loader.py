@@ -33,6 +33,19 @@ class WeightsError(ValueError):
         self.wrong_shape = list(wrong_shape)
 
 
+def header_shapes(folder: str) -> Dict[str, Tuple[int, ...]]:
+    """Names and shapes of a folder's checkpoint tensors, from the files' headers alone."""
+    shapes: Dict[str, Tuple[int, ...]] = {}
+    for path in list_weight_files(folder):
+        f = SafetensorsFile(path)
+        try:
+            for name, e in f.entries.items():
+                shapes[name] = tuple(e.shape)
+        finally:
+            f.close()
+    return shapes
+
+
 def collect_declarations(parts: Iterable[Part], shared: Optional[set] = None) -> Dict[str, TensorDecl]:
     """Every declared tensor by name; ``shared`` (a set, if given) takes the names that more than one part
     declares (tied weights)."""

@@ -125,7 +125,7 @@ class TorchOps:
 
     # ------------------------------------------------------------ attention
     def paged_attention(self, q, k_pages, v_pages, block_tables, seg, pos, nh, nkv, d, scale, window=0, batch=None,
-                        kernel=None, chunk=0, weights_f32=False, softcap=0.0):
+                        kernel=None, chunk=0, weights_f32=False, softcap=0.0, distance_bias=None):
         N = q.shape[0]
         ps = k_pages.shape[2]
         out = torch.empty((N, nh * d), dtype=q.dtype, device=q.device)
@@ -145,6 +145,9 @@ class TorchOps:
             sc = torch.einsum("hd,nhd->hn", qt, keys) * scale
             if softcap and softcap > 0:
                 sc = softcap * torch.tanh(sc / softcap)
+            if distance_bias is not None:
+                r1, r2 = distance_bias[0][:, None], distance_bias[1][:, None]
+                sc = sc - r1 * torch.log1p(r2 * (p - js).to(torch.float32)[None, :])
             pr = torch.softmax(sc, dim=-1)
             out[t] = torch.einsum("hn,nhd->hd", pr, vals).reshape(nh * d).to(q.dtype)
         return out
@@ -283,6 +286,10 @@ class TorchOps:
         out = table[ids].to(torch.float32) + pairs[rows].to(torch.float32)
         return (out, out.clone()) if keep else out
 
+    def position_embedding(self, ids, positions, table, places, scale=1.0):
+        x = table[ids.long()].to(torch.float32) * scale + places[positions.long()].to(torch.float32)
+        return x, x.to(table.dtype)
+
     def concat_rows(self, a, b, out_dtype):
         return torch.cat([a, b], -1).to(out_dtype)
 
@@ -359,7 +366,7 @@ class TorchOps:
         return heads * dim * vdim
 
     def gated_delta(self, qkv, q_at, k_at, v_at, a, dt_bias, a_log, b, state, batch, heads, kv_heads, dim, vdim,
-                    q_scale, unit_eps=1e-6):
+                    q_scale, unit_eps=1e-6, per_head=False):
         N = qkv.shape[0]
         rep = heads // kv_heads
         q = qkv[:, q_at:q_at + kv_heads * dim].to(torch.float32).reshape(N, kv_heads, dim)
@@ -368,8 +375,9 @@ class TorchOps:
         q = (q / torch.sqrt((q * q).sum(-1, keepdim=True) + unit_eps) * q_scale).repeat_interleave(rep, 1)
         k = (k / torch.sqrt((k * k).sum(-1, keepdim=True) + unit_eps)).repeat_interleave(rep, 1)
         beta = torch.sigmoid(b[:, :heads])
+        per = 1 if per_head else dim
         g = torch.exp(-torch.exp(a_log)[None, :, None] * torch.nn.functional.softplus(
-            a[:, :heads * dim] + dt_bias).reshape(N, heads, dim))
+            a[:, :heads * per] + dt_bias).reshape(N, heads, per)).expand(N, heads, dim)
         out = torch.zeros((N, heads, vdim), dtype=torch.float32)
         for t0, t1, slot in self._segments(batch):
             S = state[slot, :heads * dim * vdim].reshape(heads, dim, vdim).clone()
@@ -481,6 +489,28 @@ class TorchOps:
             state[slot, :inner * n] = S.reshape(-1)
         return y
 
+    def linear_recurrence(self, u, wr, br, wi, bi, rate, y, state, batch):
+        N, C = u.shape
+        blocks, c, _ = wr.shape
+        uf = u.to(torch.float32)
+
+        def gate(w, b):
+            parts = [uf[:, k * c:(k + 1) * c] @ w[k].to(torch.float32).t() for k in range(blocks)]
+            return torch.sigmoid(torch.cat(parts, 1) + b)
+        log_a = -rate * gate(wr, br)
+        a = torch.exp(log_a)
+        b = torch.sqrt(-torch.expm1(2.0 * log_a)) * gate(wi, bi) * uf
+        yf = y[:, :C].to(torch.float32)
+        yf = 0.5 * yf * (1.0 + torch.tanh(0.7978845608028654 * (yf + 0.044715 * yf ** 3)))
+        out = torch.empty((N, C), dtype=u.dtype)
+        for t0, t1, slot in self._segments(batch):
+            S = state[slot, :C].clone()
+            for t in range(t0, t1):
+                S = a[t] * S + b[t]
+                out[t] = (S * yf[t]).to(u.dtype)
+            state[slot, :C] = S
+        return out
+
     def mlstm_state_floats(self, heads, dim, vdim):
         return heads * dim * (vdim + 1) + heads
 
@@ -511,13 +541,17 @@ class TorchOps:
         return out
 
     def attn_prepare(self, q, k, v, heads, kv_heads, dim, vdim, padded, positions, slots, k_pages, v_pages, table=None,
-                     unit_norm_eps=None, temp_coef=0.0, temp_every=0):
+                     unit_norm_eps=None, temp_coef=0.0, temp_every=0, q_weight=None, k_weight=None):
         N = q.shape[0]
         qf = q[:, :heads * dim].to(torch.float32).reshape(N, heads, dim)
         kf = k[:, :kv_heads * dim].to(torch.float32).reshape(N, kv_heads, dim)
         if unit_norm_eps is not None:
             qf = qf / torch.sqrt((qf * qf).mean(-1, keepdim=True) + unit_norm_eps)
             kf = kf / torch.sqrt((kf * kf).mean(-1, keepdim=True) + unit_norm_eps)
+        if q_weight is not None:
+            qf = qf * q_weight
+        if k_weight is not None:
+            kf = kf * k_weight
         if table is not None:
             rot = table.shape[1]
             cs = table[positions.long()][:, None, :]
