@@ -564,6 +564,35 @@ def beside_llama_run(args, design, sizes, shapes, twin="llama"):
     print(json.dumps(out))
 
 
+def gurapel_shapes(name):
+    """A Gurapel configuration at sizes that resemble a real model's layers, and beside it the Murulorn configuration of
+    equal width and layers (the closest architecture of the package: attention within a window under a soft cap, the
+    delta rule, routed experts). Eight layers: three of attention (Gurapel: beside the linear recurrence, as wide as the
+    model in blocks of 256 channels), then one of the delta rule, twice; 2 experts a token in every layer; keys and values
+    of 128 entries, four query heads a key head, a window of 1,024; a memory per head of 64 x 128."""
+    W, H, E, eff = {"2b": (2048, 16, 16, 1024), "7b": (4096, 32, 32, 2048)}[name]
+    att = {"heads": H, "kv_heads": H // 4, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "softcap": 30.0, "mask": {"size": 1024}}
+    mem = {"heads": H, "kv_heads": H, "dim": 64, "vdim": 128, "conv": 4}
+    moe = {"kind": "moe", "expert": {"ff": eff}, "router": {"experts": E, "top": 2}}
+    both = {"left": att, "right": {"width": W, "blocks": W // 256, "conv": 4}}
+    common = {"vocab": 32000, "width": W, "norm": {"eps": 1e-6}, "max_position_embeddings": 8192, "torch_dtype": "bfloat16"}
+    gur = dict(common, architecture="Gurapel", embedding={"scale": 1.0}, max_positions=8192,
+               layers=[{"type": t, "mixer": dict(m), "mlp": dict(moe)} for t, m in ([("parallel", both)] * 3 + [("delta", mem)]) * 2])
+    att = dict(att, rot={"base": 1e6, "dims": 64})
+    mem = dict(mem, decay_rank=64, gate_rank=64)
+    mur = dict(common, architecture="Murulorn",
+               embedding={"bigram": {"buckets": 100003, "mul_prev": 1000003, "mul_cur": 31}},
+               layers=[{"type": t, "mixer": dict(m), "mlp": dict(moe)}
+                       for t, m in ([("attention", att)] * 3 + [("channel_delta", mem)]) * 2])
+    return gur, mur
+
+
+def gurapel_run(args):
+    """``--workload gurapel``: prefill and decode of a Gurapel model beside the Murulorn model of equal width and layers;
+    one JSON line, as for the other designs."""
+    beside_llama_run(args, "gurapel", args.gurapel_sizes, gurapel_shapes(args.gurapel_sizes), twin="murulorn")
+
+
 def prefill_flops(cfg, T):
     """Multiply-adds times two of a causal prefill of T tokens: the linear layers on every token, the
     attention scores and values over the causal half, the LM head on one row."""
@@ -587,13 +616,14 @@ def main():
     ap.add_argument("--max-num-batched-tokens", type=int, default=8192)
     ap.add_argument("--gpu-memory-utilization", type=float, default=0.85)
     ap.add_argument("--skip-points", action="store_true", help="leave out the batch 1 and batch 64 runs")
-    ap.add_argument("--workload", default="decode", choices=["decode", "serve", "products", "takosun", "niresun", "zevetar", "murulorn"],
+    ap.add_argument("--workload", default="decode", choices=["decode", "serve", "products", "takosun", "niresun", "zevetar", "murulorn", "gurapel"],
                     help="decode: the default line (Llama-3-8B shape); serve: continuous batching of 64 requests at "
                          "Llama-2-7B shape, a line of its own; products: a layer's matrix products alone, the "
                          "library's against the engine's choice, at --rows; takosun: a Takosun model beside the Llama model "
                          "of equal size, prefill and decode; niresun: the same for a Niresun model; zevetar: a Zevetar "
                          "model beside the Takosun model of equal size; murulorn: a Murulorn model beside the Zevetar "
-                         "model of equal width and layer runs")
+                         "model of equal width and layer runs; gurapel: a Gurapel model beside the Murulorn model of "
+                         "equal width and layers")
     ap.add_argument("--takosun-sizes", default="2b", choices=["2b", "7b"], help="takosun: the layers' sizes")
     ap.add_argument("--niresun-sizes", default="2b", choices=["2b", "7b"],
                     help="niresun: the layers' sizes (a Niresun model beside the Llama model of equal size)")
@@ -601,6 +631,8 @@ def main():
                     help="zevetar: the layers' sizes (a Zevetar model beside the Takosun model of equal size)")
     ap.add_argument("--murulorn-sizes", default="2b", choices=["2b", "7b"],
                     help="murulorn: the layers' sizes (a Murulorn model beside the Zevetar model of equal width and layer runs)")
+    ap.add_argument("--gurapel-sizes", default="2b", choices=["2b", "7b"],
+                    help="gurapel: the layers' sizes (a Gurapel model beside the Murulorn model of equal width and layers)")
     ap.add_argument("--rows", default="17,64,100,128,129,192,256,512,2048", help="products: numbers of rows")
     ap.add_argument("--prefill-chunk-size", type=int, default=1024, help="serve: longest portion of a prompt in a step")
     ap.add_argument("--shape", default="llama3-8b", choices=sorted(SHAPES),
@@ -644,6 +676,9 @@ def main():
         return
     if args.workload == "murulorn":
         murulorn_run(args)
+        return
+    if args.workload == "gurapel":
+        gurapel_run(args)
         return
     if args.workload == "zevetar":
         zevetar_run(args)

@@ -84,6 +84,83 @@ __global__ __launch_bounds__(256) void attn_prepare_kernel(
   }
 }
 
+// The same without rotation (which needs another lane's entry), for sizes that are multiples of 8 and rows and heads at
+// multiples of 16 bytes: L lanes a head (L a power of two, 8 L >= D), eight entries a lane in registers, 64 / L heads of a
+// token a wave.
+template <typename T>
+__device__ __forceinline__ void ap_load8(const T* p, float* x) {
+#pragma unroll
+  for (int h = 0; h < 8 / Vec16<T>::N; ++h) {
+    Vec16<T> v;
+    v.load(p + h * Vec16<T>::N);
+#pragma unroll
+    for (int j = 0; j < Vec16<T>::N; ++j) x[h * Vec16<T>::N + j] = v.get(j);
+  }
+}
+template <typename T>
+__device__ __forceinline__ void ap_store8(T* p, const float* x) {
+#pragma unroll
+  for (int h = 0; h < 8 / Vec16<T>::N; ++h) {
+    Vec16<T> v;
+#pragma unroll
+    for (int j = 0; j < Vec16<T>::N; ++j) v.set(j, x[h * Vec16<T>::N + j]);
+    v.store(p + h * Vec16<T>::N);
+  }
+}
+template <typename T, int L>
+__global__ __launch_bounds__(256) void attn_prepare_rows_kernel(
+    const T* __restrict__ q, long q_stride, const T* __restrict__ k, long k_stride, const T* __restrict__ v,
+    long v_stride, const int* __restrict__ positions, const int* __restrict__ slots, T* __restrict__ q_out,
+    long qo_stride, T* __restrict__ k_pages, T* __restrict__ v_pages, int n_tokens, int H, int G, int dim, int vdim,
+    int D, int ps, int unit_norm, float eps, const float* __restrict__ wq, const float* __restrict__ wk,
+    float temp_coef, int temp_every) {
+  constexpr int HPW = LMSF_WAVE / L;
+  const int per_token = (H + 2 * G + HPW - 1) / HPW;
+  const long wave = (long)blockIdx.x * (256 / LMSF_WAVE) + threadIdx.x / LMSF_WAVE;
+  const int t = (int)(wave / per_token), lane = threadIdx.x % LMSF_WAVE;
+  if (t >= n_tokens) return;
+  const int u = (int)(wave - (long)t * per_token) * HPW + lane / L, e0 = (lane % L) * 8;
+  const bool is_q = u < H, is_v = u >= H + G, live = u < H + 2 * G;
+  const int head = is_q ? u : is_v ? u - H - G : u - H, width = is_v ? vdim : dim;
+  const int slot = slots ? slots[t] : -1;
+  float x[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+  if (live && e0 < width)
+    ap_load8<T>((is_q ? q + (long)t * q_stride : is_v ? v + (long)t * v_stride : k + (long)t * k_stride) + (long)head * width + e0, x);
+  if (unit_norm) {
+    float ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) ss = fmaf(x[j], x[j], ss);
+#pragma unroll
+    for (int o = L / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o, LMSF_WAVE);       // (within the head's lanes)
+    const float inv = is_v ? 1.f : 1.f / sqrtf(ss / (float)dim + eps);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) x[j] *= inv;
+  }
+  if (!live || e0 >= D || (!is_q && slot < 0)) return;
+  const float* w = is_q ? wq : is_v ? nullptr : wk;
+  if (w && e0 < dim) {
+    const float4 a = *reinterpret_cast<const float4*>(w + e0), b = *reinterpret_cast<const float4*>(w + e0 + 4);
+    x[0] *= a.x; x[1] *= a.y; x[2] *= a.z; x[3] *= a.w; x[4] *= b.x; x[5] *= b.y; x[6] *= b.z; x[7] *= b.w;
+  }
+  if (is_q) {
+    if (temp_every > 0) {
+      const float temp = 1.f + temp_coef * logf((float)((positions[t] + 1) / temp_every) + 1.f);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) x[j] *= temp;
+    }
+    ap_store8<T>(q_out + (long)t * qo_stride + (long)head * D + e0, x);
+    return;
+  }
+  const int page = slot / ps, off = slot - page * ps;
+  if (is_v) {
+    T* dst = v_pages + (((long)page * G + head) * D + e0) * ps + off;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) dst[(long)j * ps] = from_f32<T>(x[j]);
+  } else {
+    ap_store8<T>(k_pages + (((long)page * G + head) * ps + off) * D + e0, x);
+  }
+}
+
 extern "C" int lmsf_attn_prepare(const void* q, long q_stride, const void* k, long k_stride, const void* v,
                                  long v_stride, int dtype, const int* positions, const float* table, int rot,
                                  int max_pos, const int* slots, void* q_out, long qo_stride, void* k_pages,
@@ -101,6 +178,29 @@ extern "C" int lmsf_attn_prepare(const void* q, long q_stride, const void* k, lo
   LMSF_CHECK(!slots || (k_pages && v_pages && ps > 0 && num_pages > 0), "attn_prepare: slots without pages");
   LMSF_CHECK(temp_every >= 0, "attn_prepare: negative temperature period");
   if (n_tokens == 0) return 0;
+  const int al = dtype == LMSF_F32 ? 4 : 8;         // entries in 16 bytes
+  if (!table && D <= 512 && dim % 8 == 0 && vdim % 8 == 0 && D % 8 == 0 && q_stride % al == 0 && k_stride % al == 0 &&
+      v_stride % al == 0 && qo_stride % al == 0 && lmsf_aligned16(q) && lmsf_aligned16(k) && lmsf_aligned16(v) &&
+      lmsf_aligned16(q_out) && (!slots || (lmsf_aligned16(k_pages) && lmsf_aligned16(v_pages))) &&
+      (!wq || lmsf_aligned16(wq)) && (!wk || lmsf_aligned16(wk))) {
+    const int L = D <= 32 ? 4 : D <= 64 ? 8 : D <= 128 ? 16 : D <= 256 ? 32 : 64;
+    const long waves = (long)n_tokens * ((H + 2 * G + LMSF_WAVE / L - 1) / (LMSF_WAVE / L));
+    const dim3 rgrid((unsigned)((waves + 3) / 4));
+#define AP_ROWS(T, LL)                                                                                                \
+  hipLaunchKernelGGL((attn_prepare_rows_kernel<T, LL>), rgrid, dim3(256), 0, stream, (const T*)q, q_stride, (const T*)k, \
+                     k_stride, (const T*)v, v_stride, positions, slots, (T*)q_out, qo_stride, (T*)k_pages, (T*)v_pages, \
+                     n_tokens, H, G, dim, vdim, D, ps, unit_norm, eps, wq, wk, temp_coef, temp_every)
+#define AP_L(T)                                                                                                      \
+  do {                                                                                                               \
+    if (L == 4) AP_ROWS(T, 4); else if (L == 8) AP_ROWS(T, 8); else if (L == 16) AP_ROWS(T, 16);                     \
+    else if (L == 32) AP_ROWS(T, 32); else AP_ROWS(T, 64);                                                           \
+  } while (0)
+    if (dtype == LMSF_F32) AP_L(float); else AP_L(bf16_t);
+#undef AP_L
+#undef AP_ROWS
+    LMSF_LAUNCH_CHECK("attn_prepare");
+    return 0;
+  }
   // few tokens: the heads spread over workgroups (8 tokens: 8.4 -> 4.1 us); many: a workgroup a token walks its heads
   // (2,048 tokens: 17.4 us against 23 with the heads spread)
   const dim3 grid(n_tokens, n_tokens >= 256 ? 1 : std::min((H + 2 * G + 3) / 4, 65535));

@@ -55,6 +55,11 @@ int lmsf_group_norm(const void* branch, int branch_dtype, long branch_stride, co
     float* hist, long hist_stride, int hist_index, const float* mix, const float* wn, void* out, int out_dtype,
     long out_stride, const int* rows, int n_rows, int W, int groups, float eps_b, float eps_n, hipStream_t stream);
 
+int lmsf_norm_add_fits(int W);
+int lmsf_norm_add(const void* a, long a_stride, const void* b, long b_stride, int dtype, const float* wa, const float*
+    wb, float eps_pair, float scale, const float* wn, float eps, float* residual, void* out, int n_rows, int W,
+    hipStream_t stream);
+
 // latent.hip
 int lmsf_latent_cache_write(const void* x, int dtype, long x_stride, const float* w, float eps, const int* positions,
     const float* table, int rot, int max_pos, const int* slots, void* k_pages, void* v_pages, long num_pages,

@@ -141,3 +141,154 @@ extern "C" int lmsf_group_norm(const void* branch, int branch_dtype, long branch
   LMSF_LAUNCH_CHECK("group_norm");
   return 0;
 }
+
+// ---------------------------------------------------------------- a sublayer's output, normed, into the stream
+//
+//   v = b ? scale (a / rms(a) * wa + b / rms(b) * wb) : a;    residual += v / rms(v) * wn;    out = residual in T
+//
+// (two mixers side by side are joined on the way: nothing of v goes through memory). A workgroup a row, the row in
+// registers, four neighbours an access; everything that comes from memory is asked for before the first sum.
+
+template <typename T> struct Na4;
+template <> struct Na4<float> {
+  static __device__ __forceinline__ void load(const float* p, float* x) {
+    const float4 v = *reinterpret_cast<const float4*>(p);
+    x[0] = v.x; x[1] = v.y; x[2] = v.z; x[3] = v.w;
+  }
+  static __device__ __forceinline__ void store(float* p, const float* x) {
+    *reinterpret_cast<float4*>(p) = make_float4(x[0], x[1], x[2], x[3]);
+  }
+};
+template <> struct Na4<bf16_t> {
+  static __device__ __forceinline__ void load(const bf16_t* p, float* x) {
+    const uint2 v = *reinterpret_cast<const uint2*>(p);
+    x[0] = __uint_as_float(v.x << 16); x[1] = __uint_as_float(v.x & 0xffff0000u);
+    x[2] = __uint_as_float(v.y << 16); x[3] = __uint_as_float(v.y & 0xffff0000u);
+  }
+  static __device__ __forceinline__ void store(bf16_t* p, const float* x) {
+    *reinterpret_cast<uint2*>(p) = make_uint2(pack2_bf16(x[0], x[1]), pack2_bf16(x[2], x[3]));
+  }
+};
+
+// E: groups of four entries a thread holds
+template <typename T, bool PAIR, int E>
+__global__ __launch_bounds__(1024) void norm_add_kernel(const T* __restrict__ a, long a_stride, const T* __restrict__ b,
+                                                        long b_stride, const float* __restrict__ wa,
+                                                        const float* __restrict__ wb, float eps_pair, float scale,
+                                                        const float* __restrict__ wn, float eps,
+                                                        float* __restrict__ residual, T* __restrict__ out, int W) {
+  __shared__ float red[3][16];
+  const long n = blockIdx.x;
+  const int wave = threadIdx.x / LMSF_WAVE, lane = threadIdx.x % LMSF_WAVE, n_waves = blockDim.x / LMSF_WAVE;
+  float va[E][4], vb[E][4], res[E][4], w[E][4];
+#pragma unroll
+  for (int e = 0; e < E; ++e) {
+    const int i = (threadIdx.x + e * blockDim.x) * 4;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) va[e][j] = vb[e][j] = 0.f;
+    if (i < W) {
+      Na4<T>::load(a + n * a_stride + i, va[e]);
+      if (PAIR) Na4<T>::load(b + n * b_stride + i, vb[e]);
+      Na4<float>::load(residual + n * W + i, res[e]);
+      Na4<float>::load(wn + i, w[e]);
+    }
+  }
+  if (PAIR) {
+    float sa = 0.f, sb = 0.f;
+#pragma unroll
+    for (int e = 0; e < E; ++e)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        sa = fmaf(va[e][j], va[e][j], sa);
+        sb = fmaf(vb[e][j], vb[e][j], sb);
+      }
+    sa = wave_sum(sa);
+    sb = wave_sum(sb);
+    if (lane == 0) {
+      red[0][wave] = sa;
+      red[1][wave] = sb;
+    }
+    __syncthreads();
+    sa = sb = 0.f;
+    for (int k = 0; k < n_waves; ++k) {
+      sa += red[0][k];
+      sb += red[1][k];
+    }
+    const float ia = scale / sqrtf(sa / (float)W + eps_pair), ib = scale / sqrtf(sb / (float)W + eps_pair);
+#pragma unroll
+    for (int e = 0; e < E; ++e) {
+      const int i = (threadIdx.x + e * blockDim.x) * 4;
+      if (i < W) {
+        float xa[4], xb[4];
+        Na4<float>::load(wa + i, xa);
+        Na4<float>::load(wb + i, xb);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) va[e][j] = va[e][j] * ia * xa[j] + vb[e][j] * ib * xb[j];
+      }
+    }
+  }
+  float s = 0.f;
+#pragma unroll
+  for (int e = 0; e < E; ++e)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) s = fmaf(va[e][j], va[e][j], s);
+  s = wave_sum(s);
+  if (lane == 0) red[2][wave] = s;
+  __syncthreads();
+  s = 0.f;
+  for (int k = 0; k < n_waves; ++k) s += red[2][k];
+  const float inv = 1.f / sqrtf(s / (float)W + eps);
+#pragma unroll
+  for (int e = 0; e < E; ++e) {
+    const int i = (threadIdx.x + e * blockDim.x) * 4;
+    if (i < W) {
+      float r[4];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) r[j] = res[e][j] + va[e][j] * inv * w[e][j];
+      Na4<float>::store(residual + n * W + i, r);
+      if (out) Na4<T>::store(out + n * W + i, r);
+    }
+  }
+}
+
+// Whether lmsf_norm_add takes rows of W entries (a multiple of 4 that a workgroup holds in registers).
+extern "C" int lmsf_norm_add_fits(int W) { return W > 0 && W % 4 == 0 && W <= 16384; }
+
+// a, b (null: none) [n_rows, W] of ``dtype`` with row strides that are multiples of 4 entries; residual contiguous float32
+// [n_rows, W]; out (null: none) contiguous [n_rows, W] of ``dtype``; the weights float32 [W]; every row 16-byte aligned
+// (8 bytes for bfloat16).
+extern "C" int lmsf_norm_add(const void* a, long a_stride, const void* b, long b_stride, int dtype, const float* wa,
+                             const float* wb, float eps_pair, float scale, const float* wn, float eps, float* residual,
+                             void* out, int n_rows, int W, hipStream_t stream) {
+  LMSF_CHECK(a && wn && residual && (!b || (wa && wb)), "norm_add: null pointer");
+  LMSF_CHECK(dtype == LMSF_F32 || dtype == LMSF_BF16, "norm_add: unknown dtype code %d", dtype);
+  LMSF_CHECK(lmsf_norm_add_fits(W) && a_stride >= W && (!b || b_stride >= W) && a_stride % 4 == 0 && b_stride % 4 == 0,
+             "norm_add: rows of %d entries (multiples of 4 up to 16,384) at strides of multiples of 4", W);
+  LMSF_CHECK(lmsf_aligned16(a) && (!b || lmsf_aligned16(b)) && lmsf_aligned16(residual) && lmsf_aligned16(wn) &&
+                 (!out || lmsf_aligned16(out)) && (!b || (lmsf_aligned16(wa) && lmsf_aligned16(wb))),
+             "norm_add: operands must be 16-byte aligned");
+  if (n_rows <= 0) return 0;
+  // many rows: small workgroups with several accesses a thread; few rows: as many threads as a row has groups of four
+  const int quads = W / 4, per_thread = n_rows >= 512 ? 2 : 1;
+  int threads = 64;
+  while (threads < 1024 && threads * per_thread < quads) threads *= 2;
+  const int need = (quads + threads - 1) / threads;
+#define NA(T, P, E)                                                                                                  \
+  hipLaunchKernelGGL((norm_add_kernel<T, P, E>), dim3(n_rows), dim3(threads), 0, stream, (const T*)a, a_stride,      \
+                     (const T*)b, b_stride, wa, wb, eps_pair, scale, wn, eps, residual, (T*)out, W)
+#define NA_E(T, P)               \
+  do {                           \
+    if (need <= 1) NA(T, P, 1);  \
+    else if (need <= 2) NA(T, P, 2); \
+    else NA(T, P, 4);            \
+  } while (0)
+  if (dtype == LMSF_F32) {
+    if (b) NA_E(float, true); else NA_E(float, false);
+  } else {
+    if (b) NA_E(bf16_t, true); else NA_E(bf16_t, false);
+  }
+#undef NA_E
+#undef NA
+  LMSF_LAUNCH_CHECK("norm_add");
+  return 0;
+}

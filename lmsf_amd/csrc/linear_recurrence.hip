@@ -24,13 +24,38 @@
 
 #include <math.h>
 
-__device__ __forceinline__ float lru_sigmoid(float z) { return 1.f / (1.f + expf(-z)); }
+// In a float32 run the library's functions; in a bfloat16 run the hardware's 2^x, reciprocal and square root (float32 all
+// the same, each good to the last bit or two: with the library's functions the gates' kernel took twice as long), and
+// 1 - a^2 = -(e^x - 1), x = 2 log a, by the exponential's series where |x| < 1/2 and from a elsewhere.
+template <typename T> struct LruMath;
+template <> struct LruMath<float> {
+  static __device__ __forceinline__ float sigmoid(float z) { return 1.f / (1.f + expf(-z)); }
+  static __device__ __forceinline__ float exp(float x) { return expf(x); }
+  static __device__ __forceinline__ float root_rest(float log_a, float) { return sqrtf(fmaxf(-expm1f(2.f * log_a), 0.f)); }
+};
+template <> struct LruMath<bf16_t> {
+  static __device__ __forceinline__ float sigmoid(float z) { return __builtin_amdgcn_rcpf(1.f + __expf(-z)); }
+  static __device__ __forceinline__ float exp(float x) { return __expf(x); }
+  static __device__ __forceinline__ float root_rest(float log_a, float a) {
+    const float x = 2.f * log_a;
+    float p = fmaf(x, 1.f / 40320.f, 1.f / 5040.f);
+    p = fmaf(x, p, 1.f / 720.f);
+    p = fmaf(x, p, 1.f / 120.f);
+    p = fmaf(x, p, 1.f / 24.f);
+    p = fmaf(x, p, 1.f / 6.f);
+    p = fmaf(x, p, 0.5f);
+    p = fmaf(x, p, 1.f);
+    const float rest = x > -0.5f ? -x * p : fmaf(-a, a, 1.f);
+    return __builtin_amdgcn_sqrtf(fmaxf(rest, 0.f));
+  }
+};
 
 // the two gates' pre-activations and the channel's input -> a and b
+template <typename T>
 __device__ __forceinline__ void lru_coefficients(float r_pre, float i_pre, float u, float rate, float* a, float* b) {
-  const float log_a = -rate * lru_sigmoid(r_pre);
-  *a = expf(log_a);
-  *b = sqrtf(fmaxf(-expm1f(2.f * log_a), 0.f)) * lru_sigmoid(i_pre) * u;
+  const float log_a = -rate * LruMath<T>::sigmoid(r_pre);
+  *a = LruMath<T>::exp(log_a);
+  *b = LruMath<T>::root_rest(log_a, *a) * LruMath<T>::sigmoid(i_pre) * u;
 }
 
 // Where the coefficients of (token t, channel ch) go: to memory, or (SINGLE) through the token's own state.
@@ -93,7 +118,7 @@ __global__ __launch_bounds__(256) void lru_gates_kernel(const T* __restrict__ u,
     for (int t = 0; t < LRU_TOKENS; ++t)
       if (t < nt) {
         float a, b;
-        lru_coefficients(ar[t] + br[ch], ai[t] + bi[ch], su[t * c + j], rate[ch], &a, &b);
+        lru_coefficients<T>(ar[t] + br[ch], ai[t] + bi[ch], su[t * c + j], rate[ch], &a, &b);
         float* st = SINGLE ? o.state + (long)o.slots[o.seg_of[n0 + t]] * o.state_stride : nullptr;
         lru_store<T, SINGLE>(o, n0 + t, C, ch, st, a, b);
       }
@@ -152,7 +177,7 @@ __global__ __launch_bounds__(256) void lru_gates_mfma_kernel(const bf16_t* __res
                          __uint_as_float(uw.y & 0xffff0000u)};
     float a[4], b[4];
 #pragma unroll
-    for (int j = 0; j < 4; ++j) lru_coefficients(ar[mt][j] + brv[j], ai[mt][j] + biv[j], uv[j], rav[j], &a[j], &b[j]);
+    for (int j = 0; j < 4; ++j) lru_coefficients<bf16_t>(ar[mt][j] + brv[j], ai[mt][j] + biv[j], uv[j], rav[j], &a[j], &b[j]);
     if constexpr (SINGLE) {
       float* st = o.state + (long)o.slots[o.seg_of[tok[mt]]] * o.state_stride;
 #pragma unroll
@@ -160,6 +185,60 @@ __global__ __launch_bounds__(256) void lru_gates_mfma_kernel(const bf16_t* __res
     } else {
       *reinterpret_cast<float4*>(o.a + (long)tok[mt] * C + ch0) = make_float4(a[0], a[1], a[2], a[3]);
       *reinterpret_cast<float4*>(o.b + (long)tok[mt] * C + ch0) = make_float4(b[0], b[1], b[2], b[3]);
+    }
+  }
+}
+
+// For many tokens: the workgroup's 16 MT tokens of the block lie in LDS, read once from memory and by all its waves; wave
+// w takes the outputs 16 w, 16 (w + WAVES), ... of the block. (With every wave fetching u for itself the kernel took 32 us
+// at 2,048 tokens of 2,048 channels in blocks of 256, bound by the trips to the second-level cache.)
+#define LRU_PAD 8             // entries between rows in LDS, so that the 16 rows of a fragment lie in different banks
+template <int MT, int WAVES>
+__global__ __launch_bounds__(WAVES * LMSF_WAVE) void lru_gates_tile_kernel(
+    const bf16_t* __restrict__ u, long u_stride, const bf16_t* __restrict__ Wr, const float* __restrict__ br,
+    const bf16_t* __restrict__ Wi, const float* __restrict__ bi, const float* __restrict__ rate, float* __restrict__ a_out,
+    float* __restrict__ b_out, int n_tokens, int C, int c) {
+  extern __shared__ __align__(16) bf16_t tile[];        // [16 MT][c + LRU_PAD]
+  const int blk = blockIdx.y, n0 = blockIdx.x * (16 * MT), ld = c + LRU_PAD;
+  const int wave = threadIdx.x / LMSF_WAVE, lane = threadIdx.x % LMSF_WAVE, fr = lane % 16, fg = lane / 16;
+  const int per_row = c / 8;
+  for (int i = threadIdx.x; i < 16 * MT * per_row; i += WAVES * LMSF_WAVE) {
+    const int t = i / per_row, k = (i - t * per_row) * 8;
+    *reinterpret_cast<uint4*>(tile + t * ld + k) =
+        *reinterpret_cast<const uint4*>(u + (long)min(n0 + t, n_tokens - 1) * u_stride + (long)blk * c + k);
+  }
+  __syncthreads();
+  for (int j0 = wave * 16; j0 < c; j0 += WAVES * 16) {
+    const long w_at = ((long)blk * c + j0 + fr) * c + fg * 8;
+    f32x4_t ar[MT], ai[MT];
+#pragma unroll
+    for (int mt = 0; mt < MT; ++mt) ar[mt] = ai[mt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+    for (int k = 0; k < c; k += 32) {
+      const bf16x8_t fwr = *reinterpret_cast<const bf16x8_t*>(Wr + w_at + k);
+      const bf16x8_t fwi = *reinterpret_cast<const bf16x8_t*>(Wi + w_at + k);
+#pragma unroll
+      for (int mt = 0; mt < MT; ++mt) {
+        const bf16x8_t fb = *reinterpret_cast<const bf16x8_t*>(tile + (mt * 16 + fr) * ld + k + fg * 8);
+        ar[mt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fwr, fb, ar[mt], 0, 0, 0);
+        ai[mt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fwi, fb, ai[mt], 0, 0, 0);
+      }
+    }
+    const int jl = j0 + fg * 4, ch0 = blk * c + jl;
+    const float4 vbr = *reinterpret_cast<const float4*>(br + ch0), vbi = *reinterpret_cast<const float4*>(bi + ch0);
+    const float4 vra = *reinterpret_cast<const float4*>(rate + ch0);
+#pragma unroll
+    for (int mt = 0; mt < MT; ++mt) {
+      const int t = n0 + mt * 16 + fr;
+      if (t >= n_tokens) continue;
+      const uint2 uw = *reinterpret_cast<const uint2*>(tile + (mt * 16 + fr) * ld + jl);
+      float4 a, b;
+      lru_coefficients<bf16_t>(ar[mt][0] + vbr.x, ai[mt][0] + vbi.x, __uint_as_float(uw.x << 16), vra.x, &a.x, &b.x);
+      lru_coefficients<bf16_t>(ar[mt][1] + vbr.y, ai[mt][1] + vbi.y, __uint_as_float(uw.x & 0xffff0000u), vra.y, &a.y, &b.y);
+      lru_coefficients<bf16_t>(ar[mt][2] + vbr.z, ai[mt][2] + vbi.z, __uint_as_float(uw.y << 16), vra.z, &a.z, &b.z);
+      lru_coefficients<bf16_t>(ar[mt][3] + vbr.w, ai[mt][3] + vbi.w, __uint_as_float(uw.y & 0xffff0000u), vra.w, &a.w, &b.w);
+      *reinterpret_cast<float4*>(a_out + (long)t * C + ch0) = a;
+      *reinterpret_cast<float4*>(b_out + (long)t * C + ch0) = b;
     }
   }
 }
@@ -251,6 +330,7 @@ __global__ __launch_bounds__(64) void lru_fold_kernel(const int* __restrict__ se
 // floats of scratch a chunk takes
 extern "C" long lmsf_linear_recurrence_entry_floats(int C) { return 2L * C; }
 
+#define LRU_TILE_MIN_TOKENS 256
 template <typename T, bool SINGLE>
 static void launch_gates(const void* u, int dtype, long u_stride, const void* Wr, const float* br, const void* Wi,
                          const float* bi, const float* rate, const LruOut<T>& o, int n_tokens, int C, int c,
@@ -259,6 +339,14 @@ static void launch_gates(const void* u, int dtype, long u_stride, const void* Wr
   if constexpr (sizeof(T) == 2) {
     if (c % 32 == 0 && u_stride % 8 == 0 && lmsf_aligned16(u) && lmsf_aligned16(Wr) && lmsf_aligned16(Wi) &&
         lmsf_aligned16(br) && lmsf_aligned16(bi) && lmsf_aligned16(rate) && (SINGLE || (lmsf_aligned16(o.a) && lmsf_aligned16(o.b)))) {
+      if constexpr (!SINGLE) {
+        if (n_tokens >= LRU_TILE_MIN_TOKENS && (size_t)32 * (c + LRU_PAD) * 2 <= 64 * 1024) {
+          hipLaunchKernelGGL((lru_gates_tile_kernel<2, 8>), dim3((n_tokens + 31) / 32, blocks), dim3(8 * LMSF_WAVE),
+                             (size_t)32 * (c + LRU_PAD) * 2, stream, (const bf16_t*)u, u_stride, (const bf16_t*)Wr, br,
+                             (const bf16_t*)Wi, bi, rate, o.a, o.b, n_tokens, C, c);
+          return;
+        }
+      }
       // few tokens: a wave a workgroup, so that the matrices' rows are read by as many compute units as there are
 #define LRU_MFMA(MT, W)                                                                                             \
   hipLaunchKernelGGL((lru_gates_mfma_kernel<MT, SINGLE>), dim3((n_tokens + 16 * MT - 1) / (16 * MT), blocks,        \

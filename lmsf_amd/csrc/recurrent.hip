@@ -52,6 +52,87 @@ __global__ __launch_bounds__(256) void short_conv_kernel(const T* __restrict__ u
   out[(long)t * out_stride + c] = from_f32<T>(acc);
 }
 
+// The same for portions of prompts: a thread takes two neighbouring channels of SC_TT tokens one after the other and keeps
+// their last inputs in registers, so that an input is read once and the filters once a thread. A token that begins a
+// segment takes its history from that segment's state.
+#define SC_TT 16
+template <typename T> struct Sc2;
+template <> struct Sc2<float> {
+  static __device__ __forceinline__ float2 load(const float* p) { return *reinterpret_cast<const float2*>(p); }
+  static __device__ __forceinline__ void store(float* p, float x, float y) { *reinterpret_cast<float2*>(p) = make_float2(x, y); }
+};
+template <> struct Sc2<bf16_t> {
+  static __device__ __forceinline__ float2 load(const bf16_t* p) {
+    const uint32_t v = *reinterpret_cast<const uint32_t*>(p);
+    return make_float2(__uint_as_float(v << 16), __uint_as_float(v & 0xffff0000u));
+  }
+  static __device__ __forceinline__ void store(bf16_t* p, float x, float y) { *reinterpret_cast<uint32_t*>(p) = pack2_bf16(x, y); }
+};
+template <typename T, int ACT, int TAPS>
+__global__ __launch_bounds__(256) void short_conv_tile_kernel(const T* __restrict__ u, long u_stride, const T* __restrict__ w,
+                                                              const T* __restrict__ bias, const float* __restrict__ state,
+                                                              long state_stride, const int* __restrict__ seg_of,
+                                                              const int* __restrict__ seg_starts,
+                                                              const int* __restrict__ state_slots, T* __restrict__ out,
+                                                              long out_stride, int n_tokens, int C) {
+  const int c = (blockIdx.y * 256 + threadIdx.x) * 2;
+  if (c >= C) return;
+  const int t0 = blockIdx.x * SC_TT, nt = min(SC_TT, n_tokens - t0);
+  float2 in[SC_TT];
+#pragma unroll
+  for (int i = 0; i < SC_TT; ++i) in[i] = Sc2<T>::load(u + (long)(t0 + min(i, nt - 1)) * u_stride + c);
+  float wx[TAPS], wy[TAPS];
+#pragma unroll
+  for (int j = 0; j < TAPS; ++j) {
+    wx[j] = to_f32<T>(w[(long)c * TAPS + j]);
+    wy[j] = to_f32<T>(w[(long)(c + 1) * TAPS + j]);
+  }
+  const float2 b0 = bias ? Sc2<T>::load(bias + c) : make_float2(0.f, 0.f);
+  float2 h[TAPS];                          // h[j]: the input TAPS - 1 - j tokens before the current one; h[TAPS - 1] itself
+  int s = seg_of[t0];
+  auto history = [&](int t) {              // h[0 .. TAPS - 2] before token t of segment s
+    const int start = seg_starts[s];
+    const float* st = state + (long)state_slots[s] * state_stride + (long)c * (TAPS - 1);
+#pragma unroll
+    for (int j = 0; j < TAPS - 1; ++j) {
+      const int src = t - (TAPS - 1) + j;
+      if (src >= start) {
+        h[j + 1] = Sc2<T>::load(u + (long)src * u_stride + c);
+      } else {
+        h[j + 1].x = st[(TAPS - 1) + (src - start)];
+        h[j + 1].y = st[2 * (TAPS - 1) + (src - start)];
+      }
+    }
+  };
+  history(t0);
+#pragma unroll
+  for (int i = 0; i < SC_TT; ++i) {
+    if (i < nt) {
+      if (i > 0) {
+        const int si = seg_of[t0 + i];
+        if (si != s) {
+          s = si;
+          history(t0 + i);
+        }
+      }
+#pragma unroll
+      for (int j = 0; j < TAPS - 1; ++j) h[j] = h[j + 1];
+      h[TAPS - 1] = in[i];
+      float x = b0.x, y = b0.y;
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) {
+        x = fmaf(wx[j], h[j].x, x);
+        y = fmaf(wy[j], h[j].y, y);
+      }
+      if (ACT == 1) {
+        x = x / (1.f + expf(-x));
+        y = y / (1.f + expf(-y));
+      }
+      Sc2<T>::store(out + (long)(t0 + i) * out_stride + c, x, y);
+    }
+  }
+}
+
 // state[c, h] <- the input taps - 1 - h tokens before the segment's end: of this step where the segment is long
 // enough, else what the state held that many tokens further on (read before it is overwritten: h rises).
 template <typename T>
@@ -87,16 +168,35 @@ extern "C" int lmsf_short_conv(const void* u, int dtype, long u_stride, const vo
   dim3 grid(n_tokens, (C + 255) / 256), sgrid(n_segments, (C + 255) / 256), block(256);
   // (a form with 16-byte accesses, a thread 8 neighbouring channels of a token, measured slower at 2,048 tokens of 4,096
   // channels, 74 against 60 us, and at 8 tokens, 10.7 against 3.8: its weights' loads lie 64 bytes apart across a wave)
+  const bool pairs = !single && taps >= 2 && taps <= 5 && n_tokens >= SC_TT && C % 2 == 0 && u_stride % 2 == 0 &&
+                     out_stride % 2 == 0 && ((uintptr_t)u & 7) == 0 && ((uintptr_t)out & 7) == 0 && (!bias || ((uintptr_t)bias & 7) == 0);
+#define SC_TILE(T, A, N)                                                                                             \
+  hipLaunchKernelGGL((short_conv_tile_kernel<T, A, N>), dim3((n_tokens + SC_TT - 1) / SC_TT, (C / 2 + 255) / 256), block, \
+                     0, stream, (const T*)u, u_stride, (const T*)w, (const T*)bias, state, state_stride, seg_of,      \
+                     seg_starts, state_slots, (T*)out, out_stride, n_tokens, C)
+#define SC_TAPS(T, A)                                                                                                \
+  do {                                                                                                               \
+    if (taps == 2) SC_TILE(T, A, 2); else if (taps == 3) SC_TILE(T, A, 3); else if (taps == 4) SC_TILE(T, A, 4);     \
+    else SC_TILE(T, A, 5);                                                                                           \
+  } while (0)
 #define SC(T, A)                                                                                                      \
   hipLaunchKernelGGL((short_conv_kernel<T, A>), grid, block, 0, stream, (const T*)u, u_stride, (const T*)w,           \
                      (const T*)bias, state, state_stride, seg_of, seg_starts, state_slots, (T*)out, out_stride, C, taps, \
                      single)
-  if (dtype == LMSF_F32) {
+  if (pairs) {
+    if (dtype == LMSF_F32) {
+      if (act) SC_TAPS(float, 1); else SC_TAPS(float, 0);
+    } else {
+      if (act) SC_TAPS(bf16_t, 1); else SC_TAPS(bf16_t, 0);
+    }
+  } else if (dtype == LMSF_F32) {
     if (act) SC(float, 1); else SC(float, 0);
   } else {
     if (act) SC(bf16_t, 1); else SC(bf16_t, 0);
   }
 #undef SC
+#undef SC_TAPS
+#undef SC_TILE
   LMSF_LAUNCH_CHECK("short_conv");
   if (taps > 1 && !single) {
     if (dtype == LMSF_F32)

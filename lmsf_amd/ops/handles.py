@@ -85,3 +85,31 @@ class ScaledRows:
     @property
     def device(self) -> torch.device:
         return self.xw.device
+
+
+class NormedPair:
+    """The mean of two mixers' outputs, each over its root mean square and times a weight, not joined yet:
+    ``scale`` * (a / rms(a) * wa + b / rms(b) * wb), a and b [N, W] in the run's type. ``HipOps.norm_add`` joins them on
+    the way into the stream; ``HipOps.materialize`` makes the tensor (``rms_pair``)."""
+
+    __slots__ = ("a", "b", "wa", "wb", "eps", "scale")
+
+    def __init__(self, a: torch.Tensor, b: torch.Tensor, wa: torch.Tensor, wb: torch.Tensor, eps: float, scale: float):
+        self.a = a
+        self.b = b
+        self.wa = wa
+        self.wb = wb
+        self.eps = eps
+        self.scale = scale
+
+    @property
+    def shape(self) -> Tuple[int, int]:
+        return tuple(self.a.shape)
+
+    @property
+    def dtype(self) -> torch.dtype:
+        return self.a.dtype
+
+    @property
+    def device(self) -> torch.device:
+        return self.a.device

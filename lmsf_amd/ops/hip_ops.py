@@ -12,7 +12,7 @@ import torch
 
 from . import dispatch as D
 from . import library
-from .handles import DeferredLinear, PendingProduct, ScaledRows
+from .handles import DeferredLinear, NormedPair, PendingProduct, ScaledRows
 
 F32 = 0
 BF16 = 1
@@ -275,7 +275,9 @@ class HipOps:
 
     def materialize(self, y):
         """The tensor behind ``y``: ``y`` itself, the finished sum of a ``PendingProduct``, the product of a
-        ``DeferredLinear`` or the norm of a ``ScaledRows``."""
+        ``DeferredLinear``, the norm of a ``ScaledRows`` or the mean of a ``NormedPair``."""
+        if isinstance(y, NormedPair):
+            return self.rms_pair(y.a, y.b, y.wa, y.wb, y.eps, y.scale)
         if isinstance(y, DeferredLinear):
             return self.linear(y.x, y.weight, y.bias, out_dtype=y.dtype)
         if isinstance(y, ScaledRows):
@@ -644,6 +646,35 @@ class HipOps:
             _ptr(residual), _ptr(history), hist_stride, int(index), _ptr(mix), _ptr(out_weight), _ptr(out),
             _code(out.dtype) if out is not None else F32, W, _ptr(rows), n_out, W, int(groups), float(x_eps),
             float(out_eps), self._stream()))
+        return out
+
+    def norm_add(self, branch, weight: torch.Tensor, eps: float, residual: torch.Tensor,
+                 want_out: bool = True) -> Optional[torch.Tensor]:
+        """residual += branch / rms(branch) * weight, float32 and in place; with ``want_out`` returns the new stream in the
+        branch's dtype. ``branch`` [N, W] with unit column stride, or a ``NormedPair`` (joined in the same launch);
+        ``weight`` float32 [W], ``residual`` contiguous float32 [N, W]."""
+        pair = branch if isinstance(branch, NormedPair) else None
+        a, b = (pair.a, pair.b) if pair is not None else (branch, None)
+        self._dev(a, b, weight, residual)
+        N, W = a.shape
+        views = [t for t in (a, b) if t is not None]
+        if residual.dtype != torch.float32 or not residual.is_contiguous() or tuple(residual.shape) != (N, W) \
+                or any(t.stride(1) != 1 or t.dtype != a.dtype or tuple(t.shape) != (N, W) for t in views):
+            raise ValueError("norm_add: the branch must be [N, W] with unit column stride, the stream contiguous float32")
+        self._f32_vec(weight, W, "norm_add: weight")
+        if not self.lib.lmsf_norm_add_fits(W) or any(t.stride(0) % 4 or t.data_ptr() % 16 for t in views) \
+                or residual.data_ptr() % 16:
+            x = self.materialize(pair) if pair is not None else a
+            return self.group_norm(x=x, x_weight=weight, residual=residual, x_eps=eps, out_dtype=a.dtype, want_out=want_out)
+        if pair is not None:
+            self._f32_vec(pair.wa, W, "norm_add: first weight of the pair")
+            self._f32_vec(pair.wb, W, "norm_add: second weight of the pair")
+        out = torch.empty((N, W), dtype=a.dtype, device=a.device) if want_out else None
+        self._check(self.lib.lmsf_norm_add(
+            _ptr(a), a.stride(0), _ptr(b), b.stride(0) if b is not None else 0, _code(a.dtype),
+            _ptr(pair.wa) if pair is not None else None, _ptr(pair.wb) if pair is not None else None,
+            float(pair.eps) if pair is not None else 0.0, float(pair.scale) if pair is not None else 1.0, _ptr(weight),
+            float(eps), _ptr(residual), _ptr(out), N, W, self._stream()))
         return out
 
     def latent_cache_write(self, x: torch.Tensor, weight: torch.Tensor, eps: float, rank: int, rot_width: int,

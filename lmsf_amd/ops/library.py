@@ -75,6 +75,9 @@ _SIGNATURES = {
     "lmsf_moe_route_groups": (c_int, [_P, c_long, c_int, c_int, c_int, c_int, c_int, c_int, c_int, _P, _P, _P]),
     "lmsf_group_norm": (c_int, [_P, c_int, c_long, _P, _P, _P, c_long, c_int, _P, _P, _P, c_int, c_long, _P, c_int, c_int,
                                 c_int, c_float, c_float, _P]),
+    "lmsf_norm_add_fits": (c_int, [c_int]),
+    "lmsf_norm_add": (c_int, [_P, c_long, _P, c_long, c_int, _P, _P, c_float, c_float, _P, c_float, _P, _P, c_int, c_int,
+                              _P]),
     "lmsf_latent_cache_write": (c_int, [_P, c_int, c_long, _P, c_float, _P, _P, c_int, c_int, _P, _P, _P, c_long, c_int,
                                         c_int, c_int, c_int, c_int, _P, _P, _P, c_long, c_int, _P]),
     "lmsf_head_linear": (c_int, [_P, c_int, c_long, c_int, _P, _P, c_long, c_int, _P, c_long, c_int, c_int, c_int, c_int,

@@ -360,7 +360,8 @@ class OutputNormBlock(Block):
         x += norm_a(mixer(x));   x += norm_b(ffn(x))
 
     (without a feed-forward only the first). The stream is float32; a sublayer gets it rounded to the run's type. Every
-    addition with its norm is one kernel, which also hands on the new stream in the run's type: to the feed-forward, or
+    addition with its norm is one kernel (``norm_add``; a mixer that is a pair of mixers leaves their joining to it), which
+    also hands on the new stream in the run's type: to the feed-forward, or
     in ``ctx.aux["stream_rounded"]`` to the block that always follows (``link_next``). Nothing is left to add when the
     block returns. The reference's only arrangement is the pre-norm one
     (core/src/model_executor/models/llama/llama.rs:286-340)."""
@@ -381,8 +382,10 @@ class OutputNormBlock(Block):
     def link_next(self, following: Block) -> None:
         self.hands_on = isinstance(following, OutputNormBlock)
 
-    def _add(self, norm, branch: torch.Tensor, residual: torch.Tensor, want: bool) -> Optional[torch.Tensor]:
+    def _add(self, norm, branch, residual: torch.Tensor, want: bool) -> Optional[torch.Tensor]:
         """stream += norm(branch); with ``want`` the new stream in the run's type."""
+        if norm.groups == 1:
+            return self.rt.ops.norm_add(branch, norm.weight, norm.eps, residual, want_out=want)
         # (no weight behind the sum: the kernel hands back the new stream itself)
         return self.rt.ops.group_norm(x=branch, x_weight=norm.weight, residual=residual, groups=norm.groups,
                                       x_eps=norm.eps, out_dtype=self.rt.dtype, want_out=want)
@@ -393,8 +396,12 @@ class OutputNormBlock(Block):
         x = ctx.aux.pop("stream_rounded", None)
         if x is None:
             x = self.rt.ops.group_norm(residual=residual, out_dtype=self.rt.dtype)
-        a = self.mixer.forward(x, ctx, binding)
-        x = self._add(self.norms["post_mixer"], a, residual, self.has_ffn or self.hands_on)
+        post = self.norms["post_mixer"]
+        if getattr(self.mixer, "may_return_pair", False) and post.groups == 1:
+            a = self.mixer.forward(x, ctx, binding, pair_ok=True)
+        else:
+            a = self.mixer.forward(x, ctx, binding)
+        x = self._add(post, a, residual, self.has_ffn or self.hands_on)
         if self.has_ffn:
             f = self.feed_forward.forward(x, token_ids=ctx.token_ids) if self._ffn_takes_ids else self.feed_forward.forward(x)
             x = self._add(self.norms["post_ffn"], f, residual, self.hands_on)

@@ -9,6 +9,7 @@ from typing import Callable, Dict, Optional
 
 import torch
 
+from ..ops.handles import NormedPair
 from .base import CacheBinding, CacheSpec, Mixer, PartSpec, Runtime, StateSpec, build_part, register_part
 from .recurrent import FloatVector
 
@@ -52,7 +53,12 @@ class ParallelPair(Mixer):
                             writes_cache=binding.writes_cache,
                             state=binding.state[:, a:a + n] if n and binding.state is not None else None)
 
-    def forward(self, h: torch.Tensor, ctx, binding: CacheBinding) -> torch.Tensor:
+    # ``forward(..., pair_ok=True)`` may leave the joining to whoever takes the result (ops.handles.NormedPair)
+    may_return_pair = True
+
+    def forward(self, h: torch.Tensor, ctx, binding: CacheBinding, pair_ok: bool = False):
         a = self.left.forward(h, ctx, self._child_binding(binding, 0))
         b = self.right.forward(h, ctx, self._child_binding(binding, 1))
+        if pair_ok:
+            return NormedPair(a, b, self.left_out.weight, self.right_out.weight, self.eps, self.scale)
         return self.rt.ops.rms_pair(a, b, self.left_out.weight, self.right_out.weight, self.eps, self.scale)

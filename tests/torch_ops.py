@@ -13,6 +13,8 @@ import math
 import numpy as np
 import torch
 
+from lmsf_amd.ops.handles import NormedPair
+
 
 # ---------------------------------------------------------------- counter-based noise (same as sampling.hip)
 
@@ -488,6 +490,15 @@ class TorchOps:
                 y[t] = ((S @ Cc + d_skip * xt) * (zt / (1.0 + torch.exp(-zt)))).to(x.dtype)
             state[slot, :inner * n] = S.reshape(-1)
         return y
+
+    def norm_add(self, branch, weight, eps, residual, want_out=True):
+        if isinstance(branch, NormedPair):
+            x = branch.scale * (self._gn(branch.a.to(torch.float32), branch.wa, 1, branch.eps)
+                                + self._gn(branch.b.to(torch.float32), branch.wb, 1, branch.eps))
+        else:
+            x = branch.to(torch.float32)
+        residual += self._gn(x, weight, 1, eps)
+        return residual.to(branch.dtype) if want_out else None
 
     def linear_recurrence(self, u, wr, br, wi, bi, rate, y, state, batch):
         N, C = u.shape
