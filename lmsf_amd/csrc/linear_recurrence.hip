@@ -190,8 +190,8 @@ __global__ __launch_bounds__(256) void lru_gates_mfma_kernel(const bf16_t* __res
 }
 
 // For many tokens: the workgroup's 16 MT tokens of the block lie in LDS, read once from memory and by all its waves; wave
-// w takes the outputs 16 w, 16 (w + WAVES), ... of the block. (With every wave fetching u for itself the kernel took 32 us
-// at 2,048 tokens of 2,048 channels in blocks of 256, bound by the trips to the second-level cache.)
+// w takes the outputs 16 w, 16 (w + WAVES), ... of the block. (With every wave fetching u for itself 30 us at
+// 2,048 tokens of 2,048 channels in blocks of 256.)
 #define LRU_PAD 8             // entries between rows in LDS, so that the 16 rows of a fragment lie in different banks
 template <int MT, int WAVES>
 __global__ __launch_bounds__(WAVES * LMSF_WAVE) void lru_gates_tile_kernel(
@@ -340,12 +340,22 @@ static void launch_gates(const void* u, int dtype, long u_stride, const void* Wr
     if (c % 32 == 0 && u_stride % 8 == 0 && lmsf_aligned16(u) && lmsf_aligned16(Wr) && lmsf_aligned16(Wi) &&
         lmsf_aligned16(br) && lmsf_aligned16(bi) && lmsf_aligned16(rate) && (SINGLE || (lmsf_aligned16(o.a) && lmsf_aligned16(o.b)))) {
       if constexpr (!SINGLE) {
-        if (n_tokens >= LRU_TILE_MIN_TOKENS && (size_t)32 * (c + LRU_PAD) * 2 <= 64 * 1024) {
-          hipLaunchKernelGGL((lru_gates_tile_kernel<2, 8>), dim3((n_tokens + 31) / 32, blocks), dim3(8 * LMSF_WAVE),
-                             (size_t)32 * (c + LRU_PAD) * 2, stream, (const bf16_t*)u, u_stride, (const bf16_t*)Wr, br,
-                             (const bf16_t*)Wi, bi, rate, o.a, o.b, n_tokens, C, c);
+#define LRU_TILE(MT)                                                                                                \
+  hipLaunchKernelGGL((lru_gates_tile_kernel<MT, 8>), dim3((n_tokens + 16 * MT - 1) / (16 * MT), blocks),             \
+                     dim3(8 * LMSF_WAVE), (size_t)16 * MT * (c + LRU_PAD) * 2, stream, (const bf16_t*)u, u_stride,   \
+                     (const bf16_t*)Wr, br, (const bf16_t*)Wi, bi, rate, o.a, o.b, n_tokens, C, c)
+        // 64 tokens a workgroup where that still fills the chip (the matrices are read once a workgroup: 2,048 tokens of
+        // 2,048 channels in blocks of 256 20 us against 25 with 32 tokens and 38 with 16), else 32
+        const size_t row = (size_t)(c + LRU_PAD) * 2;
+        if (n_tokens >= LRU_TILE_MIN_TOKENS && 64 * row <= 64 * 1024 && (long)((n_tokens + 63) / 64) * blocks >= lmsf_compute_units()) {
+          LRU_TILE(4);
           return;
         }
+        if (n_tokens >= LRU_TILE_MIN_TOKENS && 32 * row <= 64 * 1024) {
+          LRU_TILE(2);
+          return;
+        }
+#undef LRU_TILE
       }
       // few tokens: a wave a workgroup, so that the matrices' rows are read by as many compute units as there are
 #define LRU_MFMA(MT, W)                                                                                             \
