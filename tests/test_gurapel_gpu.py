@@ -232,6 +232,62 @@ def test_every_head_of_queries_and_keys_normed_with_a_weight(dtype, rot, H, G, d
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("N,W", [(1, 48), (3, 50), (7, 2048), (600, 96), (530, 4100), (5, 4100), (2, 12288), (1, 12290), (513, 2048)])
+def test_a_sublayers_output_and_a_pairs_join_the_stream(dtype, N, W):
+    """stream += norm(v), v a mixer's output or the mean of a pair's, each normed: widths that a workgroup holds in
+    registers and widths that go the other way, one row and many, rows at a stride."""
+    from lmsf_amd.ops.handles import NormedPair
+    o = ops()
+    g = torch.Generator().manual_seed(W)
+    a, b = [(torch.randn((N, W + 8), generator=g) * s).to(dtype) for s in (3.0, 0.1)]
+    wa, wb, wn = [1 + 0.3 * torch.randn((W,), generator=g) for _ in range(3)]
+    x0 = torch.randn((N, W), generator=g) * 2
+    va, vb = a[:, :W].double(), b[:, :W].double()
+    mean = 0.5 * (P.rms(va, 1e-5) * wa.double() + P.rms(vb, 1e-5) * wb.double())
+    ac, bc = a.cuda()[:, :W], b.cuda()[:, :W]
+    for v, branch in ((va, ac), (mean, NormedPair(ac, bc, wa.cuda(), wb.cuda(), 1e-5, 0.5))):
+        want = x0.double() + P.rms(v, 1e-6) * wn.double()
+        for want_out in (True, False):
+            x = x0.cuda()
+            out = o.norm_add(branch, wn.cuda(), 1e-6, x, want_out=want_out)
+            # (a pair that goes the other way is rounded to the run's type in between)
+            close(x, want, dtype if W % 4 else torch.float32)
+            if want_out:
+                assert torch.equal(out, x.to(dtype))
+            else:
+                assert out is None
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("C,taps,act", [(24, 2, None), (130, 3, "silu"), (514, 4, None), (600, 5, "silu"), (33, 4, "silu"),
+                                        (40, 6, None)])
+def test_the_short_convolution_across_segments_of_every_length(dtype, C, taps, act):
+    """Segments shorter than the filter, single tokens between longer ones, borders inside and on the edges of the tiles
+    of tokens that a thread walks, states that an earlier step left."""
+    o = ops()
+    g = torch.Generator().manual_seed(C)
+    lens = [1, 2, 1, 3, 40, 1, 17, 16, 5, 9]
+    slots = [7, 0, 3, 11, 2, 9, 4, 1, 8, 5]
+    N = sum(lens)
+    u = torch.randn((N, C + 6), generator=g).to(dtype)
+    w = (torch.randn((C, taps), generator=g) * 0.6).to(dtype)
+    bias = torch.randn((C,), generator=g).to(dtype)
+    state0 = torch.randn((12, C * (taps - 1) + 3), generator=g)
+    want, after, at = [], state0.clone(), 0
+    for n, slot in zip(lens, slots):
+        old = state0[slot, :C * (taps - 1)].reshape(C, taps - 1).t().double()
+        seq = torch.cat([old, u[at:at + n, :C].double()], 0)
+        y = P.short_conv(seq, w.double(), bias.double())[taps - 1:]
+        want.append(P.silu(y) if act else y)
+        after[slot, :C * (taps - 1)] = seq[-(taps - 1):].t().reshape(-1).float()
+        at += n
+    state = state0.cuda()
+    got = o.short_conv(u.cuda()[:, :C], w.cuda(), bias.cuda(), state, batch_of(lens, slots), act)
+    close(got, torch.cat(want), dtype)
+    assert torch.equal(state.cpu(), after)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
 def test_the_embedding_adds_the_positions_vector(dtype):
     g = torch.Generator().manual_seed(2)
     V, W, n = 29, 44, 50
@@ -281,6 +337,27 @@ def test_every_kind_of_layer_alone(tmp_path, which, index, dtype):
     core = load_engine_core(folder, dtype=dtype, block_size=8, num_pages=16, max_model_len=128, max_num_seqs=2)
     got = replay(core.executor, StepEntry, {"a": toks}, [[("a", c)] for c in (37, 2, 30, 1, 1, 1, 18)])["a"]
     check(got, plain_logits(cfg, w, toks), dtype, (which, index), (cfg, w, toks))
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("W,lay", [(50, pair(3, 1, 24, 300, 21, 30, 2, 3, mlp=moe(3, 2, 14))),
+                                   (46, pair(2, 2, 272, 33, 40, 28, 7, 2)), (54, delta(2, 1, 250, 7, 3, mlp=moe(4, 4, 6))),
+                                   (64, pair(20, 1, 32, 48, 77, 64, 1, 4, mlp=moe(96, 5, 8)))])
+def test_sizes_that_the_fast_kernels_do_not_take(tmp_path, W, lay, dtype):
+    """Heads wider than the matrix cores' attention takes, widths that are multiples of two only, more query heads a key
+    head than a workgroup's block, many experts."""
+    from lmsf_amd.engine import StepEntry, load_engine_core
+    folder, cfg, w = make_model(tmp_path, model(59, W, [lay], positions=200), 8)
+    toks = random_tokens(90, cfg["vocab"], 3)
+    core = load_engine_core(folder, dtype=dtype, block_size=16, num_pages=8, max_model_len=128, max_num_seqs=2)
+    got = replay(core.executor, StepEntry, {"a": toks}, [[("a", c)] for c in (41, 2, 30, 1, 1, 15)])["a"]
+    ref = plain_logits(cfg, w, toks)
+    if dtype == "float32":
+        check(got, ref, dtype, W, (cfg, w, toks))
+    else:
+        # (a router's close call may flip an expert in a few rows)
+        from gurapel_helpers import row_errs
+        assert (row_errs(got, ref) <= bfloat16_limits(cfg, w, toks, ref)).double().mean() > 0.9
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
