@@ -30,7 +30,7 @@ __global__ __launch_bounds__(GEN_THREADS) void paged_attention_generic_kernel(
     const T* __restrict__ q, long q_stride, T* __restrict__ out, long out_stride, const T* __restrict__ k_pages,
     const T* __restrict__ v_pages, const int* __restrict__ block_tables, int bt_width, const int* __restrict__ seg,
     const int* __restrict__ pos, int nh, int nkv, int d, int ps, float scale, int window, float softcap,
-    const float* __restrict__ bias) {
+    const float* __restrict__ bias, const float* __restrict__ sink) {
   extern __shared__ float smem[];
   float* sq = smem;                       // [d] query, pre-scaled
   float* sp = sq + d;                     // [256] scores, then probabilities
@@ -52,7 +52,8 @@ __global__ __launch_bounds__(GEN_THREADS) void paged_attention_generic_kernel(
   const int ngroups = GEN_THREADS / d > 0 ? GEN_THREADS / d : 1;
   const int og = tid / d, oi = tid % d;                            // (key group, output dim) of this thread
   const bool pv_active = og < ngroups;
-  float acc = 0.f, m = -INFINITY, l = 0.f;
+  // (a sink: exp(sink_h) stands in the denominator beside the keys' exponentials, so the online softmax begins with it)
+  float acc = 0.f, m = sink ? sink[h] : -INFINITY, l = sink ? 1.f : 0.f;
   float wide[3] = {0.f, 0.f, 0.f};                                 // output dims tid + 256, + 512, + 768 (d > 256)
   __syncthreads();
 
@@ -119,13 +120,13 @@ __global__ __launch_bounds__(GEN_THREADS) void paged_attention_generic_kernel(
 
 // ``softcap`` c > 0: a score s (after the scale) becomes c tanh(s / c) before the softmax; 0: scores as they are.
 // ``bias`` float32 [2, nh] or null: r1_h ln(1 + r2_h (i - j)) comes off the score of query i and key j (r2 >= 0),
-// after the cap.
+// after the cap. ``sink`` float32 [nh] or null: exp(sink_h) stands in head h's denominator.
 extern "C" int lmsf_paged_attention_generic_biased(const void* q, long q_stride, void* out, long out_stride,
                                                    const void* k_pages, const void* v_pages, long num_pages,
                                                    const int* block_tables, int bt_width, const int* seg,
                                                    const int* pos, int n_tokens, int nh, int nkv, int d, int ps,
-                                                   float scale, int window, float softcap, const float* bias, int dtype,
-                                                   hipStream_t stream) {
+                                                   float scale, int window, float softcap, const float* bias, const float* sink,
+                                                   int dtype, hipStream_t stream) {
   LMSF_CHECK(softcap >= 0.f, "paged_attention: the soft cap must be >= 0, got %g", (double)softcap);
   LMSF_CHECK(q && out && k_pages && v_pages && block_tables && seg && pos, "paged_attention: null pointer");
   LMSF_CHECK(dtype == LMSF_F32 || dtype == LMSF_BF16, "paged_attention: unknown dtype code %d", dtype);
@@ -141,11 +142,11 @@ extern "C" int lmsf_paged_attention_generic_biased(const void* q, long q_stride,
   if (dtype == LMSF_F32)
     hipLaunchKernelGGL((paged_attention_generic_kernel<float>), grid, block, smem, stream, (const float*)q, q_stride,
                        (float*)out, out_stride, (const float*)k_pages, (const float*)v_pages, block_tables, bt_width,
-                       seg, pos, nh, nkv, d, ps, scale, window, softcap, bias);
+                       seg, pos, nh, nkv, d, ps, scale, window, softcap, bias, sink);
   else
     hipLaunchKernelGGL((paged_attention_generic_kernel<bf16_t>), grid, block, smem, stream, (const bf16_t*)q, q_stride,
                        (bf16_t*)out, out_stride, (const bf16_t*)k_pages, (const bf16_t*)v_pages, block_tables,
-                       bt_width, seg, pos, nh, nkv, d, ps, scale, window, softcap, bias);
+                       bt_width, seg, pos, nh, nkv, d, ps, scale, window, softcap, bias, sink);
   LMSF_LAUNCH_CHECK("paged_attention_generic");
   return 0;
 }
@@ -157,5 +158,5 @@ extern "C" int lmsf_paged_attention_generic(const void* q, long q_stride, void* 
                                             int dtype, hipStream_t stream) {
   return lmsf_paged_attention_generic_biased(q, q_stride, out, out_stride, k_pages, v_pages, num_pages, block_tables,
                                              bt_width, seg, pos, n_tokens, nh, nkv, d, ps, scale, window, 0.f, nullptr,
-                                             dtype, stream);
+                                             nullptr, dtype, stream);
 }

@@ -126,6 +126,13 @@ struct DistanceBias {
   __device__ __forceinline__ float off(int diff) const { return b1 * __builtin_amdgcn_logf(fmaf(r2, (float)max(diff, 0), 1.f)); }
 };
 
+// A sink: a number a head whose exponential stands in the softmax's denominator beside the keys', without key or value,
+// not scaled, capped or biased. The online softmax begins with it: the running maximum is the sink (in log2 units) and
+// the sum is 1, counted by one of the four lanes that hold a row. Without sinks: nothing seen yet.
+__device__ __forceinline__ float sink_start(const float* __restrict__ sink, int head) {
+  return sink ? sink[head] * 1.44269504088896340736f : -INFINITY;
+}
+
 // One workgroup of 4 waves per (tile, kv head, block of HB heads of its group). Wave w owns the rows
 // (w * NQB + j) * 16 + c, j < NQB, c = lane % 16; row r is token r / HB of the tile and head r % HB of
 // the block. tiles[2 i], tiles[2 i + 1]: first flat token and number of tokens of tile i.
@@ -134,7 +141,8 @@ __global__ __launch_bounds__(256) void attn_prefill_mfma_kernel(
     const bf16_t* __restrict__ q, long q_stride, bf16_t* __restrict__ out, long out_stride,
     const bf16_t* __restrict__ k_pages, const bf16_t* __restrict__ v_pages, const int* __restrict__ block_tables,
     int btw, const int* __restrict__ tiles, const int* __restrict__ seg, const int* __restrict__ pos, int nh, int nkv,
-    int d, int ps, float scale_log2, float cap_raw, int window, int HB, int n_hb, const float* __restrict__ bias) {
+    int d, int ps, float scale_log2, float cap_raw, int window, int HB, int n_hb, const float* __restrict__ bias,
+    const float* __restrict__ sink) {
   constexpr int DS = DPAD / 32, DV = DPAD / 16;
   const int tile = blockIdx.x;
   const int kvh = blockIdx.y / n_hb, hb = blockIdx.y - kvh * n_hb;
@@ -145,7 +153,7 @@ __global__ __launch_bounds__(256) void attn_prefill_mfma_kernel(
   G.k = k_pages; G.v = v_pages; G.btw = btw; G.nkv = nkv; G.d = d; G.ps = ps; G.kvh = kvh;
   G.bt = block_tables + (long)seg[t0] * btw;
 
-  int rpos[NQB], rlo[NQB];
+  int rpos[NQB], rlo[NQB], rhead[NQB];
   DistanceBias db[NQB];
   long qoff[NQB], ooff[NQB];
   int wmax = -1, wlo = INT_MAX;
@@ -159,6 +167,7 @@ __global__ __launch_bounds__(256) void attn_prefill_mfma_kernel(
     rpos[j] = p;
     rlo[j] = p >= 0 ? first_visible_key(p, window) : 0;
     const int head = kvh * n_rep + (valid ? hin : 0);
+    rhead[j] = head;
     if constexpr (BIAS) db[j].load(bias, nh, head, scale_log2);
     qoff[j] = (long)tok * q_stride + (long)head * d;
     ooff[j] = (long)tok * out_stride + (long)head * d;
@@ -185,8 +194,8 @@ __global__ __launch_bounds__(256) void attn_prefill_mfma_kernel(
   float m[NQB], lsum[NQB];
 #pragma unroll
   for (int j = 0; j < NQB; ++j) {
-    m[j] = -INFINITY;
-    lsum[j] = 0.f;
+    m[j] = sink_start(sink, rhead[j]);
+    lsum[j] = sink && g == 0 ? 1.f : 0.f;
 #pragma unroll
     for (int v = 0; v < DV; ++v) acc[v][j] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
   }
@@ -374,7 +383,7 @@ __global__ __launch_bounds__(NW * 64, (NW == 8 ? 4 : 1)) void attn_prefill_dma_k
     const bf16_t* __restrict__ k_pages, const bf16_t* __restrict__ v_pages, const int* __restrict__ block_tables,
     int btw, const int* __restrict__ tiles, const int* __restrict__ seg, const int* __restrict__ pos, int nh, int nkv,
     int d, int ps_log2, float scale_log2, float cap_raw, int window, int HB, int n_hb, int bt_cap, int n_cus,
-    const float* __restrict__ bias) {
+    const float* __restrict__ bias, const float* __restrict__ sink) {
   constexpr int DS = DPAD / 32, DV = DPAD / 16;
   constexpr int PR = DPAD / 8;                   // 16-byte pieces per K row
   constexpr bool PR_POW2 = (PR & (PR - 1)) == 0;
@@ -414,7 +423,7 @@ __global__ __launch_bounds__(NW * 64, (NW == 8 ? 4 : 1)) void attn_prefill_dma_k
   int wbase = 0;
   for (int i = tid; i < min(n_blk, bt_cap) + PREFILL_BT_PAD; i += NW * 64) lds_bt[i] = bt[blk0 + min(i, n_blk - 1)];
 
-  int rpos[NQB], rlo[NQB];
+  int rpos[NQB], rlo[NQB], rhead[NQB];
   DistanceBias db[NQB];
   long qoff[NQB], ooff[NQB];
   int wmax = -1, wlo = INT_MAX, wminpos = INT_MAX, wmaxlo = 0;
@@ -428,6 +437,7 @@ __global__ __launch_bounds__(NW * 64, (NW == 8 ? 4 : 1)) void attn_prefill_dma_k
     rpos[j] = p;
     rlo[j] = p >= 0 ? first_visible_key(p, window) : 0;
     const int head = kvh * n_rep + (valid ? hin : 0);
+    rhead[j] = head;
     if constexpr (BIAS) db[j].load(bias, nh, head, scale_log2);
     qoff[j] = (long)tok * q_stride + (long)head * d;
     ooff[j] = (long)tok * out_stride + (long)head * d;
@@ -461,9 +471,9 @@ __global__ __launch_bounds__(NW * 64, (NW == 8 ? 4 : 1)) void attn_prefill_dma_k
   float m[NQB], neg_m[NQB], lsum[NQB];
 #pragma unroll
   for (int j = 0; j < NQB; ++j) {
-    m[j] = -INFINITY;
-    neg_m[j] = 0.f;
-    lsum[j] = 0.f;
+    m[j] = sink_start(sink, rhead[j]);
+    neg_m[j] = sink ? -m[j] : 0.f;
+    lsum[j] = sink && g == 0 ? 1.f : 0.f;
 #pragma unroll
     for (int v = 0; v < DV; ++v) acc[v][j] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
   }
@@ -715,7 +725,7 @@ static int launch_prefill_dma(dim3 grid, hipStream_t stream, const bf16_t* q, lo
                               long out_stride, const bf16_t* k_pages, const bf16_t* v_pages, const int* block_tables,
                               int btw, const int* tiles, const int* seg, const int* pos, int nh, int nkv, int d, int ps,
                               float scale_log2, float cap_raw, int window, int HB, int n_hb, int bt_cap,
-                              const float* bias) {
+                              const float* bias, const float* sink) {
   int ps_log2 = 0;
   while ((1 << ps_log2) < ps) ++ps_log2;
   // four stages of a head size of 128 and the table are 72 KB: two workgroups share a compute unit's LDS,
@@ -739,7 +749,7 @@ static int launch_prefill_dma(dim3 grid, hipStream_t stream, const bf16_t* q, lo
   }
   hipLaunchKernelGGL(kernel, dim3(grid.x * grid.y), dim3(NW * 64), smem, stream, q, q_stride, out, out_stride, k_pages,
                      v_pages, block_tables, btw, tiles, seg, pos, nh, nkv, d, ps_log2, scale_log2, cap_raw, window, HB, n_hb,
-                     bt_cap, lmsf_compute_units(), bias);
+                     bt_cap, lmsf_compute_units(), bias, sink);
   return 0;
 }
 
@@ -791,7 +801,7 @@ __global__ __launch_bounds__(256) void attn_decode_mfma_kernel(
     const int* __restrict__ tok_idx, const int* __restrict__ seg, const int* __restrict__ pos, int nh, int nkv, int d,
     int ps, float scale_log2, float cap_raw, int window, int HB, int n_hb, int chunk, int n_splits, float* __restrict__ part_o,
     float* __restrict__ part_ml, bf16_t* __restrict__ out, long out_stride, int heads_first,
-    const float* __restrict__ bias) {
+    const float* __restrict__ bias, const float* __restrict__ sink) {
   constexpr int DS = DPAD / 32, DV = DPAD / 16;
   extern __shared__ float lds_f[];
   // (heads_first: the heads of a token are started together, the tokens in the order of tok_idx, so that a
@@ -829,7 +839,9 @@ __global__ __launch_bounds__(256) void attn_decode_mfma_kernel(
   f32x4_t acc[DV];
 #pragma unroll
   for (int v = 0; v < DV; ++v) acc[v] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
-  float m = -INFINITY, lsum = 0.f;
+  // (of a token's splits and waves one takes the sink: the first wave of the split that ends with the token's own key)
+  const bool takes_sink = sink && w == 0 && c1 == p + 1;
+  float m = takes_sink ? sink_start(sink, head) : -INFINITY, lsum = takes_sink && g == 0 ? 1.f : 0.f;
 
   // The pages of a step's keys are looked up one step ahead (four entries of the block table a lane: the two
   // blocks of 16 keys whose rows it fetches, the two groups of four keys whose values it fetches), so that the
@@ -1119,12 +1131,14 @@ extern "C" int lmsf_attention_tile_tokens(int nh, int nkv) {
 // entries of the block table in LDS instead of 2,048, so that it moves at contexts that a test can afford.
 // ``softcap`` c > 0: a scaled score s becomes c tanh(s / c) before the softmax; 0: scores as they are.
 // ``bias`` float32 [2, nh] or null: r1_h ln(1 + r2_h (i - j)) comes off the score of query i and key j (r2 >= 0).
+// ``sink`` float32 [nh] or null: exp(sink_h) stands in head h's denominator beside the keys' exponentials.
 extern "C" int lmsf_paged_attention_prefill_mfma_biased(const void* q, long q_stride, void* out, long out_stride,
                                                         const void* k_pages, const void* v_pages, long num_pages,
                                                         const int* block_tables, int btw, const int* tiles,
                                                         int n_tiles, const int* seg, const int* pos, int nh, int nkv,
                                                         int d, int ps, float scale, int window, float softcap,
-                                                        const float* bias, int variant, hipStream_t stream) {
+                                                        const float* bias, const float* sink, int variant,
+                                                        hipStream_t stream) {
   LMSF_CHECK(softcap >= 0.f, "paged_attention_prefill: the soft cap must be >= 0, got %g", (double)softcap);
   const float cap_raw = softcap > 0.f ? softcap / scale : 0.f;
   if (int rc = check_common("paged_attention_prefill", q, out, k_pages, v_pages, block_tables, seg, pos, q_stride,
@@ -1146,7 +1160,7 @@ extern "C" int lmsf_paged_attention_prefill_mfma_biased(const void* q, long q_st
     int rc = 0;
 #define LDS_ARGS                                                                                                    \
   grid, stream, (const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)k_pages, (const bf16_t*)v_pages, \
-      block_tables, btw, tiles, seg, pos, nh, nkv, d, ps, scale_log2, cap_raw, window, HB, n_hb, bt_cap, bias
+      block_tables, btw, tiles, seg, pos, nh, nkv, d, ps, scale_log2, cap_raw, window, HB, n_hb, bt_cap, bias, sink
 #define LAUNCH_LDS(DP)                                                                                               \
   rc = bias ? (wp3 ? launch_prefill_dma<DP, 3, true>(LDS_ARGS) : launch_prefill_dma<DP, 1, true>(LDS_ARGS))          \
             : (wp3 ? launch_prefill_dma<DP, 3, false>(LDS_ARGS) : launch_prefill_dma<DP, 1, false>(LDS_ARGS))
@@ -1169,7 +1183,7 @@ extern "C" int lmsf_paged_attention_prefill_mfma_biased(const void* q, long q_st
 #define LAUNCH_W(DP, W, B)                                                                                          \
   hipLaunchKernelGGL((attn_prefill_mfma_kernel<DP, PREFILL_NQB, W, B>), grid, block, 0, stream, (const bf16_t*)q,   \
                      q_stride, (bf16_t*)out, out_stride, (const bf16_t*)k_pages, (const bf16_t*)v_pages,            \
-                     block_tables, btw, tiles, seg, pos, nh, nkv, d, ps, scale_log2, cap_raw, window, HB, n_hb, bias)
+                     block_tables, btw, tiles, seg, pos, nh, nkv, d, ps, scale_log2, cap_raw, window, HB, n_hb, bias, sink)
 #define LAUNCH(DP)                           \
   do {                                       \
     if (bias && wp3) LAUNCH_W(DP, 3, true);  \
@@ -1198,7 +1212,7 @@ static int launch_decode(dim3 grid, hipStream_t stream, const bf16_t* q, long q_
                          const bf16_t* v_pages, const int* block_tables, int btw, const int* tok_idx, const int* seg,
                          const int* pos, int nh, int nkv, int d, int ps, float scale_log2, float cap_raw, int window, int HB, int n_hb,
                          int chunk, int n_splits, float* part_o, float* part_ml, bf16_t* out, long out_stride,
-                         int heads_first, const float* bias) {
+                         int heads_first, const float* bias, const float* sink) {
   const size_t smem = (size_t)(4 * 16 * (DPAD + 4) + 128) * sizeof(float);
   auto kernel = attn_decode_mfma_kernel<DPAD, FULL, ROW8, WP, BIAS>;
   static bool configured = false;   // per instantiation
@@ -1213,7 +1227,7 @@ static int launch_decode(dim3 grid, hipStream_t stream, const bf16_t* q, long q_
   }
   hipLaunchKernelGGL(kernel, grid, dim3(256), smem, stream, q, q_stride, k_pages, v_pages, block_tables, btw, tok_idx,
                      seg, pos, nh, nkv, d, ps, scale_log2, cap_raw, window, HB, n_hb, chunk, n_splits, part_o, part_ml, out,
-                     out_stride, heads_first, bias);
+                     out_stride, heads_first, bias, sink);
   return 0;
 }
 
@@ -1228,13 +1242,13 @@ extern "C" long lmsf_attention_decode_scratch_floats(int n, int nh, int d, int n
 // n_splits * chunk must cover the longest context. scratch: lmsf_attention_decode_scratch_floats floats
 // (not touched with n_splits == 1). seg null: token i is the only token of request i (row i of the block tables),
 // as in a step of single tokens.
-// ``bias``: as for the prefill kernels.
+// ``bias``, ``sink``: as for the prefill kernels.
 extern "C" int lmsf_paged_attention_decode_mfma_biased(const void* q, long q_stride, void* out, long out_stride,
                                                        const void* k_pages, const void* v_pages, long num_pages,
                                                        const int* block_tables, int btw, const int* tok_idx, int n,
                                                        const int* seg, const int* pos, int nh, int nkv, int d, int ps,
                                                        float scale, int window, float softcap, const float* bias,
-                                                       int chunk, int n_splits, float* scratch, int order,
+                                                       const float* sink, int chunk, int n_splits, float* scratch, int order,
                                                        hipStream_t stream) {
   LMSF_CHECK(softcap >= 0.f && scale > 0.f, "paged_attention_decode: the soft cap must be >= 0 and the scale positive");
   const float cap_raw = softcap > 0.f ? softcap / scale : 0.f;
@@ -1265,7 +1279,7 @@ extern "C" int lmsf_paged_attention_decode_mfma_biased(const void* q, long q_str
 #define DECODE_ARGS                                                                                                 \
   grid, stream, (const bf16_t*)q, q_stride, (const bf16_t*)k_pages, (const bf16_t*)v_pages, block_tables, btw, tok_idx, \
       seg, pos, nh, nkv, d, ps, scale_log2, cap_raw, window, HB, n_hb, chunk, n_splits, part_o, part_ml, (bf16_t*)out,       \
-      out_stride, heads_first, bias
+      out_stride, heads_first, bias, sink
   const bool row8 = ps % 32 == 0;   // (needs pages of a multiple of 8 tokens; chosen from 32 on)
 #define LAUNCH_W(DP, W, B)                                                                                       \
   rc = d == DP ? (row8 ? launch_decode<DP, true, true, W, B>(DECODE_ARGS) : launch_decode<DP, true, false, W, B>(DECODE_ARGS)) \
@@ -1310,7 +1324,7 @@ extern "C" int lmsf_paged_attention_prefill_mfma(const void* q, long q_stride, v
                                                  float scale, int window, int variant, hipStream_t stream) {
   return lmsf_paged_attention_prefill_mfma_biased(q, q_stride, out, out_stride, k_pages, v_pages, num_pages,
                                                   block_tables, btw, tiles, n_tiles, seg, pos, nh, nkv, d, ps, scale,
-                                                  window, 0.f, nullptr, variant, stream);
+                                                  window, 0.f, nullptr, nullptr, variant, stream);
 }
 
 extern "C" int lmsf_paged_attention_decode_mfma(const void* q, long q_stride, void* out, long out_stride,
@@ -1321,5 +1335,5 @@ extern "C" int lmsf_paged_attention_decode_mfma(const void* q, long q_stride, vo
                                                 int order, hipStream_t stream) {
   return lmsf_paged_attention_decode_mfma_biased(q, q_stride, out, out_stride, k_pages, v_pages, num_pages,
                                                  block_tables, btw, tok_idx, n, seg, pos, nh, nkv, d, ps, scale,
-                                                 window, 0.f, nullptr, chunk, n_splits, scratch, order, stream);
+                                                 window, 0.f, nullptr, nullptr, chunk, n_splits, scratch, order, stream);
 }

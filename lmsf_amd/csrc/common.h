@@ -159,6 +159,14 @@ __device__ __forceinline__ float gated_product_activation(float g) {
   return 0.5f * g * (1.0f + tanhf(0.79788456080286536f * (g + 0.044715f * g * g * g)));
 }
 
+// The gated activation whose two operands are bounded: g' sigmoid(1.702 g') (u' + 1) with g' = min(g, limit) and u' = u
+// within [-limit, limit].
+__device__ __forceinline__ float bounded_gate(float g, float u, float limit) {
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g / (1.0f + expf(-1.702f * g)) * (u + 1.0f);
+}
+
 // The first key position that a query at position p attends to; the last is p itself. ``window`` > 0: the last
 // ``window`` positions; < 0: the positions of p's own chunk of -window positions, chunks counted from position 0 of
 // the request (wherever a prompt was cut into steps); 0: every position. It never falls as p rises.

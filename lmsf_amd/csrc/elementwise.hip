@@ -64,27 +64,33 @@ extern "C" int lmsf_patch_tokens(int* ids, const int* src, const int* prev, int 
 // kind 0: silu(x) = x / (1 + exp(-x))   (vllm/kernels/activation_kernels.cu:26-42)
 // kind 1: gelu(x) = x/2 (1 + erf(x / sqrt 2)) (vllm/kernels/activation_kernels.cu:44-51)
 // kind 2: the tanh form of gelu, x/2 (1 + tanh(sqrt(2/pi) (x + 0.044715 x^3)))
+// kind 3: both operands bounded by ``limit`` (common.h: bounded_gate)
 template <int KIND>
 __device__ __forceinline__ float gate_activation(float x) {
   if (KIND == 0) return x / (1.0f + expf(-x));
   if (KIND == 1) return 0.5f * x * (1.0f + erff(x * 0.70710678118654752f));
   return 0.5f * x * (1.0f + tanhf(0.79788456080286536f * (x + 0.044715f * x * x * x)));
 }
+template <int KIND>
+__device__ __forceinline__ float gated_value(float g, float u, float limit) {
+  if (KIND == 3) return bounded_gate(g, u, limit);
+  return gate_activation<KIND>(g) * u;
+}
 template <typename T, int KIND>
 __global__ __launch_bounds__(256) void gated_act_kernel(const T* __restrict__ in, T* __restrict__ out, int I,
-                                                        long in_stride) {
+                                                        long in_stride, float limit) {
   const long t = blockIdx.x;
   const int i = blockIdx.y * blockDim.x + threadIdx.x;
   if (i >= I) return;
   const float g = to_f32<T>(in[t * in_stride + i]);
   const float u = to_f32<T>(in[t * in_stride + I + i]);
-  out[t * (long)I + i] = from_f32<T>(gate_activation<KIND>(g) * u);
+  out[t * (long)I + i] = from_f32<T>(gated_value<KIND>(g, u, limit));
 }
 
 // The same with 16-byte accesses: 8 bfloat16 or 4 float32 per thread.
 template <typename T, int KIND>
 __global__ __launch_bounds__(256) void gated_act_vec_kernel(const T* __restrict__ in, T* __restrict__ out, int I,
-                                                            long in_stride) {
+                                                            long in_stride, float limit) {
   constexpr int N = Vec16<T>::N;
   const long t = blockIdx.x;
   const int i = (blockIdx.y * blockDim.x + threadIdx.x) * N;
@@ -94,18 +100,19 @@ __global__ __launch_bounds__(256) void gated_act_vec_kernel(const T* __restrict_
   u.load(in + t * in_stride + I + i);
 #pragma unroll
   for (int e = 0; e < N; ++e) {
-    o.set(e, gate_activation<KIND>(g.get(e)) * u.get(e));
+    o.set(e, gated_value<KIND>(g.get(e), u.get(e), limit));
   }
   o.store(out + t * (long)I + i);
 }
 
-extern "C" int lmsf_gated_act(const void* in, void* out, int dtype, int n_tokens, int I, long in_stride, int kind,
-                              hipStream_t stream) {
+// ``limit``: of kind 3 (the others ignore it)
+extern "C" int lmsf_gated_act_limit(const void* in, void* out, int dtype, int n_tokens, int I, long in_stride, int kind,
+                                    float limit, hipStream_t stream) {
   LMSF_CHECK(in && out, "gated_act: null pointer");
   LMSF_CHECK(n_tokens >= 0 && I > 0 && in_stride >= 2L * I, "gated_act: bad sizes n=%d I=%d stride=%ld", n_tokens, I,
              in_stride);
   LMSF_CHECK((I + 255) / 256 <= 65535, "gated_act: intermediate size %d too large", I);
-  LMSF_CHECK(kind >= 0 && kind <= 2, "gated_act: unknown activation %d", kind);
+  LMSF_CHECK(kind >= 0 && kind <= 3, "gated_act: unknown activation %d", kind);
   LMSF_CHECK(dtype == LMSF_F32 || dtype == LMSF_BF16, "gated_act: unknown dtype code %d", dtype);
   if (n_tokens == 0) return 0;
   const int per = dtype == LMSF_F32 ? 4 : 8;   // elements of a 16-byte access
@@ -113,24 +120,30 @@ extern "C" int lmsf_gated_act(const void* in, void* out, int dtype, int n_tokens
     const int vecs = I / per;
     dim3 vgrid(n_tokens, (vecs + 255) / 256), vblock(256);
 #define GAV(T, K) \
-  hipLaunchKernelGGL((gated_act_vec_kernel<T, K>), vgrid, vblock, 0, stream, (const T*)in, (T*)out, I, in_stride)
+  hipLaunchKernelGGL((gated_act_vec_kernel<T, K>), vgrid, vblock, 0, stream, (const T*)in, (T*)out, I, in_stride, limit)
     if (dtype == LMSF_F32) {
-      if (kind == 0) GAV(float, 0); else if (kind == 1) GAV(float, 1); else GAV(float, 2);
+      if (kind == 0) GAV(float, 0); else if (kind == 1) GAV(float, 1); else if (kind == 2) GAV(float, 2); else GAV(float, 3);
     } else {
-      if (kind == 0) GAV(bf16_t, 0); else if (kind == 1) GAV(bf16_t, 1); else GAV(bf16_t, 2);
+      if (kind == 0) GAV(bf16_t, 0); else if (kind == 1) GAV(bf16_t, 1); else if (kind == 2) GAV(bf16_t, 2); else GAV(bf16_t, 3);
     }
 #undef GAV
     LMSF_LAUNCH_CHECK("gated_act");
     return 0;
   }
   dim3 grid(n_tokens, (I + 255) / 256), block(256);
-#define GA(T, K) hipLaunchKernelGGL((gated_act_kernel<T, K>), grid, block, 0, stream, (const T*)in, (T*)out, I, in_stride)
+#define GA(T, K) hipLaunchKernelGGL((gated_act_kernel<T, K>), grid, block, 0, stream, (const T*)in, (T*)out, I, in_stride, limit)
   if (dtype == LMSF_F32) {
-    if (kind == 0) GA(float, 0); else if (kind == 1) GA(float, 1); else GA(float, 2);
+    if (kind == 0) GA(float, 0); else if (kind == 1) GA(float, 1); else if (kind == 2) GA(float, 2); else GA(float, 3);
   } else {
-    if (kind == 0) GA(bf16_t, 0); else if (kind == 1) GA(bf16_t, 1); else GA(bf16_t, 2);
+    if (kind == 0) GA(bf16_t, 0); else if (kind == 1) GA(bf16_t, 1); else if (kind == 2) GA(bf16_t, 2); else GA(bf16_t, 3);
   }
 #undef GA
   LMSF_LAUNCH_CHECK("gated_act");
   return 0;
+}
+
+extern "C" int lmsf_gated_act(const void* in, void* out, int dtype, int n_tokens, int I, long in_stride, int kind,
+                              hipStream_t stream) {
+  LMSF_CHECK(kind <= 2, "gated_act: unknown activation %d", kind);
+  return lmsf_gated_act_limit(in, out, dtype, n_tokens, I, in_stride, kind, 0.f, stream);
 }

@@ -29,11 +29,11 @@ int lmsf_paged_attention_decode_mfma(const void* q, long q_stride, void* out, lo
 int lmsf_paged_attention_prefill_mfma_biased(const void* q, long q_stride, void* out, long out_stride, const void*
     k_pages, const void* v_pages, long num_pages, const int* block_tables, int btw, const int* tiles, int n_tiles,
     const int* seg, const int* pos, int nh, int nkv, int d, int ps, float scale, int window, float softcap, const
-    float* bias, int variant, hipStream_t stream);
+    float* bias, const float* sink, int variant, hipStream_t stream);
 int lmsf_paged_attention_decode_mfma_biased(const void* q, long q_stride, void* out, long out_stride, const void*
     k_pages, const void* v_pages, long num_pages, const int* block_tables, int btw, const int* tok_idx, int n, const
     int* seg, const int* pos, int nh, int nkv, int d, int ps, float scale, int window, float softcap, const float*
-    bias, int chunk, int n_splits, float* scratch, int order, hipStream_t stream);
+    bias, const float* sink, int chunk, int n_splits, float* scratch, int order, hipStream_t stream);
 
 // token_extras.hip
 int lmsf_position_embedding(const int* ids, const int* pos, const void* table, const void* places, int dtype, float
@@ -59,6 +59,27 @@ int lmsf_norm_add_fits(int W);
 int lmsf_norm_add(const void* a, long a_stride, const void* b, long b_stride, int dtype, const float* wa, const float*
     wb, float eps_pair, float scale, const float* wn, float eps, float* residual, void* out, int n_rows, int W,
     hipStream_t stream);
+
+// streams.hip
+int lmsf_mix_streams(float* X, int ns, const void* y, long y_stride, const float* M, const float* b, const float* a, const
+    float* w, float eps, const int* rows, void* out, int dtype, int n_rows, int W, hipStream_t stream);
+int lmsf_stream_embedding(const int* ids, const void* table, int dtype, float scale, float* X, int n_tokens, int ns, int V,
+    int W, int* bad_flag, hipStream_t stream);
+
+// state_space.hip
+long lmsf_state_space_state_floats(int H, int N, int dv);
+int lmsf_state_space_chunk_tokens(int dtype, int N, int dv);
+long lmsf_state_space_entry_floats(int H, int N, int dv);
+int lmsf_state_space_tokens(const void* xbc, int dtype, long xbc_stride, int x_at, int b_at, int c_at, const float* dt_pre,
+    long dt_stride, const float* dt_bias, const float* rate, const float* D, float* state, long state_stride, const int*
+    seg_starts, const int* state_slots, float* y, long y_stride, int n_tokens, int n_segments, int H, int G, int N, int dv,
+    hipStream_t stream);
+int lmsf_state_space_chunked(const void* xbc, int dtype, long xbc_stride, int x_at, int b_at, int c_at, const float*
+    dt_pre, long dt_stride, const float* dt_bias, const float* rate, const float* D, float* state, long state_stride, const
+    int* state_slots, const int* chunks, const int* bases, int n_chunks, float* entries, float* y, long y_stride, int
+    n_tokens, int n_segments, int H, int G, int N, int dv, hipStream_t stream);
+int lmsf_gated_group_norm(const float* y, long y_stride, const void* z, long z_stride, int dtype, const float* w, void*
+    out, long out_stride, int n_rows, int inner, int parts, float eps, hipStream_t stream);
 
 // latent.hip
 int lmsf_latent_cache_write(const void* x, int dtype, long x_stride, const float* w, float eps, const int* positions,

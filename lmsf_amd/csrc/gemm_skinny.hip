@@ -69,6 +69,7 @@ struct NormAroundArgs {
   int in_tiles;
   float eps;
   int H;                      // columns of the stream: the mean is over these
+  float limit;                // ACT == 6: the bound of the gated activation's operands (no norm is meant)
 };
 
 // ACT: 0 none (plain linear layer), 1 silu-gated, 2 gelu-gated (5: its tanh form), 3 rotary embedding and cache write,
@@ -82,7 +83,7 @@ __global__ __launch_bounds__(NW * 64) void gemm_skinny_kernel(const bf16_t* __re
                                                               long ldy, int M, int N, int K, RopeCacheArgs rc,
                                                               NormAroundArgs na) {
   using T = SkinnyTile<KC>;
-  constexpr int WT = ((ACT >= 1 && ACT <= 3) || ACT == 5) ? 2 : 1;   // W tiles per chunk: gate and up, the two halves of a head, or one
+  constexpr int WT = ((ACT >= 1 && ACT <= 3) || ACT >= 5) ? 2 : 1;   // W tiles per chunk: gate and up, the two halves of a head, or one
   constexpr int XLOADS = (XROWS + T::ROWS_PER_LOAD - 1) / T::ROWS_PER_LOAD;   // load instructions per tile of x
   static_assert(XROWS == 16 || (XROWS == 8 && MT == 1 && XLOADS < T::LOADS), "8 rows of x: one row tile, and a whole load fewer");
   static_assert(!(SCALED || ACT == 4) || MT == 1, "the forms around a norm take up to 16 rows");
@@ -325,7 +326,7 @@ __global__ __launch_bounds__(NW * 64) void gemm_skinny_kernel(const bf16_t* __re
         // stores them (so both paths give the same bits)
         g = bf16_to_f32(f32_to_bf16(g));
         u = bf16_to_f32(f32_to_bf16(u));
-        r = gated_product_activation<ACT>(g) * u;
+        r = ACT == 6 ? bounded_gate(g, u, na.limit) : gated_product_activation<ACT>(g) * u;
       }
       y[(long)m * ldy + n] = from_f32<TOut>(r);
     }
@@ -348,7 +349,7 @@ template <int MT, int KC, int NW, typename TOut, int ACT, int DEPTH, bool SCALED
 static int launch_skinny_x(const void* x, long ldx, const void* W, long ldw, const void* bias, void* y, long ldy, int M,
                            int N, int K, hipStream_t stream, RopeCacheArgs rc, NormAroundArgs na) {
   using T = SkinnyTile<KC>;
-  constexpr int WT = ((ACT >= 1 && ACT <= 3) || ACT == 5) ? 2 : 1;
+  constexpr int WT = ((ACT >= 1 && ACT <= 3) || ACT >= 5) ? 2 : 1;
   const size_t stage = (size_t)NW * (WT + MT) * T::TILE_BYTES;
   const size_t red = (size_t)NW * WT * MT * 64 * 4 * sizeof(float) + ((SCALED || ACT == 4) ? 256 * sizeof(float) : 0);
   const size_t smem = stage > red ? stage : red;
@@ -386,10 +387,11 @@ static int launch_skinny(const void* x, long ldx, const void* W, long ldw, const
 // y [M, N] of out_dtype. Needs M <= 64, K a multiple of 8, 16-byte aligned x and W and row strides
 // that are multiples of 8 elements; anything else is refused. ``variant`` picks the tiling (0: default).
 // act 0: y = x W^T + bias. act 1 (silu) or 2 (gelu): W is [2 N, K] and bias [2 N], gate rows first;
-// y = act(x Wgate^T + bgate) * (x Wup^T + bup), bfloat16 output only.
-extern "C" int lmsf_gemm_skinny(const void* x, long ldx, const void* W, long ldw, const void* bias, void* y,
-                                int out_dtype, long ldy, int M, int N, int K, int variant, int act,
-                                hipStream_t stream) {
+// y = act(x Wgate^T + bgate) * (x Wup^T + bup), bfloat16 output only. act 6: the gated form with both operands bounded by
+// ``limit`` (common.h: bounded_gate).
+extern "C" int lmsf_gemm_skinny_limit(const void* x, long ldx, const void* W, long ldw, const void* bias, void* y,
+                                      int out_dtype, long ldy, int M, int N, int K, int variant, int act, float limit,
+                                      hipStream_t stream) {
   LMSF_CHECK(x && W && y, "gemm_skinny: null pointer");
   LMSF_CHECK(M >= 0 && M <= 64, "gemm_skinny: M=%d outside [0, 64]", M);
   LMSF_CHECK(N > 0 && K > 0 && K % 8 == 0, "gemm_skinny: K=%d must be a positive multiple of 8 (N=%d)", K, N);
@@ -397,16 +399,19 @@ extern "C" int lmsf_gemm_skinny(const void* x, long ldx, const void* W, long ldw
              "gemm_skinny: row strides must cover K and be multiples of 8");
   LMSF_CHECK(lmsf_aligned16(x) && lmsf_aligned16(W), "gemm_skinny: x and W must be 16-byte aligned");
   LMSF_CHECK(out_dtype == LMSF_F32 || out_dtype == LMSF_BF16, "gemm_skinny: unknown output dtype %d", out_dtype);
-  LMSF_CHECK((act >= 0 && act <= 2) || act == 5, "gemm_skinny: unknown activation %d", act);
+  LMSF_CHECK((act >= 0 && act <= 2) || act == 5 || act == 6, "gemm_skinny: unknown activation %d", act);
   LMSF_CHECK(act == 0 || out_dtype == LMSF_BF16, "gemm_skinny: the gated form writes bfloat16 only");
   if (M == 0) return 0;
   const int mt = (M + 15) / 16;
   int rc = 0;
+  NormAroundArgs bound = NormAroundArgs();
+  bound.limit = limit;
   if (act) {
 #define SKG(MT_, KC_, NW_)                                                                                     \
   rc = act == 1   ? launch_skinny<MT_, KC_, NW_, bf16_t, 1>(x, ldx, W, ldw, bias, y, ldy, M, N, K, stream)     \
        : act == 2 ? launch_skinny<MT_, KC_, NW_, bf16_t, 2>(x, ldx, W, ldw, bias, y, ldy, M, N, K, stream)     \
-                  : launch_skinny<MT_, KC_, NW_, bf16_t, 5>(x, ldx, W, ldw, bias, y, ldy, M, N, K, stream)
+       : act == 5 ? launch_skinny<MT_, KC_, NW_, bf16_t, 5>(x, ldx, W, ldw, bias, y, ldy, M, N, K, stream)     \
+                  : launch_skinny<MT_, KC_, NW_, bf16_t, 6>(x, ldx, W, ldw, bias, y, ldy, M, N, K, stream, RopeCacheArgs(), bound)
     if (mt == 1) {
       // 8 waves with two chunks each in flight: measured 3 % ahead of 16 waves with one (deeper: slower)
       if (variant == 1) SKG(1, 128, 8);
@@ -414,7 +419,8 @@ extern "C" int lmsf_gemm_skinny(const void* x, long ldx, const void* W, long ldw
       else   // (variant 2 of the plain product splits K over 8 waves as well: the same order of summation)
         rc = act == 1   ? launch_skinny<1, 64, 8, bf16_t, 1, 2>(x, ldx, W, ldw, bias, y, ldy, M, N, K, stream)
              : act == 2 ? launch_skinny<1, 64, 8, bf16_t, 2, 2>(x, ldx, W, ldw, bias, y, ldy, M, N, K, stream)
-                        : launch_skinny<1, 64, 8, bf16_t, 5, 2>(x, ldx, W, ldw, bias, y, ldy, M, N, K, stream);
+             : act == 5 ? launch_skinny<1, 64, 8, bf16_t, 5, 2>(x, ldx, W, ldw, bias, y, ldy, M, N, K, stream)
+                        : launch_skinny<1, 64, 8, bf16_t, 6, 2>(x, ldx, W, ldw, bias, y, ldy, M, N, K, stream, RopeCacheArgs(), bound);
     } else if (mt == 2) {
       SKG(2, 64, 16);
     } else if (mt == 3) {
@@ -447,6 +453,13 @@ extern "C" int lmsf_gemm_skinny(const void* x, long ldx, const void* W, long ldw
   if (rc) return rc;
   LMSF_LAUNCH_CHECK("gemm_skinny");
   return 0;
+}
+
+extern "C" int lmsf_gemm_skinny(const void* x, long ldx, const void* W, long ldw, const void* bias, void* y,
+                                int out_dtype, long ldy, int M, int N, int K, int variant, int act,
+                                hipStream_t stream) {
+  LMSF_CHECK(act != 6, "gemm_skinny: the bounded form needs its limit");
+  return lmsf_gemm_skinny_limit(x, ldx, W, ldw, bias, y, out_dtype, ldy, M, N, K, variant, act, 0.f, stream);
 }
 
 // The fused QKV projection with rotary embedding and cache write as its epilogue, for M <= 16 tokens:

@@ -49,6 +49,7 @@ struct GemvNorm {
   float* sumsq_out;
   const float* sumsq_in;
   int n_partials;
+  float limit;            // ACT 6: the bound of the gated activation's operands (no norm is meant)
 };
 
 template <int NX, int ACT, typename TOut, bool SC>
@@ -57,7 +58,7 @@ __global__ __launch_bounds__(GEMV_WAVES * 64) void gemv_kernel(const bf16_t* __r
                                                                const bf16_t* __restrict__ bias, TOut* __restrict__ y,
                                                                long ldy, int N, int K, int n_units, RopeCacheArgs rc,
                                                                GemvNorm nm) {
-  constexpr int ROWS = (ACT == 0 || ACT == 4) ? 1 : 2;
+  constexpr int ROWS = (ACT == 0 || ACT == 4) ? 1 : 2;      // (ACT 6: the gated form with bounded operands)
   extern __shared__ __align__(16) unsigned char lds_raw[];
   bf16_t* xs = reinterpret_cast<bf16_t*>(lds_raw);             // [NX][K]
   __shared__ float norm_red[GEMV_WAVES][NX];
@@ -164,10 +165,10 @@ __global__ __launch_bounds__(GEMV_WAVES * 64) void gemv_kernel(const bf16_t* __r
           nm.xw_out[(long)m * nm.ld_xw + n] = f32_to_bf16(v * (bf16_to_f32(nm.weight[n]) + nm.offset));
           sq_acc[m] += v * v;
         }
-      } else if (ACT == 1 || ACT == 2 || ACT == 5) {
+      } else if (ACT == 1 || ACT == 2 || ACT == 5 || ACT == 6) {
         // the two products are rounded to the storage type before the activation, as the unfused path stores them
         const float g = bf16_to_f32(f32_to_bf16(a)), u = bf16_to_f32(f32_to_bf16(b));
-        y[(long)m * ldy + n] = from_f32<TOut>(gated_product_activation<ACT>(g) * u);
+        y[(long)m * ldy + n] = from_f32<TOut>(ACT == 6 ? bounded_gate(g, u, nm.limit) : gated_product_activation<ACT>(g) * u);
       } else {
         // rounded to the storage type first, as the product stores them when the rotation is a kernel of its own
         a = bf16_to_f32(f32_to_bf16(a));
@@ -312,20 +313,24 @@ static int gemv_check(const char* who, const void* x, long ldx, const void* W, l
 
 // x [M, K] bfloat16, M <= 2; W [N, K] (act 0) or [2 N, K] (act 1 silu, 2 gelu: gate rows first); bias likewise or
 // null; y [M, N] of out_dtype (float32 only without activation). K a multiple of 8, x and W 16-byte aligned
-// with row strides that are multiples of 8; M * K * 2 bytes must fit LDS.
-extern "C" int lmsf_gemv(const void* x, long ldx, const void* W, long ldw, const void* bias, void* y, int out_dtype,
-                         long ldy, int M, int N, int K, int act, hipStream_t stream) {
+// with row strides that are multiples of 8; M * K * 2 bytes must fit LDS. act 6: the gated form with both operands bounded
+// by ``limit`` (common.h: bounded_gate).
+extern "C" int lmsf_gemv_limit(const void* x, long ldx, const void* W, long ldw, const void* bias, void* y, int out_dtype,
+                               long ldy, int M, int N, int K, int act, float limit, hipStream_t stream) {
   if (int rc = gemv_check("gemv", x, ldx, W, ldw, M, N, K)) return rc;
   LMSF_CHECK(y != nullptr && ldy >= N, "gemv: bad output");
-  LMSF_CHECK((act >= 0 && act <= 2) || act == 5, "gemv: unknown activation %d", act);
+  LMSF_CHECK((act >= 0 && act <= 2) || act == 5 || act == 6, "gemv: unknown activation %d", act);
   LMSF_CHECK(out_dtype == LMSF_BF16 || (out_dtype == LMSF_F32 && act == 0),
              "gemv: output is bfloat16, or float32 without activation");
   if (M == 0) return 0;
+  GemvNorm bound = GemvNorm();
+  bound.limit = limit;
   int r;
 #define GV(NX_)                                                                                              \
   r = act == 1   ? launch_gemv<NX_, 1, bf16_t>(x, ldx, W, ldw, bias, y, ldy, N, K, N, stream)                 \
       : act == 2 ? launch_gemv<NX_, 2, bf16_t>(x, ldx, W, ldw, bias, y, ldy, N, K, N, stream)                 \
       : act == 5 ? launch_gemv<NX_, 5, bf16_t>(x, ldx, W, ldw, bias, y, ldy, N, K, N, stream)                 \
+      : act == 6 ? launch_gemv<NX_, 6, bf16_t>(x, ldx, W, ldw, bias, y, ldy, N, K, N, stream, RopeCacheArgs(), bound) \
       : out_dtype == LMSF_F32 ? launch_gemv<NX_, 0, float>(x, ldx, W, ldw, bias, y, ldy, N, K, N, stream)     \
                               : launch_gemv<NX_, 0, bf16_t>(x, ldx, W, ldw, bias, y, ldy, N, K, N, stream)
   if (M == 1) GV(1); else GV(2);
@@ -333,6 +338,12 @@ extern "C" int lmsf_gemv(const void* x, long ldx, const void* W, long ldw, const
   if (r) return r;
   LMSF_LAUNCH_CHECK("gemv");
   return 0;
+}
+
+extern "C" int lmsf_gemv(const void* x, long ldx, const void* W, long ldw, const void* bias, void* y, int out_dtype,
+                         long ldy, int M, int N, int K, int act, hipStream_t stream) {
+  LMSF_CHECK(act != 6, "gemv: the bounded form needs its limit");
+  return lmsf_gemv_limit(x, ldx, W, ldw, bias, y, out_dtype, ldy, M, N, K, act, 0.f, stream);
 }
 
 // The fused QKV projection with rotary embedding (NeoX pairing over the whole head) and cache write as its

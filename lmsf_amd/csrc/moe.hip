@@ -18,8 +18,9 @@
 // (token, choice) a float32 factor on the expert's *input*, y_e(s h), which the gate and up products take as a factor on
 // their results before these are rounded (W (s h) = s (W h)); ``base_scale`` a float32 factor per token on ``base``;
 // ``out_scale`` a float32 factor per (token, choice) on what the expert returns. Experts may also be of one matrix in,
-// y_e(h) = Wd_e relu(Wu_e h)^2 with Wgu [E, F, W] (lmsf_table_moe_act). A second router (lmsf_moe_route_groups) takes
-// softmax scores and chooses within the best groups of neighbouring experts.
+// y_e(h) = Wd_e relu(Wu_e h)^2 with Wgu [E, F, W], or gated with bounded operands, and experts after the last may have no
+// matrices and return their input (lmsf_table_moe_act). A second router (lmsf_moe_route_groups) takes softmax scores,
+// chooses within the best groups of neighbouring experts and may choose by corrected scores.
 #include "common.h"
 
 #include <math.h>
@@ -66,11 +67,12 @@ template <typename T>
 __global__ __launch_bounds__(MOE_THREADS) void moe_gate_up_kernel(
     const T* __restrict__ h, long h_stride, const T* __restrict__ Wgu, const int* __restrict__ ids,
     const int* __restrict__ table, int vocab, int top, int E, T* __restrict__ act, int F, int W, int vec,
-    const float* __restrict__ pair_scale, int gated) {
+    const float* __restrict__ pair_scale, int gated, float limit, int identity) {
   extern __shared__ float sh[];   // [W]
   const int nk = blockIdx.x, n = nk / top, k = nk - n * top;
   const int id = min(max(ids ? ids[n] : n, 0), vocab - 1);
-  const int e = min(max(table[(long)id * top + k], 0), E - 1);
+  const int e = min(max(table[(long)id * top + k], 0), E + identity - 1);
+  if (e >= E) return;             // (what an expert without matrices returns is its input: the kernel below)
   const float ps = pair_scale ? pair_scale[nk] : 1.f;
   for (int i = threadIdx.x; i < W; i += MOE_THREADS) sh[i] = ps * to_f32<T>(h[(long)n * h_stride + i]);
   __syncthreads();
@@ -102,7 +104,7 @@ __global__ __launch_bounds__(MOE_THREADS) void moe_gate_up_kernel(
         gg = to_f32<T>(from_f32<T>(ag[r]));
         uu = to_f32<T>(from_f32<T>(au[r]));
       }
-    act[(long)nk * F + f0 + lane] = from_f32<T>(gg / (1.f + expf(-gg)) * uu);
+    act[(long)nk * F + f0 + lane] = from_f32<T>(limit > 0.f ? bounded_gate(gg, uu, limit) : gg / (1.f + expf(-gg)) * uu);
   }
 }
 
@@ -112,7 +114,8 @@ __global__ __launch_bounds__(MOE_THREADS) void moe_down_kernel(
     const T* __restrict__ act, const T* __restrict__ Wd, const int* __restrict__ ids, const int* __restrict__ table,
     int vocab, int top, int E, float weight, const T* __restrict__ base, long base_stride, T* __restrict__ out,
     long out_stride, int F, int W, int vec, const float* __restrict__ base_scale,
-    const float* __restrict__ out_scale) {
+    const float* __restrict__ out_scale, int identity, const T* __restrict__ h, long h_stride,
+    const float* __restrict__ pair_scale) {
   extern __shared__ float sa[];   // [top, F]
   const int n = blockIdx.x;
   const int id = min(max(ids ? ids[n] : n, 0), vocab - 1);
@@ -126,9 +129,15 @@ __global__ __launch_bounds__(MOE_THREADS) void moe_down_kernel(
 #pragma unroll
   for (int r = 0; r < MOE_OUT_PER_WAVE; ++r) total[r] = 0.f;
   for (int k = 0; k < top; ++k) {
-    const int e = min(max(table[(long)id * top + k], 0), E - 1);
+    const int e = min(max(table[(long)id * top + k], 0), E + identity - 1);
     float part[MOE_OUT_PER_WAVE];
     const float os = out_scale ? out_scale[(long)n * top + k] : 1.f;
+    if (e >= E) {      // an expert without matrices returns its input
+      const float f = os * (pair_scale ? pair_scale[(long)n * top + k] : 1.f);
+#pragma unroll
+      for (int r = 0; r < MOE_OUT_PER_WAVE; ++r) total[r] += f * to_f32<T>(h[(long)n * h_stride + o0 + min(r, valid - 1)]);
+      continue;
+    }
     moe_rows_dot<T, MOE_OUT_PER_WAVE>(Wd + ((long)e * W + o0) * F, F, valid, sa + k * F, F, lane, vec, part);
 #pragma unroll
     for (int r = 0; r < MOE_OUT_PER_WAVE; ++r) total[r] += os * part[r];
@@ -152,7 +161,7 @@ __global__ __launch_bounds__(MOE_THREADS) void moe_down_kernel(
 // tile (of up to ``tile_pairs`` pairs) its expert, its first place and its number of pairs; n_tiles[0]: how many
 // tiles there are. One workgroup.
 __global__ __launch_bounds__(1024) void moe_group_kernel(const int* __restrict__ ids, const int* __restrict__ table,
-                                                        int vocab, int top, int E, int P, int tile_pairs,
+                                                        int vocab, int top, int E, int identity, int P, int tile_pairs,
                                                         int* __restrict__ order, int* __restrict__ tiles,
                                                         int* __restrict__ n_tiles) {
   extern __shared__ int sm[];   // [E] counts, [E] first places, [E] fill counters
@@ -163,7 +172,8 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(const int* __restrict__
   __syncthreads();
   for (int p = threadIdx.x; p < P; p += blockDim.x) {
     const int id = min(max(ids ? ids[p / top] : p / top, 0), vocab - 1);
-    atomicAdd(&cnt[min(max(table[(long)id * top + p % top], 0), E - 1)], 1);
+    const int e = min(max(table[(long)id * top + p % top], 0), E + identity - 1);
+    if (e < E) atomicAdd(&cnt[e], 1);
   }
   __syncthreads();
   if (threadIdx.x == 0) {
@@ -183,8 +193,8 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(const int* __restrict__
   __syncthreads();
   for (int p = threadIdx.x; p < P; p += blockDim.x) {
     const int id = min(max(ids ? ids[p / top] : p / top, 0), vocab - 1);
-    const int e = min(max(table[(long)id * top + p % top], 0), E - 1);
-    order[first[e] + atomicAdd(&fill[e], 1)] = p;
+    const int e = min(max(table[(long)id * top + p % top], 0), E + identity - 1);
+    if (e < E) order[first[e] + atomicAdd(&fill[e], 1)] = p;
   }
 }
 
@@ -204,7 +214,7 @@ __global__ __launch_bounds__(256) void moe_tile_lds_kernel(const bf16_t* __restr
                                                            const bf16_t* __restrict__ Wm, const int* __restrict__ order,
                                                            const int* __restrict__ tiles, const int* __restrict__ n_tiles,
                                                            void* __restrict__ y, int O, int K,
-                                                           const float* __restrict__ pair_scale) {
+                                                           const float* __restrict__ pair_scale, float limit) {
   constexpr bool GATED = KIND == 1, UP = KIND != 0;
   constexpr int AR = GATED ? 256 : 128;            // rows of W a step
   constexpr int NLA = AR * 4 / 256;                // 16-byte pieces of W a thread copies a step
@@ -297,7 +307,7 @@ __global__ __launch_bounds__(256) void moe_tile_lds_kernel(const bf16_t* __restr
         if (o >= O) continue;
         if (GATED) {
           const float g = bf16_to_f32(f32_to_bf16(ps * acc[a][mt][j])), u = bf16_to_f32(f32_to_bf16(ps * acc[NA - 4 + a][mt][j]));
-          reinterpret_cast<bf16_t*>(y)[(long)p * O + o] = f32_to_bf16(g / (1.f + expf(-g)) * u);
+          reinterpret_cast<bf16_t*>(y)[(long)p * O + o] = f32_to_bf16(limit > 0.f ? bounded_gate(g, u, limit) : g / (1.f + expf(-g)) * u);
         } else if (UP) {
           const float u = fmaxf(bf16_to_f32(f32_to_bf16(ps * acc[a][mt][j])), 0.f);
           reinterpret_cast<bf16_t*>(y)[(long)p * O + o] = f32_to_bf16(u * u);
@@ -308,18 +318,29 @@ __global__ __launch_bounds__(256) void moe_tile_lds_kernel(const bf16_t* __restr
   }
 }
 
-// out[n, o] = base[n, o] + weight * sum_k rows[n * top + k, o]
+// out[n, o] = base[n, o] + weight * sum_k rows[n * top + k, o]; the choices of ``table`` (row ids[n], or n) from E on are
+// experts without matrices, which return their input
 __global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restrict__ rows, int top, float weight,
                                                           const bf16_t* __restrict__ base, long base_stride,
                                                           bf16_t* __restrict__ out, long out_stride, int W,
                                                           const float* __restrict__ base_scale,
-                                                          const float* __restrict__ out_scale) {
+                                                          const float* __restrict__ out_scale,
+                                                          const int* __restrict__ ids, const int* __restrict__ table,
+                                                          int vocab, int E, int identity,
+                                                          const bf16_t* __restrict__ h, long h_stride,
+                                                          const float* __restrict__ pair_scale) {
   const int n = blockIdx.x;
+  const int* chosen = table + (long)(identity > 0 ? min(max(ids ? ids[n] : n, 0), vocab - 1) : 0) * top;
   const float bs = base_scale ? base_scale[n] : 1.f;
   for (int o = threadIdx.x; o < W; o += 256) {
     float s = 0.f;
-    for (int k = 0; k < top; ++k)
-      s += (out_scale ? out_scale[(long)n * top + k] : 1.f) * rows[((long)n * top + k) * W + o];
+    for (int k = 0; k < top; ++k) {
+      const float os = out_scale ? out_scale[(long)n * top + k] : 1.f;
+      if (identity > 0 && chosen[k] >= E)
+        s += os * (pair_scale ? pair_scale[(long)n * top + k] : 1.f) * bf16_to_f32(h[(long)n * h_stride + o]);
+      else
+        s += os * rows[((long)n * top + k) * W + o];
+    }
     const float b = base ? bs * bf16_to_f32(base[(long)n * base_stride + o]) : 0.f;
     out[(long)n * out_stride + o] = f32_to_bf16(b + weight * s);
   }
@@ -339,15 +360,19 @@ extern "C" int lmsf_table_moe_grouped(int dtype, int n_tokens, int top, int E, i
 }
 
 // ``act_kind`` 0: gated experts, Wgu [E, 2 F, W]; 1: experts of one matrix, Wgu [E, F, W], y_e(h) = Wd_e relu(Wu_e h)^2.
-// ``out_scale``: a float32 factor per (token, choice) on what the expert returns (null: none).
+// 2: gated experts whose activation has both operands bounded by ``limit`` (common.h: bounded_gate).
+// ``out_scale``: a float32 factor per (token, choice) on what the expert returns (null: none). ``identity``: so many
+// experts after the E with matrices (choices E .. E + identity - 1) have none and return their input.
 extern "C" int lmsf_table_moe_act(const void* h, int dtype, long h_stride, const void* Wgu, const void* Wd,
                                   const int* ids, const int* table, int vocab, int top, int E, float weight,
                                   const void* base, long base_stride, const float* pair_scale,
-                                  const float* base_scale, const float* out_scale, int act_kind, void* act, void* out,
+                                  const float* base_scale, const float* out_scale, int act_kind, float limit,
+                                  int identity, void* act, void* out,
                                   long out_stride, int n_tokens, int F, int W, int* scratch_ints,
                                   float* scratch_rows, hipStream_t stream) {
-  LMSF_CHECK(act_kind == 0 || act_kind == 1, "table_moe: unknown kind of expert %d", act_kind);
-  const int gated = act_kind == 0;
+  LMSF_CHECK(act_kind >= 0 && act_kind <= 2, "table_moe: unknown kind of expert %d", act_kind);
+  LMSF_CHECK((act_kind == 2) == (limit > 0.f) && identity >= 0, "table_moe: a limit goes with bounded experts");
+  const int gated = act_kind != 1;
   LMSF_CHECK(h && Wgu && Wd && table && act && out, "table_moe: null pointer");
   LMSF_CHECK(ids || vocab >= n_tokens, "table_moe: without token ids the table has a row per token");
   LMSF_CHECK(dtype == LMSF_F32 || dtype == LMSF_BF16, "table_moe: unknown dtype code %d", dtype);
@@ -362,19 +387,20 @@ extern "C" int lmsf_table_moe_act(const void* h, int dtype, long h_stride, const
     int* order = scratch_ints;
     int* tiles = order + P;
     int* n_tiles = tiles + 3 * (max_tiles + 1);
-    hipLaunchKernelGGL(moe_group_kernel, dim3(1), dim3(1024), (size_t)3 * E * 4, stream, ids, table, vocab, top, E, P,
-                       MOE_TILE, order, tiles, n_tiles);
+    hipLaunchKernelGGL(moe_group_kernel, dim3(1), dim3(1024), (size_t)3 * E * 4, stream, ids, table, vocab, top, E, identity,
+                       P, MOE_TILE, order, tiles, n_tiles);
     if (gated)
       hipLaunchKernelGGL((moe_tile_lds_kernel<1>), dim3(max_tiles, (F + 127) / 128), dim3(256), 0, stream,
-                         (const bf16_t*)h, h_stride, top, (const bf16_t*)Wgu, order, tiles, n_tiles, act, F, W, pair_scale);
+                         (const bf16_t*)h, h_stride, top, (const bf16_t*)Wgu, order, tiles, n_tiles, act, F, W, pair_scale, limit);
     else
       hipLaunchKernelGGL((moe_tile_lds_kernel<2>), dim3(max_tiles, (F + 127) / 128), dim3(256), 0, stream,
-                         (const bf16_t*)h, h_stride, top, (const bf16_t*)Wgu, order, tiles, n_tiles, act, F, W, pair_scale);
+                         (const bf16_t*)h, h_stride, top, (const bf16_t*)Wgu, order, tiles, n_tiles, act, F, W, pair_scale, limit);
     hipLaunchKernelGGL((moe_tile_lds_kernel<0>), dim3(max_tiles, (W + 127) / 128), dim3(256), 0, stream,
                        (const bf16_t*)act, (long)F, top, (const bf16_t*)Wd, order, tiles, n_tiles, (void*)scratch_rows, W,
-                       F, (const float*)nullptr);
+                       F, (const float*)nullptr, 0.f);
     hipLaunchKernelGGL(moe_combine_kernel, dim3(n_tokens), dim3(256), 0, stream, scratch_rows, top, weight,
-                       (const bf16_t*)base, base_stride, (bf16_t*)out, out_stride, W, base_scale, out_scale);
+                       (const bf16_t*)base, base_stride, (bf16_t*)out, out_stride, W, base_scale, out_scale, ids, table,
+                       vocab, E, identity, (const bf16_t*)h, h_stride, pair_scale);
     LMSF_LAUNCH_CHECK("table_moe (grouped)");
     return 0;
   }
@@ -384,16 +410,20 @@ extern "C" int lmsf_table_moe_act(const void* h, int dtype, long h_stride, const
   const int vec1 = W % vn == 0 && lmsf_aligned16(Wgu), vec2 = F % vn == 0 && lmsf_aligned16(Wd);
   if (dtype == LMSF_F32) {
     hipLaunchKernelGGL((moe_gate_up_kernel<float>), g1, dim3(MOE_THREADS), (size_t)W * 4, stream, (const float*)h,
-                       h_stride, (const float*)Wgu, ids, table, vocab, top, E, (float*)act, F, W, vec1, pair_scale, gated);
+                       h_stride, (const float*)Wgu, ids, table, vocab, top, E, (float*)act, F, W, vec1, pair_scale, gated, limit,
+                       identity);
     hipLaunchKernelGGL((moe_down_kernel<float>), g2, dim3(MOE_THREADS), (size_t)top * F * 4, stream, (const float*)act,
                        (const float*)Wd, ids, table, vocab, top, E, weight, (const float*)base, base_stride,
-                       (float*)out, out_stride, F, W, vec2, base_scale, out_scale);
+                       (float*)out, out_stride, F, W, vec2, base_scale, out_scale, identity, (const float*)h, h_stride,
+                       pair_scale);
   } else {
     hipLaunchKernelGGL((moe_gate_up_kernel<bf16_t>), g1, dim3(MOE_THREADS), (size_t)W * 4, stream, (const bf16_t*)h,
-                       h_stride, (const bf16_t*)Wgu, ids, table, vocab, top, E, (bf16_t*)act, F, W, vec1, pair_scale, gated);
+                       h_stride, (const bf16_t*)Wgu, ids, table, vocab, top, E, (bf16_t*)act, F, W, vec1, pair_scale, gated, limit,
+                       identity);
     hipLaunchKernelGGL((moe_down_kernel<bf16_t>), g2, dim3(MOE_THREADS), (size_t)top * F * 4, stream,
                        (const bf16_t*)act, (const bf16_t*)Wd, ids, table, vocab, top, E, weight, (const bf16_t*)base,
-                       base_stride, (bf16_t*)out, out_stride, F, W, vec2, base_scale, out_scale);
+                       base_stride, (bf16_t*)out, out_stride, F, W, vec2, base_scale, out_scale, identity,
+                       (const bf16_t*)h, h_stride, pair_scale);
   }
   LMSF_LAUNCH_CHECK("table_moe");
   return 0;
@@ -405,7 +435,7 @@ extern "C" int lmsf_table_moe(const void* h, int dtype, long h_stride, const voi
                               long out_stride, int n_tokens, int F, int W, int* scratch_ints, float* scratch_rows,
                               hipStream_t stream) {
   return lmsf_table_moe_act(h, dtype, h_stride, Wgu, Wd, ids, table, vocab, top, E, weight, base, base_stride,
-                            pair_scale, base_scale, nullptr, 0, act, out, out_stride, n_tokens, F, W, scratch_ints,
+                            pair_scale, base_scale, nullptr, 0, 0.f, 0, act, out, out_stride, n_tokens, F, W, scratch_ints,
                             scratch_rows, stream);
 }
 
@@ -477,8 +507,9 @@ extern "C" int lmsf_moe_route(const float* z, long z_stride, int n_tokens, int E
 // lane, lane + 64, ... (at most 256 groups).
 __global__ __launch_bounds__(256) void moe_route_groups_kernel(const float* __restrict__ z, long z_stride, int n_tokens,
                                                                int E, int top, int softmax, int groups, int keep,
-                                                               int renorm, int* __restrict__ choice,
-                                                               float* __restrict__ weight) {
+                                                               int renorm, const float* __restrict__ correction,
+                                                               float scale, int extra, int* __restrict__ choice,
+                                                               float* __restrict__ weight, float* __restrict__ gate) {
   const int n = blockIdx.x * (256 / LMSF_WAVE) + threadIdx.x / LMSF_WAVE, lane = threadIdx.x % LMSF_WAVE;
   if (n >= n_tokens) return;
   const float* row = z + (long)n * z_stride;
@@ -489,6 +520,9 @@ __global__ __launch_bounds__(256) void moe_route_groups_kernel(const float* __re
     for (int e = lane; e < E; e += LMSF_WAVE) sum += expf(row[e] - mx);
     sum = wave_sum(sum);
   }
+  // what a choice compares: the logit, which orders as its score does, or the score plus the expert's correction
+  auto score = [&](float x) { return softmax ? expf(x - mx) / sum : 1.f / (1.f + expf(-x)); };
+  auto key = [&](int e) { return correction ? score(row[e]) + correction[e] : row[e]; };
   const int per = E / groups;
   float gbest[4];
   unsigned kept = 0;           // bit i: group lane + 64 i is kept
@@ -497,7 +531,7 @@ __global__ __launch_bounds__(256) void moe_route_groups_kernel(const float* __re
     const int g = lane + LMSF_WAVE * i;
     gbest[i] = -INFINITY;
     if (g < groups)
-      for (int e = g * per; e < (g + 1) * per; ++e) gbest[i] = fmaxf(gbest[i], row[e]);
+      for (int e = g * per; e < (g + 1) * per; ++e) gbest[i] = fmaxf(gbest[i], key(e));
   }
   if (keep >= groups) kept = 0xFu;
   else
@@ -533,7 +567,7 @@ __global__ __launch_bounds__(256) void moe_route_groups_kernel(const float* __re
       const int g = min(e, E - 1) / per;
       const unsigned flags = __shfl(kept, g % LMSF_WAVE, LMSF_WAVE);
       if (e >= E || !((flags >> (g / LMSF_WAVE)) & 1u)) continue;
-      const float sc = row[e];
+      const float sc = key(e);
       const bool below = sc < last || (sc == last && e > last_e);
       if (below && (sc > best || (sc == best && e < best_e))) {
         best = sc;
@@ -551,7 +585,7 @@ __global__ __launch_bounds__(256) void moe_route_groups_kernel(const float* __re
     }
     last = best;
     last_e = best_e;
-    const float sc = softmax ? expf(best - mx) / sum : 1.f / (1.f + expf(-best));
+    const float sc = score(row[min(best_e, E - 1)]);
     total += sc;
     if (lane == k) {
       mine = sc;
@@ -560,21 +594,25 @@ __global__ __launch_bounds__(256) void moe_route_groups_kernel(const float* __re
   }
   if (lane < top) {
     choice[(long)n * top + lane] = mine_e;
-    weight[(long)n * top + lane] = renorm ? mine / total : mine;
+    weight[(long)n * top + lane] = scale * (renorm ? mine / (total + 1e-20f) : mine);
   }
+  if (extra >= 0 && lane == 0) gate[n] = 1.f / (1.f + expf(-row[extra]));
 }
 
+// ``correction`` float32 [E] or null: added to the scores for the choice alone, not for the weights. ``scale`` multiplies
+// the weights. ``extra``, ``gate``: as for lmsf_moe_route.
 extern "C" int lmsf_moe_route_groups(const float* z, long z_stride, int n_tokens, int E, int top, int softmax,
-                                     int groups, int keep, int renorm, int* choice, float* weight,
-                                     hipStream_t stream) {
-  LMSF_CHECK(z && choice && weight, "moe_route_groups: null pointer");
-  LMSF_CHECK(E > 0 && top > 0 && top <= E && top <= LMSF_WAVE && z_stride >= E, "moe_route_groups: bad sizes");
+                                     int groups, int keep, int renorm, const float* correction, float scale, int extra,
+                                     int* choice, float* weight, float* gate, hipStream_t stream) {
+  LMSF_CHECK(z && choice && weight && (extra < 0 || gate), "moe_route_groups: null pointer");
+  LMSF_CHECK(E > 0 && top > 0 && top <= E && top <= LMSF_WAVE && z_stride >= E && extra < z_stride,
+             "moe_route_groups: bad sizes");
   LMSF_CHECK(groups > 0 && groups <= 256 && E % groups == 0 && keep > 0 && keep <= groups &&
                  (long)keep * (E / groups) >= top,
              "moe_route_groups: %d of %d groups of %d experts cannot hold %d choices", keep, groups, E, top);
   if (n_tokens <= 0) return 0;
   hipLaunchKernelGGL(moe_route_groups_kernel, dim3((n_tokens + 3) / 4), dim3(256), 0, stream, z, z_stride, n_tokens, E,
-                     top, softmax, groups, keep, renorm, choice, weight);
+                     top, softmax, groups, keep, renorm, correction, scale, extra, choice, weight, gate);
   LMSF_LAUNCH_CHECK("moe_route_groups");
   return 0;
 }

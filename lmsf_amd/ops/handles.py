@@ -113,3 +113,24 @@ class NormedPair:
     @property
     def device(self) -> torch.device:
         return self.a.device
+
+
+class StreamUpdate:
+    """A sublayer's result that a residual of several streams X [N, s, W] has not taken yet: the streams become
+    X_t = sum_u mix[u, t] X_u + add_t y. ``y`` [N, W] in the run's type, ``mix`` float32 [s, s] (from row to column),
+    ``add`` float32 [s]. ``HipOps.mix_streams`` carries it out together with the norm that follows."""
+
+    __slots__ = ("y", "mix", "add")
+
+    def __init__(self, y: torch.Tensor, mix: torch.Tensor, add: torch.Tensor):
+        self.y = y
+        self.mix = mix
+        self.add = add
+
+    @property
+    def shape(self) -> Tuple[int, int]:
+        return tuple(self.y.shape)
+
+    @property
+    def device(self) -> torch.device:
+        return self.y.device

@@ -12,7 +12,7 @@ import torch
 
 from . import dispatch as D
 from . import library
-from .handles import DeferredLinear, NormedPair, PendingProduct, ScaledRows
+from .handles import DeferredLinear, NormedPair, PendingProduct, ScaledRows, StreamUpdate
 
 F32 = 0
 BF16 = 1
@@ -442,14 +442,16 @@ class HipOps:
                         block_tables: torch.Tensor, seg: torch.Tensor, pos: torch.Tensor, nh: int, nkv: int, d: int,
                         scale: float, window: int = 0, batch=None, kernel: Optional[str] = None,
                         chunk: int = 0, weights_f32: bool = False, softcap: float = 0.0,
-                        distance_bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+                        distance_bias: Optional[torch.Tensor] = None,
+                        sink: Optional[torch.Tensor] = None) -> torch.Tensor:
         """Attention of every query token over the cached keys of its request: those at positions up to its own,
         within the last ``window`` positions if a window is given, or within its own chunk of ``chunk`` positions
         (chunks counted from position 0 of the request) if a chunk size is given. ``weights_f32``: in a bfloat16 run
         the softmax weights enter the product with the values in full float32 (as three bfloat16 parts on the
         matrix cores) instead of rounded to bfloat16; scores, maxima and sums are float32 either way. ``softcap``
         c > 0: a scaled score s enters the softmax as c tanh(s / c). ``distance_bias`` (float32 [2, nh], rows r1 and
-        r2 >= 0): r1_h ln(1 + r2_h (i - j)) comes off the score of query i and key j, after the cap.
+        r2 >= 0): r1_h ln(1 + r2_h (i - j)) comes off the score of query i and key j, after the cap. ``sink`` (float32
+        [nh]): exp(sink_h) stands in head h's softmax denominator beside the keys' exponentials.
 
         ``q`` is [N, >= nh*d] with unit column stride (it may be the fused QKV buffer, of which the
         first nh*d columns are read). ``k_pages`` [pages, nkv, page_size, d], ``v_pages``
@@ -476,6 +478,9 @@ class HipOps:
         if distance_bias is not None:
             self._dev(distance_bias)
             self._f32_vec(distance_bias, 2 * nh, "paged_attention: distance_bias")
+        if sink is not None:
+            self._dev(sink)
+            self._f32_vec(sink, nh, "paged_attention: sink")
         bias = _ptr(distance_bias)
         out = torch.empty((N, nh * d), dtype=q.dtype, device=q.device)
         if N == 0:
@@ -493,7 +498,7 @@ class HipOps:
             self._check(self.lib.lmsf_paged_attention_generic_biased(
                 _ptr(q), q.stride(0), _ptr(out), out.stride(0), _ptr(k_pages), _ptr(v_pages), num_pages,
                 _ptr(block_tables), block_tables.shape[1], _ptr(seg), _ptr(pos), N, nh, nkv, d, ps, float(scale),
-                int(window or 0), float(softcap), bias, _code(q.dtype), self._stream()))
+                int(window or 0), float(softcap), bias, _ptr(sink), _code(q.dtype), self._stream()))
             return out
         plan = self._attention_plan(batch, seg, pos, nh, nkv)
         exact = self.ATTENTION_WEIGHTS_F32 if weights_f32 else 0
@@ -501,7 +506,7 @@ class HipOps:
         if plan.tiles is not None:
             self._check(self.lib.lmsf_paged_attention_prefill_mfma_biased(
                 _ptr(q), q.stride(0), _ptr(out), out.stride(0), *common, _ptr(plan.tiles), plan.n_tiles,
-                _ptr(seg), _ptr(pos), nh, nkv, d, ps, float(scale), int(window or 0), float(softcap), bias,
+                _ptr(seg), _ptr(pos), nh, nkv, d, ps, float(scale), int(window or 0), float(softcap), bias, _ptr(sink),
                 self.prefill_attention_variant + exact, self._stream()))
         if plan.n_single:
             c_chunk, c_splits = ctypes.c_int(0), ctypes.c_int(0)
@@ -513,7 +518,7 @@ class HipOps:
             self._check(self.lib.lmsf_paged_attention_decode_mfma_biased(
                 _ptr(q), q.stride(0), _ptr(out), out.stride(0), *common, _ptr(plan.single_tokens), plan.n_single,
                 None if plan.token_is_request else _ptr(seg), _ptr(pos), nh, nkv, d, ps, float(scale),
-                int(window or 0), float(softcap), bias, chunk, n_splits, _ptr(scratch), self.decode_attention_order + exact,
+                int(window or 0), float(softcap), bias, _ptr(sink), chunk, n_splits, _ptr(scratch), self.decode_attention_order + exact,
                 self._stream()))
         return out
 
@@ -773,10 +778,13 @@ class HipOps:
     def table_moe(self, h: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.Tensor, token_ids: Optional[torch.Tensor],
                   table: torch.Tensor, weight: float, base: Optional[torch.Tensor] = None,
                   pair_scale: Optional[torch.Tensor] = None, base_scale: Optional[torch.Tensor] = None,
-                  out_scale: Optional[torch.Tensor] = None, gated: bool = True) -> torch.Tensor:
+                  out_scale: Optional[torch.Tensor] = None, gated: bool = True, limit: float = 0.0,
+                  identity: int = 0) -> torch.Tensor:
         """out[n] = base[n] + weight * sum_k down_e(silu(gate_e h[n]) * up_e h[n]) over e = table[token_ids[n], k].
         ``gated`` False: experts of one matrix, ``w_gate_up`` [E, F, W], down_e(relu(up_e h[n])^2). ``out_scale``
-        (float32 [N, top]): what the expert of (n, k) returns is multiplied by out_scale[n, k].
+        (float32 [N, top]): what the expert of (n, k) returns is multiplied by out_scale[n, k]. ``limit`` > 0: gated
+        experts whose activation has both operands bounded (``gated_act``, kind "bounded"). ``identity``: choices E to
+        E + identity - 1 are experts without matrices that return their input.
         ``w_gate_up`` [E, 2 F, W] (gate rows first), ``w_down`` [E, W, F], ``table`` int32 [vocab, top].
         ``token_ids`` None: row n of the table is token n's choice (a router's, ``moe_route``). ``pair_scale``
         (float32 [N, top]): the expert of (n, k) gets pair_scale[n, k] * h[n] as its input. ``base_scale``
@@ -806,6 +814,8 @@ class HipOps:
                                       or not out_scale.is_contiguous()):
             raise ValueError("table_moe: out_scale must be contiguous float32 [%d, %d]" % (N, top))
         self._dev(out_scale)
+        if limit < 0 or (limit > 0 and not gated) or identity < 0:
+            raise ValueError("table_moe: a limit goes with gated experts")
         act = torch.empty((N * top, F), dtype=h.dtype, device=h.device)
         out = torch.empty((N, W), dtype=h.dtype, device=h.device)
         ints = rows = None
@@ -816,18 +826,24 @@ class HipOps:
         self._check(self.lib.lmsf_table_moe_act(
             _ptr(h), _code(h.dtype), h.stride(0), _ptr(w_gate_up), _ptr(w_down), _ptr(token_ids), _ptr(table), vocab,
             top, E, float(weight), _ptr(base), base.stride(0) if base is not None else 0, _ptr(pair_scale),
-            _ptr(base_scale), _ptr(out_scale), 0 if gated else 1, _ptr(act), _ptr(out), out.stride(0), N, F, W,
+            _ptr(base_scale), _ptr(out_scale), (2 if limit > 0 else 0) if gated else 1, float(limit), int(identity), _ptr(act), _ptr(out), out.stride(0), N, F, W,
             _ptr(ints), _ptr(rows), self._stream()))
         return out
 
     def moe_route_groups(self, logits: torch.Tensor, experts: int, top: int, softmax: bool = True, groups: int = 1,
-                         keep: int = 1, renorm: bool = False):
+                         keep: int = 1, renorm: bool = False, correction: Optional[torch.Tensor] = None,
+                         scale: float = 1.0, extra: int = -1):
         """A router's choice from float32 logits [N, >= experts] with scores softmax(logits) over all experts (or
         sigmoid), where only experts of the ``keep`` best of ``groups`` equal groups of neighbours may be chosen (a
         group's score is its best expert's): (choice int32 [N, top], weight float32 [N, top]), the weights the
-        chosen experts' scores, over their sum with ``renorm``."""
-        self._dev(logits)
-        if logits.dtype != torch.float32 or logits.dim() != 2 or logits.stride(1) != 1 or logits.shape[1] < experts:
+        chosen experts' scores, over their sum with ``renorm``, times ``scale``. ``correction`` (float32 [experts]) is
+        added to the scores for the choice alone. ``extra`` >= 0: a third result, float32 [N], the sigmoid of that column
+        (beside the experts')."""
+        self._dev(logits, correction)
+        if correction is not None:
+            self._f32_vec(correction, experts, "moe_route_groups: correction")
+        if logits.dtype != torch.float32 or logits.dim() != 2 or logits.stride(1) != 1 or logits.shape[1] < experts \
+                or extra >= logits.shape[1]:
             raise ValueError("moe_route_groups: logits must be float32 [N, >= %d] with unit column stride" % experts)
         if not (0 < top <= experts and top <= 64) or not (0 < keep <= groups <= 256) or experts % groups \
                 or keep * (experts // groups) < top:
@@ -835,10 +851,12 @@ class HipOps:
         N = logits.shape[0]
         choice = torch.empty((N, top), dtype=torch.int32, device=logits.device)
         weight = torch.empty((N, top), dtype=torch.float32, device=logits.device)
+        gate = torch.empty((N,), dtype=torch.float32, device=logits.device) if extra >= 0 else None
         self._check(self.lib.lmsf_moe_route_groups(_ptr(logits), logits.stride(0), N, int(experts), int(top),
                                                    1 if softmax else 0, int(groups), int(keep), 1 if renorm else 0,
-                                                   _ptr(choice), _ptr(weight), self._stream()))
-        return choice, weight
+                                                   _ptr(correction), float(scale), int(extra), _ptr(choice), _ptr(weight),
+                                                   _ptr(gate), self._stream()))
+        return (choice, weight, gate) if extra >= 0 else (choice, weight)
 
     def moe_route(self, logits: torch.Tensor, experts: int, top: int, renorm: bool = False, extra: int = -1):
         """A router's choice from float32 logits [N, >= experts]: (choice int32 [N, top], weight float32 [N, top],
@@ -1079,6 +1097,132 @@ class HipOps:
         self._check(self.lib.lmsf_head_rms_gate(
             _ptr(raw), raw.stride(0), _ptr(weight), _ptr(gate), gate.stride(0) if gate is not None else 0, act, _ptr(out),
             out.stride(0), _code(out_dtype), N, int(heads), int(vdim), float(eps), self._stream()))
+        return out
+
+    # ------------------------------------------------------------------ a residual of several streams
+
+    def stream_embedding(self, ids: torch.Tensor, table: torch.Tensor, streams: int, scale: float = 1.0) -> torch.Tensor:
+        """float32 [N, streams, W]: for every stream the rows of ``table`` [V, W] selected by int32 ``ids`` [N], times
+        ``scale``."""
+        self._dev(ids, table)
+        self._i32(ids, "ids")
+        if table.dim() != 2 or not table.is_contiguous():
+            raise ValueError("embedding table must be contiguous [V, W]")
+        n, (V, W) = ids.numel(), table.shape
+        out = torch.empty((n, streams, W), dtype=torch.float32, device=table.device)
+        self._check(self.lib.lmsf_stream_embedding(_ptr(ids), _ptr(table), _code(table.dtype), float(scale), _ptr(out), n,
+                                                   int(streams), V, W, _ptr(self._bad_token_flag(table.device)),
+                                                   self._stream()))
+        return out
+
+    def mix_streams(self, X: torch.Tensor, update: Optional[StreamUpdate] = None, read: Optional[torch.Tensor] = None,
+                    weight: Optional[torch.Tensor] = None, eps: float = 1e-5, out_dtype: Optional[torch.dtype] = None,
+                    rows: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+        """The streams ``X`` (contiguous float32 [N, s, W]) brought up to date by ``update``, in place, and with
+        ``weight`` (float32 [W]) the RMS norm of sum_s read_s X_s (``read`` float32 [s]; None: ones) times weight, in
+        ``out_dtype``. ``rows`` (int32): the norm at these tokens alone, of their streams as the update would leave them;
+        X is not written then."""
+        if X.dim() != 3 or X.dtype != torch.float32 or not X.is_contiguous():
+            raise ValueError("mix_streams: the streams must be contiguous float32 [N, s, W]")
+        N, s, W = X.shape
+        self._dev(X, read, weight, rows)
+        y = mix = add = None
+        if update is not None:
+            y, mix, add = update.y, update.mix, update.add
+            self._dev(y, mix, add)
+            if tuple(y.shape) != (N, W) or y.stride(1) != 1:
+                raise ValueError("mix_streams: the sublayer's result must be [%d, %d] with unit column stride" % (N, W))
+            self._f32_vec(mix, s * s, "mix_streams: mix")
+            self._f32_vec(add, s, "mix_streams: add")
+        elif weight is None:
+            raise ValueError("mix_streams: neither an update nor a norm")
+        dtype = out_dtype or (y.dtype if y is not None else torch.float32)
+        if y is not None and weight is not None and y.dtype != dtype:
+            raise ValueError("mix_streams: the sublayer's result and the norm's must be of one dtype")
+        for t, n, name in ((read, s, "read"), (weight, W, "weight")):
+            if t is not None:
+                self._f32_vec(t, n, "mix_streams: " + name)
+        self._i32(rows, "rows")
+        n_rows = N if rows is None else rows.numel()
+        out = torch.empty((n_rows, W), dtype=dtype, device=X.device) if weight is not None else None
+        self._check(self.lib.lmsf_mix_streams(
+            _ptr(X), s, _ptr(y), y.stride(0) if y is not None else 0, _ptr(mix), _ptr(add), _ptr(read), _ptr(weight),
+            float(eps), _ptr(rows), _ptr(out), _code(y.dtype if y is not None else dtype), n_rows, W, self._stream()))
+        return out
+
+    # ------------------------------------------------------------------ a recurrence with one decay a head
+
+    def state_space_state_floats(self, heads: int, n: int, vdim: int) -> int:
+        return int(self.lib.lmsf_state_space_state_floats(heads, n, vdim))
+
+    state_space_chunked_min_tokens = 16    # a step whose longest segment has as many tokens takes the chunked form
+
+    def state_space(self, xbc: torch.Tensor, x_at: int, b_at: int, c_at: int, dt: torch.Tensor, dt_bias: torch.Tensor,
+                    rate: torch.Tensor, d_skip: torch.Tensor, state: torch.Tensor, batch, heads: int, groups: int, n: int,
+                    vdim: int, form: Optional[str] = None) -> torch.Tensor:
+        """The linear recurrence over each request's tokens, the state [heads, vdim, n] carried in ``state`` (float32
+        [slots, >= state_space_state_floats]): with dt = softplus(``dt`` + dt_bias) (``dt`` float32 [N, >= heads]) and B, C
+        of a head's group, S <- exp(-rate dt) S + dt B x^T, y = S^T C + d_skip x. x: ``heads`` heads of vdim from column
+        x_at of ``xbc``; B, C: ``groups`` groups of n from b_at and c_at. Returns y as float32 [N, heads * vdim].
+        ``form`` forces "tokens" or "chunks" (tests)."""
+        self._dev(xbc, dt, dt_bias, rate, d_skip)
+        N = xbc.shape[0]
+        need = max(x_at + heads * vdim, b_at + groups * n, c_at + groups * n)
+        if xbc.dim() != 2 or xbc.stride(1) != 1 or xbc.shape[1] < need or heads % groups:
+            raise ValueError("state_space: xbc must be [N, >= %d] with unit column stride" % need)
+        if dt.dtype != torch.float32 or dt.dim() != 2 or dt.shape[0] != N or dt.shape[1] < heads or dt.stride(1) != 1:
+            raise ValueError("state_space: dt must be float32 [%d, >= %d]" % (N, heads))
+        for t, name in ((dt_bias, "dt_bias"), (rate, "rate"), (d_skip, "d_skip")):
+            self._f32_vec(t, heads, "state_space: " + name)
+        self._state_view(state, self.state_space_state_floats(heads, n, vdim), "state_space")
+        _, seg_starts, slots, S = self._segments(batch, N)
+        y = torch.empty((N, heads * vdim), dtype=torch.float32, device=xbc.device)
+        head = (_ptr(xbc), _code(xbc.dtype), xbc.stride(0), int(x_at), int(b_at), int(c_at), _ptr(dt), dt.stride(0),
+                _ptr(dt_bias), _ptr(rate), _ptr(d_skip), _ptr(state), state.stride(0))
+        tail = (_ptr(y), y.stride(0), N, S, int(heads), int(groups), int(n), int(vdim), self._stream())
+        L = self.lib.lmsf_state_space_chunk_tokens(_code(xbc.dtype), int(n), int(vdim))
+        lens = getattr(batch, "host_seg_lens", None)
+        chunks_ok = L > 0 and lens and not getattr(batch, "replayed", False)
+        if form == "chunks" and not chunks_ok:
+            raise ValueError("state_space: no chunked form for this step")
+        if form == "chunks" or (form is None and chunks_ok and not getattr(batch, "all_single", False)
+                                and max(lens) >= self.state_space_chunked_min_tokens):
+            key = ("state_space_chunks", L)
+            aux = getattr(batch, "aux", None)
+            plan = aux.get(key) if aux is not None else None
+            if plan is None:
+                rows, bases, at = [], [0], 0
+                for s, m in enumerate(lens):
+                    for t in range(0, m, L):
+                        rows += [at + t, min(L, m - t), s]
+                    at += m
+                    bases.append(len(rows) // 3)
+                both = self.upload_ints(rows + bases, xbc.device)
+                plan = (both[:len(rows)], both[len(rows):], len(rows) // 3)
+                if aux is not None:
+                    aux[key] = plan
+            chunks, bases, n_chunks = plan
+            entries = torch.empty(n_chunks * self.lib.lmsf_state_space_entry_floats(heads, n, vdim), dtype=torch.float32,
+                                  device=xbc.device)
+            self._check(self.lib.lmsf_state_space_chunked(*head, _ptr(slots), _ptr(chunks), _ptr(bases), n_chunks,
+                                                          _ptr(entries), *tail))
+            return y
+        self._check(self.lib.lmsf_state_space_tokens(*head, _ptr(seg_starts), _ptr(slots), *tail))
+        return y
+
+    def gated_group_norm(self, y: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, parts: int, eps: float) -> torch.Tensor:
+        """y silu(z) cut into ``parts`` equal pieces, each over its own root mean square, times ``weight`` (float32
+        [inner]): y float32 [N, inner], z [N, >= inner] with unit column stride; returns [N, inner] in z's dtype."""
+        self._dev(y, z, weight)
+        N, inner = y.shape
+        if y.dtype != torch.float32 or y.stride(1) != 1 or z.dim() != 2 or z.shape[0] != N or z.shape[1] < inner \
+                or z.stride(1) != 1 or inner % parts:
+            raise ValueError("gated_group_norm: y float32 [N, inner] and z [N, >= inner] with unit column stride, whole parts")
+        self._f32_vec(weight, inner, "gated_group_norm: weight")
+        out = torch.empty((N, inner), dtype=z.dtype, device=z.device)
+        self._check(self.lib.lmsf_gated_group_norm(_ptr(y), y.stride(0), _ptr(z), z.stride(0), _code(z.dtype), _ptr(weight),
+                                                   _ptr(out), out.stride(0), N, inner, int(parts), float(eps),
+                                                   self._stream()))
         return out
 
     # ------------------------------------------------------------------ layer scale, logit cap
@@ -1513,18 +1657,21 @@ class HipOps:
 
     # ------------------------------------------------------------------ feed-forward
 
-    def gated_act(self, gu: torch.Tensor, kind: str = "silu") -> torch.Tensor:
-        """act(gu[:, :I]) * gu[:, I:] for gu [N, 2I]; kind "silu", "gelu" (erf form) or "gelu_tanh"."""
+    def gated_act(self, gu: torch.Tensor, kind: str = "silu", limit: float = 0.0) -> torch.Tensor:
+        """act(gu[:, :I]) * gu[:, I:] for gu [N, 2I]; kind "silu", "gelu" (erf form), "gelu_tanh", or "bounded":
+        g sigmoid(1.702 g) (u + 1) with g = min(gu[:, :I], limit) and u = gu[:, I:] within [-limit, limit]."""
         self._dev(gu)
         if gu.dim() != 2 or gu.stride(1) != 1 or gu.shape[1] % 2 != 0:
             raise ValueError("gated_act input must be [N, 2I] with unit column stride")
-        kinds = {"silu": 0, "gelu": 1, "gelu_tanh": 2}
+        kinds = {"silu": 0, "gelu": 1, "gelu_tanh": 2, "bounded": 3}
         if kind not in kinds:
             raise ValueError("unknown activation %r (known: %s)" % (kind, ", ".join(kinds)))
+        if (kind == "bounded") != (limit > 0):
+            raise ValueError("a limit > 0 goes with the activation 'bounded'")
         N, I = gu.shape[0], gu.shape[1] // 2
         out = torch.empty((N, I), dtype=gu.dtype, device=gu.device)
-        self._check(self.lib.lmsf_gated_act(_ptr(gu), _ptr(out), _code(gu.dtype), N, I, gu.stride(0), kinds[kind],
-                                            self._stream()))
+        self._check(self.lib.lmsf_gated_act_limit(_ptr(gu), _ptr(out), _code(gu.dtype), N, I, gu.stride(0), kinds[kind],
+                                                  float(limit), self._stream()))
         return out
 
     # ------------------------------------------------------------------ matrix products
@@ -1645,16 +1792,17 @@ class HipOps:
         return self.linear(x, weight, bias, out_dtype=torch.float32)
 
     def linear_gated(self, x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor] = None,
-                     kind: str = "silu") -> torch.Tensor:
+                     kind: str = "silu", limit: float = 0.0) -> torch.Tensor:
         """act(x Wg^T + bg) * (x Wu^T + bu) for the fused weight [2 I, K] = [Wg; Wu] (bias [2 I] likewise);
         [M, I] in x's dtype. Where ``lmsf_route_linear_gated`` says so the activation is the epilogue of the
         product; otherwise the product and the activation kernel run one after the other. Both ways round
         the two products to the storage type before the activation, so they give the same bits wherever
         they add up K in the same order (the default tilings of the fused and the plain product do not: they
-        split K over 8 and over 16 waves). ``x`` may be a ``ScaledRows``."""
+        split K over 8 and over 16 waves). ``x`` may be a ``ScaledRows``. kind "bounded" takes its ``limit``
+        (``gated_act``)."""
         if weight.dim() != 2 or weight.shape[0] % 2 != 0:
             raise ValueError("linear_gated: weight must be [2 I, K]")
-        kinds = {"silu": 1, "gelu": 2, "gelu_tanh": 5}
+        kinds = {"silu": 1, "gelu": 2, "gelu_tanh": 5, "bounded": 6}
         if kind not in kinds:
             raise ValueError("unknown activation %r (known: %s)" % (kind, ", ".join(kinds)))
         M, I = x.shape[0], weight.shape[0] // 2
@@ -1667,10 +1815,12 @@ class HipOps:
         self.lib.lmsf_route_linear_gated(ctypes.byref(self._tun), ctypes.byref(self._shape(xt, weight, xt.dtype)),
                                          x.rows_per_tile if scaled else 0, x.tiles if scaled else 0, ctypes.byref(rt))
         if rt.route == D.MATERIALIZE:
-            return self.linear_gated(self.materialize(x), weight, bias, kind)
-        if rt.route == D.SEPARATE or (kind == "gelu_tanh" and rt.route not in (D.GEMV, D.SKINNY)):
-            # (the tanh form of GELU is an epilogue of the one-row and the few-rows product only)
-            return self.gated_act(self.linear(self.materialize(x), weight, bias), kind)
+            return self.linear_gated(self.materialize(x), weight, bias, kind, limit)
+        if (kind == "bounded") != (limit > 0):
+            raise ValueError("a limit > 0 goes with the activation 'bounded'")
+        if rt.route == D.SEPARATE or (kind in ("gelu_tanh", "bounded") and rt.route not in (D.GEMV, D.SKINNY)):
+            # (these two are epilogues of the one-row and the few-rows product only)
+            return self.gated_act(self.linear(self.materialize(x), weight, bias), kind, limit)
         self._dev(xt, weight, bias)
         if bias is not None and (bias.shape != (2 * I,) or bias.dtype != weight.dtype or not bias.is_contiguous()):
             raise ValueError("linear_gated: bias must be [%d] of the weight's dtype" % (2 * I))
@@ -1690,10 +1840,11 @@ class HipOps:
             self._check(self.lib.lmsf_gemm_skinny_scaled(*head, y.stride(0), M, I, K, kinds[kind], _ptr(x.sumsq),
                                                          x.tiles, x.eps, self.skinny_variant, self._stream()))
         elif rt.route == D.GEMV:
-            self._check(self.lib.lmsf_gemv(*head, BF16, y.stride(0), M, I, K, kinds[kind], self._stream()))
+            self._check(self.lib.lmsf_gemv_limit(*head, BF16, y.stride(0), M, I, K, kinds[kind], float(limit),
+                                                 self._stream()))
         else:
-            self._check(self.lib.lmsf_gemm_skinny(*head, BF16, y.stride(0), M, I, K, self.skinny_variant, kinds[kind],
-                                                  self._stream()))
+            self._check(self.lib.lmsf_gemm_skinny_limit(*head, BF16, y.stride(0), M, I, K, self.skinny_variant, kinds[kind],
+                                                        float(limit), self._stream()))
         return y
 
     def _linear_mid(self, x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor], act: int,

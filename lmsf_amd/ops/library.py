@@ -10,7 +10,7 @@ from typing import Optional
 from ..csrc import build as _build
 from .dispatch import ProductShape, Route, Tunables
 
-ABI_VERSION = 35
+ABI_VERSION = 36
 
 _lib: Optional[ctypes.CDLL] = None
 _lib_path: Optional[str] = None
@@ -40,12 +40,12 @@ _SIGNATURES = {
                                                  c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_int, _P, c_int,
                                                  _P]),
     "lmsf_paged_attention_generic_biased": (c_int, [_P, c_long, _P, c_long, _P, _P, c_long, _P, c_int, _P, _P, c_int,
-                                                    c_int, c_int, c_int, c_int, c_float, c_int, c_float, _P, c_int, _P]),
+                                                    c_int, c_int, c_int, c_int, c_float, c_int, c_float, _P, _P, c_int, _P]),
     "lmsf_paged_attention_prefill_mfma_biased": (c_int, [_P, c_long, _P, c_long, _P, _P, c_long, _P, c_int, _P, c_int, _P,
                                                          _P, c_int, c_int, c_int, c_int, c_float, c_int, c_float, _P,
-                                                         c_int, _P]),
+                                                         _P, c_int, _P]),
     "lmsf_paged_attention_decode_mfma_biased": (c_int, [_P, c_long, _P, c_long, _P, _P, c_long, _P, c_int, _P, c_int, _P,
-                                                        _P, c_int, c_int, c_int, c_int, c_float, c_int, c_float, _P, c_int,
+                                                        _P, c_int, c_int, c_int, c_int, c_float, c_int, c_float, _P, _P, c_int,
                                                         c_int, _P, c_int, _P]),
     "lmsf_position_embedding": (c_int, [_P, _P, _P, _P, c_int, c_float, _P, _P, c_int, c_int, c_int, c_int, _P, _P]),
     "lmsf_linear_recurrence_entry_floats": (c_long, [c_int]),
@@ -71,8 +71,19 @@ _SIGNATURES = {
                                  c_int, _P]),
     "lmsf_head_rms_gate": (c_int, [_P, c_long, _P, _P, c_long, c_int, _P, c_long, c_int, c_int, c_int, c_int, c_float, _P]),
     "lmsf_table_moe_act": (c_int, [_P, c_int, c_long, _P, _P, _P, _P, c_int, c_int, c_int, c_float, _P, c_long, _P, _P, _P,
-                                   c_int, _P, _P, c_long, c_int, c_int, c_int, _P, _P, _P]),
-    "lmsf_moe_route_groups": (c_int, [_P, c_long, c_int, c_int, c_int, c_int, c_int, c_int, c_int, _P, _P, _P]),
+                                   c_int, c_float, c_int, _P, _P, c_long, c_int, c_int, c_int, _P, _P, _P]),
+    "lmsf_moe_route_groups": (c_int, [_P, c_long, c_int, c_int, c_int, c_int, c_int, c_int, c_int, _P, c_float, c_int, _P,
+                                      _P, _P, _P]),
+    "lmsf_mix_streams": (c_int, [_P, c_int, _P, c_long, _P, _P, _P, _P, c_float, _P, _P, c_int, c_int, c_int, _P]),
+    "lmsf_stream_embedding": (c_int, [_P, _P, c_int, c_float, _P, c_int, c_int, c_int, c_int, _P, _P]),
+    "lmsf_state_space_state_floats": (c_long, [c_int, c_int, c_int]),
+    "lmsf_state_space_chunk_tokens": (c_int, [c_int, c_int, c_int]),
+    "lmsf_state_space_entry_floats": (c_long, [c_int, c_int, c_int]),
+    "lmsf_state_space_tokens": (c_int, [_P, c_int, c_long, c_int, c_int, c_int, _P, c_long, _P, _P, _P, _P, c_long, _P, _P,
+                                        _P, c_long, c_int, c_int, c_int, c_int, c_int, c_int, _P]),
+    "lmsf_state_space_chunked": (c_int, [_P, c_int, c_long, c_int, c_int, c_int, _P, c_long, _P, _P, _P, _P, c_long, _P, _P,
+                                         _P, c_int, _P, _P, c_long, c_int, c_int, c_int, c_int, c_int, c_int, _P]),
+    "lmsf_gated_group_norm": (c_int, [_P, c_long, _P, c_long, c_int, _P, _P, c_long, c_int, c_int, c_int, c_float, _P]),
     "lmsf_group_norm": (c_int, [_P, c_int, c_long, _P, _P, _P, c_long, c_int, _P, _P, _P, c_int, c_long, _P, c_int, c_int,
                                 c_int, c_float, c_float, _P]),
     "lmsf_norm_add_fits": (c_int, [c_int]),
@@ -119,8 +130,11 @@ _SIGNATURES = {
                                   c_int, _P]),
     "lmsf_head_gate": (c_int, [_P, c_int, c_long, c_int, _P, c_long, _P, c_long, c_int, c_int, c_int, _P]),
     "lmsf_rms_pair": (c_int, [_P, c_long, _P, c_long, c_int, _P, _P, _P, c_int, c_int, c_float, c_float, _P]),
+    "lmsf_gated_act_limit": (c_int, [_P, _P, c_int, c_int, c_int, c_long, c_int, c_float, _P]),
     "lmsf_gated_act": (c_int, [_P, _P, c_int, c_int, c_int, c_long, c_int, _P]),
     "lmsf_gemm_plain": (c_int, [_P, c_int, c_long, _P, c_int, c_long, _P, _P, c_int, c_long, c_int, c_int, c_int, _P]),
+    "lmsf_gemm_skinny_limit": (c_int, [_P, c_long, _P, c_long, _P, _P, c_int, c_long, c_int, c_int, c_int, c_int, c_int,
+                                       c_float, _P]),
     "lmsf_gemm_skinny": (c_int, [_P, c_long, _P, c_long, _P, _P, c_int, c_long, c_int, c_int, c_int, c_int, c_int, _P]),
     "lmsf_gemm_qkv_rope_cache": (c_int, [_P, c_long, _P, c_long, _P, _P, c_long, c_int, c_int, _P, _P, c_int, _P, _P, _P,
                                          c_long, c_int, c_int, c_int, c_int, c_int, _P]),
@@ -130,6 +144,7 @@ _SIGNATURES = {
                                         c_float, c_int, _P]),
     "lmsf_gemm_qkv_rope_cache_scaled": (c_int, [_P, c_long, _P, c_long, _P, _P, c_long, c_int, c_int, _P, _P, c_int, _P,
                                                 _P, _P, c_long, c_int, c_int, c_int, c_int, _P, c_int, c_float, _P]),
+    "lmsf_gemv_limit": (c_int, [_P, c_long, _P, c_long, _P, _P, c_int, c_long, c_int, c_int, c_int, c_int, c_float, _P]),
     "lmsf_gemv": (c_int, [_P, c_long, _P, c_long, _P, _P, c_int, c_long, c_int, c_int, c_int, c_int, _P]),
     "lmsf_gemv_qkv_rope_cache": (c_int, [_P, c_long, _P, c_long, _P, _P, c_long, c_int, c_int, _P, _P, c_int, _P, _P, _P,
                                          c_long, c_int, c_int, c_int, c_int, _P]),

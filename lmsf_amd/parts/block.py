@@ -3,6 +3,7 @@ from typing import Optional
 
 import torch
 
+from ..ops.handles import StreamUpdate
 from .base import Block, CacheBinding, Part, Runtime, TensorDecl, build_part, register_part
 from .linear import Linear
 
@@ -408,3 +409,77 @@ class OutputNormBlock(Block):
         if self.hands_on:
             ctx.aux["stream_rounded"] = x
         return None
+
+
+class StreamMix(Part):
+    """How one sublayer reads and writes a residual of s streams: ``in`` [s] (what it reads is the weighted sum), ``mix``
+    [s, s] (from row to column: how the streams mix) and ``out`` [s] (how its result, times ``scale``, enters each)."""
+
+    graph_safe = True
+    recordable = False
+
+    def __init__(self, prefix: str, rt: Runtime, streams: int, scale: float):
+        super().__init__(prefix, rt)
+        self.s, self.scale = int(streams), float(scale)
+        self.read: Optional[torch.Tensor] = None
+        self.mix: Optional[torch.Tensor] = None
+        self.add: Optional[torch.Tensor] = None
+
+    def checkpoint_tensors(self):
+        # (random weights: every stream alike, mixed evenly)
+        even = "const:%r" % (1.0 / self.s)
+        return {self.prefix + ".in": TensorDecl((self.s,), init=even, keeps_float32=True),
+                self.prefix + ".out": TensorDecl((self.s,), init="ones", keeps_float32=True),
+                self.prefix + ".mix": TensorDecl((self.s, self.s), init=even, keeps_float32=True)}
+
+    def load_weights(self, fetch) -> None:
+        self.read = fetch(self.prefix + ".in").to(torch.float32).contiguous()
+        self.mix = fetch(self.prefix + ".mix").to(torch.float32).contiguous()
+        self.add = (fetch(self.prefix + ".out").to(torch.float32) * self.scale).contiguous()
+
+    def tensors(self):
+        return [t for t in (self.read, self.mix, self.add) if t is not None]
+
+
+@register_part("block", "stream_residual")
+class StreamResidualBlock(Block):
+    """Hyper-connections: a residual of s streams X [N, s, W], float32, and for every sublayer f numbers a, b [s] and M
+    [s, s] of its own (``StreamMix``):
+
+        y = f(norm(sum_u a_u X_u));   X_t <- sum_u M[u, t] X_u + scale b_t y
+
+    first the mixer, then the feed-forward (where there is one). An update is carried out by the kernel that reads the
+    streams next (``mix_streams``: update, weighted sum and norm in one launch): the block receives the previous block's
+    last result as a ``StreamUpdate`` and returns its own. The reference's residual is one stream
+    (core/src/model_executor/models/llama/llama.rs:286-340)."""
+
+    graph_safe = True
+    recordable = False
+
+    ROLES = ("input",)          # and "post_mixer" where there is a feed-forward
+
+    def __init__(self, prefix: str, rt: Runtime, mixer, feed_forward, norms, streams: int, scale: float = 1.0,
+                 names=("hc1", "hc2")):
+        super().__init__(prefix, rt, mixer, feed_forward, norms)
+        self.has_ffn = not getattr(feed_forward, "absent", False)
+        if self.has_ffn and "post_mixer" not in norms:
+            raise ValueError("block %s needs the norm post_mixer before its feed-forward" % prefix)
+        if any(getattr(n, "groups", 1) != 1 for n in norms.values()):
+            raise ValueError("block %s takes norms over whole rows" % prefix)
+        self.first = StreamMix("%s.%s" % (prefix, names[0]), rt, streams, scale)
+        self.second = StreamMix("%s.%s" % (prefix, names[1]), rt, streams, scale) if self.has_ffn else None
+
+    def children(self):
+        return super().children() + [m for m in (self.first, self.second) if m is not None]
+
+    def _open(self, mix: StreamMix, norm, update, X: torch.Tensor) -> torch.Tensor:
+        return self.rt.ops.mix_streams(X, update=update, read=mix.read, weight=norm.weight, eps=norm.eps,
+                                       out_dtype=self.rt.dtype)
+
+    def forward(self, branch, residual: torch.Tensor, ctx, binding: CacheBinding) -> StreamUpdate:
+        h = self._open(self.first, self.norms["input"], branch, residual)
+        y = StreamUpdate(self.mixer.forward(h, ctx, binding), self.first.mix, self.first.add)
+        if not self.has_ffn:
+            return y
+        h = self._open(self.second, self.norms["post_mixer"], y, residual)
+        return StreamUpdate(self.feed_forward.forward(h), self.second.mix, self.second.add)

@@ -136,6 +136,21 @@ class PositionedEmbedding(Part):
         return x
 
 
+@register_part("embedding", "stream_embedding")
+class StreamEmbedding(TokenEmbedding):
+    """The token's row as the start of every one of ``streams`` residual streams: float32 [N, streams, W]."""
+
+    recordable = False
+
+    def __init__(self, prefix: str, rt: Runtime, vocab_size: int, hidden_size: int, streams: int, scale: float = 1.0,
+                 weight_name: str = "weight"):
+        super().__init__(prefix, rt, vocab_size, hidden_size, scale, weight_name)
+        self.streams = int(streams)
+
+    def forward(self, token_ids: torch.Tensor) -> torch.Tensor:
+        return self.rt.ops.stream_embedding(token_ids, self.weight, self.streams, self.scale)
+
+
 @register_part("head", "lm_head")
 class LMHead(Part):
     """``weight_name`` is the full checkpoint name of the [V, H] matrix: the head's own, or the

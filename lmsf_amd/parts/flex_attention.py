@@ -13,7 +13,9 @@ or key, ``vdim`` a value. In the order in which they act, each optional:
 - score = q . k * scale, bounded by cap tanh(score / cap) (``softcap``), less r1_h ln(1 + r2_h (i - j)) for query i and
   key j, two numbers a head (``distance_bias``); causal, within a window of the last positions, or within the query's own chunk of
   ``chunk`` positions (chunks counted from position 0 of the request);
-- the concatenated heads times sigmoid(W_g h), elementwise, before the output projection.
+- a number a head whose exponential stands in the softmax's denominator beside the keys' (``sink``);
+- the concatenated heads times sigmoid(W_g h), elementwise (``output_gate``), or head h times sigmoid(W_g h)_h, one
+  number a head (``head_gate``), before the output projection.
 
 The attention kernels take one head size: the cache holds keys and values padded with zeros to
 D = max(dim, vdim) rounded up to 16 (zeros in a key change no score; the outputs that padded values give are
@@ -42,7 +44,8 @@ class FlexAttention(Mixer):
                  conv_taps: int = 0, unit_norm_eps: Optional[float] = None, temp_coef: float = 0.0, temp_every: int = 0,
                  window: Optional[int] = None, chunk: Optional[int] = None, output_gate: bool = False,
                  names: Optional[Dict[str, str]] = None, bias_name: str = "b", head_norm_weights: bool = False,
-                 softcap: float = 0.0, distance_bias: bool = False, weights_f32: bool = False):
+                 softcap: float = 0.0, distance_bias: bool = False, weights_f32: bool = False, sink: bool = False,
+                 head_gate: bool = False):
         super().__init__(prefix, rt)
         self.H, self.G, self.dim, self.vdim = int(num_heads), int(num_kv_heads), int(head_dim), int(v_head_dim)
         if self.H % self.G:
@@ -56,6 +59,9 @@ class FlexAttention(Mixer):
         if self.head_norm_weights and unit_norm_eps is None:
             raise ValueError("%s: weights of a head norm without its eps" % prefix)
         self.weights_f32 = bool(weights_f32)
+        self.has_sink, self.has_head_gate = bool(sink), bool(head_gate)
+        if self.has_head_gate and output_gate:
+            raise ValueError("%s: a gate per entry or one a head, not both" % prefix)
         self.window = int(window) if window else None
         self.chunk = int(chunk) if chunk else None
         self.unit_norm_eps = None if unit_norm_eps is None else float(unit_norm_eps)
@@ -64,20 +70,24 @@ class FlexAttention(Mixer):
         check = getattr(rt.ops, "check_head_dim", None)
         if check is not None:
             check(self.D, 1024)
-        nm = dict(q="q", k="k", v="v", g="g", o="o", conv="conv", q_norm="q.norm", k_norm="k.norm", r1="r1", r2="r2")
+        nm = dict(q="q", k="k", v="v", g="g", o="o", conv="conv", q_norm="q.norm", k_norm="k.norm", r1="r1", r2="r2", sink="sink")
         nm.update(names or {})
         self.nm = nm
         self.q_weight: Optional[torch.Tensor] = None       # float32 [dim]
         self.k_weight: Optional[torch.Tensor] = None
         self.distance: Optional[torch.Tensor] = None       # float32 [2, H]: r1, r2
+        self.sink: Optional[torch.Tensor] = None           # float32 [H]
         H, G = self.H, self.G
         self.n_qkv = (H + G) * self.dim + G * self.vdim
         sources = [(nm["q"], H * self.dim), (nm["k"], G * self.dim), (nm["v"], G * self.vdim)]
         self.has_gate = bool(output_gate)
         if self.has_gate:
             sources.append((nm["g"], H * self.vdim))
+        elif self.has_head_gate:
+            sources.append((nm["g"], H))
         bias = [nm["q"], nm["k"], nm["v"]] if qkv_bias else False
-        self.proj = FusedLinear(prefix, rt, hidden_size, sources, bias=bias, bare_names=True, bias_name=bias_name)
+        self.proj = FusedLinear(prefix, rt, hidden_size, sources, bias=bias, bare_names=True, bias_name=bias_name,
+                                pad_rows_to=8 if self.has_head_gate else 1)
         self.conv: Optional[ShortConv] = None
         if conv_taps and int(conv_taps) >= 1:          # (one tap: a weight per channel, and no state)
             self.conv = ShortConv(prefix, rt, [("%s.%s" % (nm[x], nm["conv"]), n) for x, n in zip("qkv", (
@@ -99,6 +109,8 @@ class FlexAttention(Mixer):
         if self.has_distance_bias:
             for what in ("r1", "r2"):
                 out[self._full(what)] = TensorDecl((self.H,), init="const:0.5", keeps_float32=True)
+        if self.has_sink:
+            out[self._full("sink")] = TensorDecl((self.H,), init="zeros", keeps_float32=True)
         return out
 
     def load_weights(self, fetch: Callable[[str], torch.Tensor]) -> None:
@@ -107,9 +119,11 @@ class FlexAttention(Mixer):
             self.k_weight = fetch(self._full("k_norm")).to(torch.float32).contiguous()
         if self.has_distance_bias:
             self.distance = torch.stack([fetch(self._full(w)).to(torch.float32) for w in ("r1", "r2")]).contiguous()
+        if self.has_sink:
+            self.sink = fetch(self._full("sink")).to(torch.float32).contiguous()
 
     def tensors(self):
-        return [t for t in (self.q_weight, self.k_weight, self.distance) if t is not None]
+        return [t for t in (self.q_weight, self.k_weight, self.distance, self.sink) if t is not None]
 
     def cache_spec(self) -> Optional[CacheSpec]:
         return CacheSpec(num_kv_heads=self.G, head_dim=self.D, window=self.window)
@@ -129,7 +143,7 @@ class FlexAttention(Mixer):
             if rotary is None or not rotary[2]:
                 raise ValueError("%s rotates pairs (i, i + rot/2) from a table" % self.prefix)
             table = rotary[0]
-        p = self.proj.forward(h)                                   # [N, q | k | v (| g)]
+        p = self.proj.forward(h)                                   # [N, q | k | v (| g) (| padding)]
         qkv = p[:, :self.n_qkv]
         if self.conv is not None:
             qkv = self.conv.forward(qkv, ctx, binding.state)
@@ -140,7 +154,9 @@ class FlexAttention(Mixer):
                               temp_every=self.temp_every, q_weight=self.q_weight, k_weight=self.k_weight)
         a = ops.paged_attention(qa, binding.k_pages, binding.v_pages, group.block_tables, ctx.seg_of_token,
                                 ctx.positions, H, G, D, self.scale, self.window or 0, batch=ctx, chunk=self.chunk or 0,
-                                weights_f32=self.weights_f32, softcap=self.softcap, distance_bias=self.distance)
-        if self.has_gate or D != vdim:
+                                weights_f32=self.weights_f32, softcap=self.softcap, distance_bias=self.distance, sink=self.sink)
+        if self.has_head_gate:
+            a = ops.attn_finish(a, D, H, vdim, ctx.positions, gate=p[:, self.n_qkv:self.n_qkv + H])
+        elif self.has_gate or D != vdim:
             a = ops.head_gate(a, D, H, vdim, gate=p[:, self.n_qkv:] if self.has_gate else None)
         return self.o.forward(a)

@@ -67,6 +67,17 @@ class GroupRMSNorm(Norm):
             out_dtype=self.rt.dtype, history=history, index=index, mix=mix, want_out=then is not None)
 
 
+@register_part("norm", "stream_sum_norm")
+class StreamSumNorm(GroupRMSNorm):
+    """The RMS norm of the sum of a residual's streams [N, s, W], the last sublayer's result (``StreamUpdate``) taken on
+    the way."""
+
+    def forward_add(self, branch, residual: torch.Tensor, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """At ``rows`` the streams are left as they were (the end of a model)."""
+        return self.rt.ops.mix_streams(residual, update=branch, weight=self.weight, eps=self.eps, out_dtype=self.rt.dtype,
+                                       rows=rows)
+
+
 @register_part("norm", "depth_mix")
 class DepthMix(Part):
     """The weights of the average over the results of the layers so far: one per result, float32."""

@@ -119,6 +119,6 @@ class Linear(FusedLinear):
     """A single checkpoint matrix ``prefix.name.weight`` [out_features, in_features]."""
 
     def __init__(self, prefix: str, rt: Runtime, name: str, in_features: int, out_features: int, bias: bool = False,
-                 bare_names: bool = False, bias_name: str = "bias", row_order=None):
+                 bare_names: bool = False, bias_name: str = "bias", row_order=None, pad_rows_to: int = 1):
         super().__init__(prefix, rt, in_features, [(name, out_features)], bias, bare_names, bias_name,
-                         row_orders={name: row_order} if row_order is not None else None)
+                         row_orders={name: row_order} if row_order is not None else None, pad_rows_to=pad_rows_to)

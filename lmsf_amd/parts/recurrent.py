@@ -1,11 +1,11 @@
 """Mixers whose memory of a request is a state of fixed size: the selective scan, a matrix memory with
-exponential gates and a gated linear recurrence, and the short causal convolution that both they and some attention layers put behind a
-projection.
+exponential gates, a gated linear recurrence and a recurrence of matrices with one decay a head, and the short causal
+convolution that both they and some attention layers put behind a projection.
 
 A request's state is one row of float32 numbers in the engine's state slots (``StateSpec``); a mixer says how
 many it needs and gets ``binding.state`` [slots, that many]. The engine clears a row when a request takes it, so
 "zeros before the sequence's start" and "the state starts at zero" need no code here. Everything that enters a
-recurrence is float32 (csrc/recurrent.hip, csrc/linear_recurrence.hip); the projections run in the run's dtype. The reference has no mixer
+recurrence is float32 (csrc/recurrent.hip, csrc/linear_recurrence.hip, csrc/state_space.hip); the projections run in the run's dtype. The reference has no mixer
 with state (its only one is attention over a paged cache, core/src/model_executor/layers/attention.rs:91-231).
 """
 from typing import Callable, Dict, Optional, Sequence, Tuple
@@ -59,12 +59,15 @@ class ShortConv(Part):
 
 
 class FloatVector(Part):
-    """A checkpoint tensor that is kept in float32 whatever the run's dtype (what enters a recurrence)."""
+    """A checkpoint tensor that is kept in float32 whatever the run's dtype (what enters a recurrence); ``transform``:
+    what is kept is this function of it."""
 
     graph_safe = True
 
-    def __init__(self, name: str, rt: Runtime, shape: Tuple[int, ...], init: str = "normal"):
+    def __init__(self, name: str, rt: Runtime, shape: Tuple[int, ...], init: str = "normal",
+                 transform: Optional[Callable[[torch.Tensor], torch.Tensor]] = None):
         super().__init__(name, rt)
+        self.transform = transform
         self.shape, self.init = tuple(shape), init
         self.weight: Optional[torch.Tensor] = None
 
@@ -72,7 +75,8 @@ class FloatVector(Part):
         return {self.prefix: TensorDecl(self.shape, init=self.init, keeps_float32=True)}
 
     def load_weights(self, fetch: Callable[[str], torch.Tensor]) -> None:
-        self.weight = fetch(self.prefix).to(torch.float32).contiguous()
+        w = fetch(self.prefix).to(torch.float32)
+        self.weight = (self.transform(w) if self.transform is not None else w).contiguous()
 
 
 @register_part("mixer", "selective_scan")
@@ -226,3 +230,61 @@ class GatedLinearRecurrence(Mixer):
         u = self.conv.forward(p[:, self.C:], ctx, st[:, self.C:] if self.taps > 1 else None)
         o = self.rt.ops.linear_recurrence(u, self.wr, self.br, self.wi, self.bi, self.rate, p[:, :self.C], st, ctx)
         return self.o.forward(o)
+
+
+@register_part("mixer", "state_space")
+class StateSpace(Mixer):
+    """Mamba-2's mixer. inner = heads * vdim; [z | x | B | C | dt] = W_in h with B and C of ``groups`` groups of ``state``
+    entries and one dt a head; [x | B | C] <- silu(conv(.) + b); dt <- softplus(dt + dt_bias). Per head, with B and C of
+    its group: S <- exp(-exp(A_log) dt) S + dt B x^T, y = S^T C + D x. The heads' y, concatenated, times silu(z), then an
+    RMS norm in ``norm_groups`` equal parts times a weight, then W_o. State of a request: S of every head and the
+    convolution's last taps - 1 inputs."""
+
+    graph_safe = True
+    recordable = False
+
+    def __init__(self, prefix: str, rt: Runtime, hidden_size: int, heads: int, vdim: int, state: int, groups: int, conv: int,
+                 eps: float, norm_groups: int = 1, names: Optional[Dict[str, str]] = None):
+        super().__init__(prefix, rt)
+        self.H, self.dv, self.n, self.G, self.taps = int(heads), int(vdim), int(state), int(groups), int(conv)
+        self.norm_groups, self.eps = int(norm_groups), float(eps)
+        self.inner = self.H * self.dv
+        if min(self.H, self.dv, self.n, self.G, self.taps, self.norm_groups) < 1 or self.H % self.G \
+                or self.inner % self.norm_groups or self.n > 1024:
+            raise ValueError("%s: %d heads of %d x %d (states of at most 1,024 rows) in %d groups, normed in %d parts"
+                             % (prefix, self.H, self.n, self.dv, self.G, self.norm_groups))
+        nm = dict(in_proj="in", conv="conv", conv_bias="conv.b", dt_bias="dt_bias", a_log="A_log", d="D", norm="norm",
+                  out="o")
+        nm.update(names or {})
+        self.channels = self.inner + 2 * self.G * self.n
+        self.n_main = self.inner + self.channels          # z | x | B | C: a product in the run's type; dt's is float32
+        self.in_proj = Linear(prefix, rt, nm["in_proj"], hidden_size, self.n_main + self.H, bare_names=True, pad_rows_to=8)
+        self.conv = ShortConv(prefix, rt, [(nm["conv"], self.channels)], self.taps, bias_name=nm["conv_bias"],
+                              activation="silu")
+        self.dt_bias = FloatVector("%s.%s" % (prefix, nm["dt_bias"]), rt, (self.H,), init="zeros")
+        self.rate = FloatVector("%s.%s" % (prefix, nm["a_log"]), rt, (self.H,), init="const:0.0", transform=torch.exp)
+        self.d = FloatVector("%s.%s" % (prefix, nm["d"]), rt, (self.H,), init="ones")
+        self.norm = FloatVector("%s.%s" % (prefix, nm["norm"]), rt, (self.inner,), init="ones")
+        self.o = Linear(prefix, rt, nm["out"], self.inner, hidden_size, bare_names=True)
+        sizer = getattr(rt.ops, "state_space_state_floats", None)
+        floats = int(sizer(self.H, self.n, self.dv)) if sizer is not None else self.H * self.n * self.dv
+        self.state_floats = (floats + 3) // 4 * 4         # (the convolution's part begins at a multiple of 16 bytes)
+
+    def children(self):
+        return [self.in_proj, self.conv, self.dt_bias, self.rate, self.d, self.norm, self.o]
+
+    def state_spec(self) -> Optional[StateSpec]:
+        total = self.state_floats + self.conv.state_floats
+        return StateSpec(((total + 3) // 4 * 4,), torch.float32)
+
+    def forward(self, h: torch.Tensor, ctx, binding: CacheBinding) -> torch.Tensor:
+        ops = self.rt.ops
+        st = binding.state
+        w = self.in_proj.weight
+        p = ops.linear(h, w[:self.n_main])                                       # [N, z | x | B | C]
+        dt = ops.linear_wide(h, w[self.n_main:], None)                           # float32 [N, >= H]: step sizes
+        u = self.conv.forward(p[:, self.inner:], ctx, st[:, self.state_floats:] if self.taps > 1 else None)
+        b_at = self.inner
+        y = ops.state_space(u, 0, b_at, b_at + self.G * self.n, dt, self.dt_bias.weight, self.rate.weight, self.d.weight, st, ctx,
+                            self.H, self.G, self.n, self.dv)
+        return self.o.forward(ops.gated_group_norm(y, p[:, :self.inner], self.norm.weight, self.norm_groups, self.eps))

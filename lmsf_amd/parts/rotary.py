@@ -24,6 +24,21 @@ import torch
 from .base import PositionEncoding, Runtime, register_part
 
 
+def yarn_frequencies(rotary_dim: int, theta: float, scaling: Mapping[str, Any]) -> torch.Tensor:
+    """float64 [rotary_dim / 2]: the frequencies under "yarn" scaling."""
+    factor, orig = float(scaling["factor"]), float(scaling["original_max_position_embeddings"])
+
+    def turn(t: float) -> float:
+        return rotary_dim * math.log(orig / (2.0 * math.pi * t)) / (2.0 * math.log(theta))
+
+    lo = max(math.floor(turn(float(scaling["beta_fast"]))), 0)
+    hi = min(math.ceil(turn(float(scaling["beta_slow"]))), rotary_dim - 1)
+    idx = torch.arange(rotary_dim // 2, dtype=torch.float64)
+    f = torch.pow(torch.tensor(float(theta), dtype=torch.float64), -2.0 * idx / rotary_dim)
+    ramp = torch.clamp((idx - lo) / max(hi - lo, 0.001), 0.0, 1.0)
+    return f / factor * ramp + f * (1.0 - ramp)
+
+
 def inverse_frequencies(rotary_dim: int, theta: float, scaling: Optional[Mapping[str, Any]]) -> torch.Tensor:
     """float32 [rotary_dim / 2]."""
     exponent = torch.arange(0, rotary_dim, 2, dtype=torch.float32) / float(rotary_dim)
@@ -32,17 +47,7 @@ def inverse_frequencies(rotary_dim: int, theta: float, scaling: Optional[Mapping
     if kind == "default":
         return inv
     if kind == "yarn":
-        factor, orig = float(scaling["factor"]), float(scaling["original_max_position_embeddings"])
-
-        def turn(t: float) -> float:
-            return rotary_dim * math.log(orig / (2.0 * math.pi * t)) / (2.0 * math.log(theta))
-
-        lo = max(math.floor(turn(float(scaling["beta_fast"]))), 0)
-        hi = min(math.ceil(turn(float(scaling["beta_slow"]))), rotary_dim - 1)
-        idx = torch.arange(rotary_dim // 2, dtype=torch.float64)
-        f = torch.pow(torch.tensor(float(theta), dtype=torch.float64), -2.0 * idx / rotary_dim)
-        ramp = torch.clamp((idx - lo) / max(hi - lo, 0.001), 0.0, 1.0)
-        return (f / factor * ramp + f * (1.0 - ramp)).to(torch.float32)
+        return yarn_frequencies(rotary_dim, theta, scaling).to(torch.float32)
     if kind != "llama3":
         raise ValueError("rotary scaling %r is not supported (default, llama3, yarn)" % kind)
     factor = float(scaling["factor"])
@@ -74,9 +79,9 @@ class RotaryEncoding(PositionEncoding):
                  scaling: Optional[Mapping[str, Any]] = None, style: str = "neox", angles: str = "float32"):
         super().__init__(prefix, rt)
         # "float64": frequencies, angles, cosines and sines are worked out in float64 and rounded once, into the
-        # float32 table (unscaled frequencies only); "float32": in float32 throughout, as the reference does
-        if angles not in ("float32", "float64") or (angles == "float64" and scaling):
-            raise ValueError("rotary angles %r unknown (float32, float64 without scaling)" % angles)
+        # float32 table (unscaled or "yarn" frequencies); "float32": in float32 throughout, as the reference does
+        if angles not in ("float32", "float64") or (angles == "float64" and scaling and scaling.get("rope_type") != "yarn"):
+            raise ValueError("rotary angles %r unknown (float32, float64 without scaling or with yarn)" % angles)
         self.angles = angles
         self.head_dim = int(head_dim)
         self.rotary_dim = int(rotary_dim) if rotary_dim else self.head_dim
@@ -96,10 +101,14 @@ class RotaryEncoding(PositionEncoding):
     def load_weights(self, fetch: Callable[[str], torch.Tensor]) -> None:
         key = self._key()
         if key not in self.rt.shared and self.angles == "float64":
-            idx = torch.arange(self.rotary_dim // 2, dtype=torch.float64)
-            inv = torch.pow(torch.tensor(self.theta, dtype=torch.float64), -2.0 * idx / self.rotary_dim)
+            if self.scaling:
+                inv = yarn_frequencies(self.rotary_dim, self.theta, self.scaling)
+            else:
+                idx = torch.arange(self.rotary_dim // 2, dtype=torch.float64)
+                inv = torch.pow(torch.tensor(self.theta, dtype=torch.float64), -2.0 * idx / self.rotary_dim)
             angles = torch.arange(self.rt.max_positions, dtype=torch.float64)[:, None] * inv[None, :]
-            table = torch.cat([torch.cos(angles), torch.sin(angles)], dim=1).to(torch.float32).contiguous()
+            table = torch.cat([torch.cos(angles), torch.sin(angles)], dim=1) * table_gain(self.scaling)
+            table = table.to(torch.float32).contiguous()
             self.rt.shared[key] = table.to(self.rt.device)
         if key not in self.rt.shared:
             inv = inverse_frequencies(self.rotary_dim, self.theta, self.scaling)

@@ -127,7 +127,7 @@ class TorchOps:
 
     # ------------------------------------------------------------ attention
     def paged_attention(self, q, k_pages, v_pages, block_tables, seg, pos, nh, nkv, d, scale, window=0, batch=None,
-                        kernel=None, chunk=0, weights_f32=False, softcap=0.0, distance_bias=None):
+                        kernel=None, chunk=0, weights_f32=False, softcap=0.0, distance_bias=None, sink=None):
         N = q.shape[0]
         ps = k_pages.shape[2]
         out = torch.empty((N, nh * d), dtype=q.dtype, device=q.device)
@@ -150,7 +150,9 @@ class TorchOps:
             if distance_bias is not None:
                 r1, r2 = distance_bias[0][:, None], distance_bias[1][:, None]
                 sc = sc - r1 * torch.log1p(r2 * (p - js).to(torch.float32)[None, :])
-            pr = torch.softmax(sc, dim=-1)
+            if sink is not None:          # one more exponential in the denominator, without a value
+                sc = torch.cat([sc, sink[:, None]], 1)
+            pr = torch.softmax(sc, dim=-1)[:, :len(js)]
             out[t] = torch.einsum("hn,nhd->hd", pr, vals).reshape(nh * d).to(q.dtype)
         return out
 
@@ -228,14 +230,20 @@ class TorchOps:
             out[:, h * out_head + out_at + width:(h + 1) * out_head] = 0
 
     def table_moe(self, h, w_gate_up, w_down, token_ids, table, weight, base=None, pair_scale=None, base_scale=None,
-                  out_scale=None, gated=True):
+                  out_scale=None, gated=True, limit=0.0, identity=0):
+        E = w_gate_up.shape[0]
         F = w_gate_up.shape[1] // 2 if gated else w_gate_up.shape[1]
         out = torch.zeros(h.shape, dtype=torch.float32)
         for n in range(h.shape[0]):
             for k, e in enumerate(table[int(token_ids[n]) if token_ids is not None else n].tolist()):
                 x = h[n].to(torch.float32) * (float(pair_scale[n, k]) if pair_scale is not None else 1.0)
+                if e >= E:
+                    out[n] += x * (float(out_scale[n, k]) if out_scale is not None else 1.0)
+                    continue
                 gu = (w_gate_up[e].to(torch.float32) @ x).to(h.dtype).to(torch.float32)
-                if gated:
+                if gated and limit > 0:
+                    a = self._bounded(gu[:F], gu[F:], limit).to(h.dtype).to(torch.float32)
+                elif gated:
                     a = (gu[:F] / (1.0 + torch.exp(-gu[:F])) * gu[F:]).to(h.dtype).to(torch.float32)
                 else:
                     a = (torch.relu(gu) ** 2).to(h.dtype).to(torch.float32)
@@ -257,20 +265,23 @@ class TorchOps:
         return order.to(torch.int32).contiguous(), w.contiguous(), gate
 
     # ------------------------------------------------------------ a token's extras, norms and rotated values, delta rule
-    def moe_route_groups(self, logits, experts, top, softmax=True, groups=1, keep=1, renorm=False):
+    def moe_route_groups(self, logits, experts, top, softmax=True, groups=1, keep=1, renorm=False, correction=None,
+                         scale=1.0, extra=-1):
         z = logits[:, :experts].to(torch.float32)
         sc = torch.softmax(z, -1) if softmax else torch.sigmoid(z)
         N = z.shape[0]
         per = experts // groups
-        best = z.reshape(N, groups, per).max(-1).values
+        key = z if correction is None else sc + correction
+        best = key.reshape(N, groups, per).max(-1).values
         kept = torch.zeros((N, groups), dtype=torch.bool)
         kept.scatter_(1, torch.topk(best, keep, -1).indices, True)
-        masked = z.masked_fill(~kept.repeat_interleave(per, 1), float("-inf"))
+        masked = key.masked_fill(~kept.repeat_interleave(per, 1), float("-inf"))
         choice = torch.topk(masked, top, -1).indices
         w = torch.gather(sc, 1, choice)
         if renorm:
-            w = w / w.sum(-1, keepdim=True)
-        return choice.to(torch.int32), w.contiguous()
+            w = w / (w.sum(-1, keepdim=True) + 1e-20)
+        out = choice.to(torch.int32), (w * scale).contiguous()
+        return out + (torch.sigmoid(logits[:, extra]).contiguous(),) if extra >= 0 else out
 
     def hashed_pair_embedding(self, batch, table, pairs, prev_state, mul_prev, mul_cur, keep=False):
         ids = batch.token_ids.long()
@@ -401,6 +412,48 @@ class TorchOps:
             g = gate[:, :heads * vdim].to(torch.float32).reshape(N, heads, vdim)
             y = y * (torch.sigmoid(g) if activation == "sigmoid" else g * torch.sigmoid(g))
         return y.reshape(N, heads * vdim).to(out_dtype)
+
+    def stream_embedding(self, ids, table, streams, scale=1.0):
+        return (table[ids.long()].to(torch.float32) * scale)[:, None].repeat(1, streams, 1)
+
+    def mix_streams(self, X, update=None, read=None, weight=None, eps=1e-5, out_dtype=None, rows=None):
+        new = X
+        if update is not None:
+            y = update.y.to(torch.float32)
+            new = torch.stack([sum(update.mix[s, t] * X[:, s] for s in range(X.shape[1])) + update.add[t] * y
+                               for t in range(X.shape[1])], 1)
+            if rows is None:
+                X.copy_(new)
+        if weight is None:
+            return None
+        if rows is not None:
+            new = new[rows.long()]
+        u = new.sum(1) if read is None else (new * read[None, :, None]).sum(1)
+        u = u / torch.sqrt((u * u).mean(-1, keepdim=True) + eps) * weight
+        return u.to(out_dtype or (update.y.dtype if update is not None else torch.float32))
+
+    def state_space_state_floats(self, heads, n, vdim):
+        return heads * n * vdim
+
+    def state_space(self, xbc, x_at, b_at, c_at, dt, dt_bias, rate, d_skip, state, batch, heads, groups, n, vdim, form=None):
+        N = xbc.shape[0]
+        v = xbc.to(torch.float32)
+        x = v[:, x_at:x_at + heads * vdim].reshape(N, heads, vdim)
+        rep = heads // groups
+        B, C = (v[:, at:at + groups * n].reshape(N, groups, n).repeat_interleave(rep, 1) for at in (b_at, c_at))
+        step = torch.nn.functional.softplus(dt[:, :heads] + dt_bias, threshold=30.0)
+        y = torch.empty((N, heads * vdim), dtype=torch.float32)
+        for a, b, slot in self._segments(batch):
+            S = state[slot, :heads * vdim * n].reshape(heads, vdim, n).clone()
+            for t in range(a, b):
+                S = torch.exp(-rate * step[t])[:, None, None] * S + x[t][:, :, None] * (step[t][:, None] * B[t])[:, None, :]
+                y[t] = ((S * C[t][:, None, :]).sum(-1) + d_skip[:, None] * x[t]).reshape(-1)
+            state[slot, :heads * vdim * n] = S.reshape(-1)
+        return y
+
+    def gated_group_norm(self, y, z, weight, parts, eps):
+        g = z.to(torch.float32)[:, :y.shape[1]]
+        return self._gn(y * (g / (1.0 + torch.exp(-g))), weight, parts, eps).to(z.dtype)
 
     def scale_add_norm(self, a, scale_a, b, scale_b, residual, weight=None, eps=1e-5):
         r = residual + scale_a * a.to(torch.float32)
@@ -600,7 +653,12 @@ class TorchOps:
         return (scale * (na + nb)).to(a.dtype)
 
     # ------------------------------------------------------------ feed-forward / linear
-    def gated_act(self, gu, kind="silu"):
+    @staticmethod
+    def _bounded(g, u, limit):
+        g, u = g.clamp(max=limit), u.clamp(-limit, limit)
+        return g * torch.sigmoid(1.702 * g) * (u + 1.0)
+
+    def gated_act(self, gu, kind="silu", limit=0.0):
         I = gu.shape[1] // 2
         g, u = gu[:, :I].to(torch.float32), gu[:, I:].to(torch.float32)
         if kind == "silu":
@@ -609,12 +667,14 @@ class TorchOps:
             a = 0.5 * g * (1.0 + torch.erf(g / math.sqrt(2.0)))
         elif kind == "gelu_tanh":
             a = 0.5 * g * (1.0 + torch.tanh(math.sqrt(2.0 / math.pi) * (g + 0.044715 * g * g * g)))
+        elif kind == "bounded":
+            return self._bounded(g, u, limit).to(gu.dtype)
         else:
             raise ValueError(kind)
         return (a * u).to(gu.dtype)
 
-    def linear_gated(self, x, weight, bias=None, kind="silu"):
-        return self.gated_act(self.linear(x, weight, bias), kind)
+    def linear_gated(self, x, weight, bias=None, kind="silu", limit=0.0):
+        return self.gated_act(self.linear(x, weight, bias), kind, limit)
 
     def linear(self, x, weight, bias=None, out_dtype=None, pending_ok=False, out=None):
         y = x.to(torch.float32) @ weight.to(torch.float32).t()
