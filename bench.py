@@ -593,6 +593,36 @@ def gurapel_run(args):
     beside_llama_run(args, "gurapel", args.gurapel_sizes, gurapel_shapes(args.gurapel_sizes), twin="murulorn")
 
 
+def zunilorn_shapes(name):
+    """A Zunilorn configuration at sizes that resemble a real model's layers, and beside it the Gurapel configuration of
+    equal width and number of layer runs (the closest architecture of the package: attention under a soft cap with float32
+    weights, a memory of matrices, gated experts chosen by a softmax router). Six layers of which the second and third run
+    twice, eight runs: Mamba-2 + dense, (attention + experts, Mamba-2 + experts) twice, Mamba-2 + experts, attention +
+    experts, Mamba-2 + experts; four streams; heads of 64 with states of 128 rows, twice the width in all; keys and values
+    of 128 entries, four query heads a key head; 2 experts a token of as many as Gurapel's and a quarter more that return
+    their input, and a shared one."""
+    gur, _ = gurapel_shapes(name)
+    W, H, E, eff, ff = {"2b": (2048, 16, 16, 1024, 8192), "7b": (4096, 32, 32, 2048, 14336)}[name]
+    att = {"heads": H, "kv_heads": H // 4, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "softcap": 30.0,
+           "rot": {"base": 1e6, "dims": 128, "scaling": {"factor": 4.0, "original": 2048, "fast": 32.0, "slow": 1.0}}}
+    ssm = {"heads": 2 * W // 64, "vdim": 64, "state": 128, "groups": 8, "conv": 4, "norm_groups": 8}
+    dense = {"kind": "dense", "ff": ff, "limit": 7.0}
+    moe = {"kind": "moe", "expert": {"ff": eff, "limit": 7.0}, "shared": {"ff": eff, "limit": 7.0},
+           "router": {"experts": E, "identity": E // 4, "top": 2, "scale": 1.5}}
+    kinds = [("mamba2", ssm, dense), ("attention", att, moe), ("mamba2", ssm, moe), ("mamba2", ssm, moe),
+             ("attention", att, moe), ("mamba2", ssm, moe)]
+    zun = {"architecture": "Zunilorn", "vocab": 32000, "width": W, "streams": 4, "residual_mult": 0.5, "norm": {"eps": 1e-6},
+           "logit_softcap": 30.0, "loop": {"start": 1, "stop": 3, "times": 2}, "max_position_embeddings": 8192,
+           "torch_dtype": "bfloat16", "layers": [{"type": t, "mixer": dict(m), "mlp": dict(f)} for t, m, f in kinds]}
+    return zun, gur
+
+
+def zunilorn_run(args):
+    """``--workload zunilorn``: prefill and decode of a Zunilorn model beside the Gurapel model of equal width and layer
+    runs; one JSON line, as for the other designs."""
+    beside_llama_run(args, "zunilorn", args.zunilorn_sizes, zunilorn_shapes(args.zunilorn_sizes), twin="gurapel")
+
+
 def prefill_flops(cfg, T):
     """Multiply-adds times two of a causal prefill of T tokens: the linear layers on every token, the
     attention scores and values over the causal half, the LM head on one row."""
@@ -616,14 +646,16 @@ def main():
     ap.add_argument("--max-num-batched-tokens", type=int, default=8192)
     ap.add_argument("--gpu-memory-utilization", type=float, default=0.85)
     ap.add_argument("--skip-points", action="store_true", help="leave out the batch 1 and batch 64 runs")
-    ap.add_argument("--workload", default="decode", choices=["decode", "serve", "products", "takosun", "niresun", "zevetar", "murulorn", "gurapel"],
+    ap.add_argument("--workload", default="decode", choices=["decode", "serve", "products", "takosun", "niresun", "zevetar", "murulorn", "gurapel",
+                                                                "zunilorn"],
                     help="decode: the default line (Llama-3-8B shape); serve: continuous batching of 64 requests at "
                          "Llama-2-7B shape, a line of its own; products: a layer's matrix products alone, the "
                          "library's against the engine's choice, at --rows; takosun: a Takosun model beside the Llama model "
                          "of equal size, prefill and decode; niresun: the same for a Niresun model; zevetar: a Zevetar "
                          "model beside the Takosun model of equal size; murulorn: a Murulorn model beside the Zevetar "
                          "model of equal width and layer runs; gurapel: a Gurapel model beside the Murulorn model of "
-                         "equal width and layers")
+                         "equal width and layers; zunilorn: a Zunilorn model beside the Gurapel model of equal width and "
+                         "layer runs")
     ap.add_argument("--takosun-sizes", default="2b", choices=["2b", "7b"], help="takosun: the layers' sizes")
     ap.add_argument("--niresun-sizes", default="2b", choices=["2b", "7b"],
                     help="niresun: the layers' sizes (a Niresun model beside the Llama model of equal size)")
@@ -633,6 +665,8 @@ def main():
                     help="murulorn: the layers' sizes (a Murulorn model beside the Zevetar model of equal width and layer runs)")
     ap.add_argument("--gurapel-sizes", default="2b", choices=["2b", "7b"],
                     help="gurapel: the layers' sizes (a Gurapel model beside the Murulorn model of equal width and layers)")
+    ap.add_argument("--zunilorn-sizes", default="2b", choices=["2b", "7b"],
+                    help="zunilorn: the layers' sizes (a Zunilorn model beside the Gurapel model of equal width and layer runs)")
     ap.add_argument("--rows", default="17,64,100,128,129,192,256,512,2048", help="products: numbers of rows")
     ap.add_argument("--prefill-chunk-size", type=int, default=1024, help="serve: longest portion of a prompt in a step")
     ap.add_argument("--shape", default="llama3-8b", choices=sorted(SHAPES),
@@ -679,6 +713,9 @@ def main():
         return
     if args.workload == "gurapel":
         gurapel_run(args)
+        return
+    if args.workload == "zunilorn":
+        zunilorn_run(args)
         return
     if args.workload == "zevetar":
         zevetar_run(args)

@@ -193,6 +193,7 @@ __global__ __launch_bounds__(256) void attn_finish_kernel(const T* __restrict__ 
     orow[i0] = from_f32<T>(x0 * gt);
     orow[i1] = from_f32<T>(x1 * gt);
   }
+  if (vdim % 2 && lane == 0) orow[vdim - 1] = from_f32<T>(to_f32<T>(ar[vdim - 1]) * gt);
 }
 
 // a [N, H D] (the attention's result), gate [N, >= H] (one pre-activation a head; null: none), out [N, H vdim]
@@ -201,7 +202,7 @@ extern "C" int lmsf_attn_finish(const void* a, long a_stride, const void* gate, 
                                 long out_stride, int n_tokens, int H, int vdim, int D, hipStream_t stream) {
   LMSF_CHECK(a && positions && out, "attn_finish: null pointer");
   LMSF_CHECK(dtype == LMSF_F32 || dtype == LMSF_BF16, "attn_finish: unknown dtype code %d", dtype);
-  LMSF_CHECK(H > 0 && vdim > 0 && vdim % 2 == 0 && D >= vdim && max_pos > 0 && a_stride >= (long)H * D &&
+  LMSF_CHECK(H > 0 && vdim > 0 && (vdim % 2 == 0 || !table_v) && D >= vdim && max_pos > 0 && a_stride >= (long)H * D &&
                  out_stride >= (long)H * vdim && (!gate || gate_stride >= H), "attn_finish: bad sizes");
   if (n_tokens <= 0) return 0;
   const dim3 grid((unsigned)(((long)n_tokens * H + 3) / 4));

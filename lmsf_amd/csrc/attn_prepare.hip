@@ -84,9 +84,9 @@ __global__ __launch_bounds__(256) void attn_prepare_kernel(
   }
 }
 
-// The same without rotation (which needs another lane's entry), for sizes that are multiples of 8 and rows and heads at
-// multiples of 16 bytes: L lanes a head (L a power of two, 8 L >= D), eight entries a lane in registers, 64 / L heads of a
-// token a wave.
+// The same for sizes that are multiples of 8 (the rotated part of 16) and rows and heads at multiples of 16 bytes: L lanes
+// a head (L a power of two, 8 L >= D), eight entries a lane in registers, 64 / L heads of a token a wave. A rotation's
+// partner entries are another lane's eight.
 template <typename T>
 __device__ __forceinline__ void ap_load8(const T* p, float* x) {
 #pragma unroll
@@ -110,8 +110,9 @@ __device__ __forceinline__ void ap_store8(T* p, const float* x) {
 template <typename T, int L>
 __global__ __launch_bounds__(256) void attn_prepare_rows_kernel(
     const T* __restrict__ q, long q_stride, const T* __restrict__ k, long k_stride, const T* __restrict__ v,
-    long v_stride, const int* __restrict__ positions, const int* __restrict__ slots, T* __restrict__ q_out,
-    long qo_stride, T* __restrict__ k_pages, T* __restrict__ v_pages, int n_tokens, int H, int G, int dim, int vdim,
+    long v_stride, const int* __restrict__ positions, const float* __restrict__ table, int rot, int max_pos,
+    const int* __restrict__ slots, T* __restrict__ q_out, long qo_stride, T* __restrict__ k_pages,
+    T* __restrict__ v_pages, int n_tokens, int H, int G, int dim, int vdim,
     int D, int ps, int unit_norm, float eps, const float* __restrict__ wq, const float* __restrict__ wk,
     float temp_coef, int temp_every) {
   constexpr int HPW = LMSF_WAVE / L;
@@ -136,12 +137,33 @@ __global__ __launch_bounds__(256) void attn_prepare_rows_kernel(
 #pragma unroll
     for (int j = 0; j < 8; ++j) x[j] *= inv;
   }
-  if (!live || e0 >= D || (!is_q && slot < 0)) return;
   const float* w = is_q ? wq : is_v ? nullptr : wk;
   if (w && e0 < dim) {
     const float4 a = *reinterpret_cast<const float4*>(w + e0), b = *reinterpret_cast<const float4*>(w + e0 + 4);
     x[0] *= a.x; x[1] *= a.y; x[2] *= a.z; x[3] *= a.w; x[4] *= b.x; x[5] *= b.y; x[6] *= b.z; x[7] *= b.w;
   }
+  const int p = table ? positions[t] : max_pos;
+  if (table && p < max_pos) {       // (the same for the whole wave: it holds heads of one token)
+    const int half = rot / 2;
+    const bool turns = e0 < rot, first = e0 < half;
+    const int from = turns ? lane + (first ? half / 8 : -(half / 8)) : lane;
+    float other[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) other[j] = __shfl(x[j], from, LMSF_WAVE);
+    if (turns && !is_v) {
+      const float* cs = table + (long)p * rot + (first ? e0 : e0 - half);
+      float c[8], sn[8];
+      ap_load8<float>(cs, c);
+      ap_load8<float>(cs + half, sn);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        float a, b;
+        if (first) rope_rotate(x[j], other[j], c[j], sn[j], &a, &b); else rope_rotate(other[j], x[j], c[j], sn[j], &b, &a);
+        x[j] = a;
+      }
+    }
+  }
+  if (!live || e0 >= D || (!is_q && slot < 0)) return;
   if (is_q) {
     if (temp_every > 0) {
       const float temp = 1.f + temp_coef * logf((float)((positions[t] + 1) / temp_every) + 1.f);
@@ -179,7 +201,7 @@ extern "C" int lmsf_attn_prepare(const void* q, long q_stride, const void* k, lo
   LMSF_CHECK(temp_every >= 0, "attn_prepare: negative temperature period");
   if (n_tokens == 0) return 0;
   const int al = dtype == LMSF_F32 ? 4 : 8;         // entries in 16 bytes
-  if (!table && D <= 512 && dim % 8 == 0 && vdim % 8 == 0 && D % 8 == 0 && q_stride % al == 0 && k_stride % al == 0 &&
+  if ((!table || (rot % 16 == 0 && lmsf_aligned16(table))) && D <= 512 && dim % 8 == 0 && vdim % 8 == 0 && D % 8 == 0 && q_stride % al == 0 && k_stride % al == 0 &&
       v_stride % al == 0 && qo_stride % al == 0 && lmsf_aligned16(q) && lmsf_aligned16(k) && lmsf_aligned16(v) &&
       lmsf_aligned16(q_out) && (!slots || (lmsf_aligned16(k_pages) && lmsf_aligned16(v_pages))) &&
       (!wq || lmsf_aligned16(wq)) && (!wk || lmsf_aligned16(wk))) {
@@ -188,7 +210,7 @@ extern "C" int lmsf_attn_prepare(const void* q, long q_stride, const void* k, lo
     const dim3 rgrid((unsigned)((waves + 3) / 4));
 #define AP_ROWS(T, LL)                                                                                                \
   hipLaunchKernelGGL((attn_prepare_rows_kernel<T, LL>), rgrid, dim3(256), 0, stream, (const T*)q, q_stride, (const T*)k, \
-                     k_stride, (const T*)v, v_stride, positions, slots, (T*)q_out, qo_stride, (T*)k_pages, (T*)v_pages, \
+                     k_stride, (const T*)v, v_stride, positions, table, rot, max_pos, slots, (T*)q_out, qo_stride, (T*)k_pages, (T*)v_pages, \
                      n_tokens, H, G, dim, vdim, D, ps, unit_norm, eps, wq, wk, temp_coef, temp_every)
 #define AP_L(T)                                                                                                      \
   do {                                                                                                               \

@@ -319,7 +319,8 @@ __global__ __launch_bounds__(256) void moe_tile_lds_kernel(const bf16_t* __restr
 }
 
 // out[n, o] = base[n, o] + weight * sum_k rows[n * top + k, o]; the choices of ``table`` (row ids[n], or n) from E on are
-// experts without matrices, which return their input
+// experts without matrices, which return their input. VEC: four neighbours a thread (W and the strides multiples of 4).
+template <bool VEC>
 __global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restrict__ rows, int top, float weight,
                                                           const bf16_t* __restrict__ base, long base_stride,
                                                           bf16_t* __restrict__ out, long out_stride, int W,
@@ -332,17 +333,47 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restric
   const int n = blockIdx.x;
   const int* chosen = table + (long)(identity > 0 ? min(max(ids ? ids[n] : n, 0), vocab - 1) : 0) * top;
   const float bs = base_scale ? base_scale[n] : 1.f;
-  for (int o = threadIdx.x; o < W; o += 256) {
-    float s = 0.f;
+  constexpr int V = VEC ? 4 : 1;
+  for (int o = threadIdx.x * V; o < W; o += 256 * V) {
+    float s[4], x[4];
+#pragma unroll
+    for (int j = 0; j < V; ++j) s[j] = 0.f;
+    auto bf4 = [&](const bf16_t* p) {
+      if (VEC) {
+        const uint2 v = *reinterpret_cast<const uint2*>(p);
+        x[0] = __uint_as_float(v.x << 16), x[1] = __uint_as_float(v.x & 0xffff0000u);
+        x[2] = __uint_as_float(v.y << 16), x[3] = __uint_as_float(v.y & 0xffff0000u);
+      } else {
+        x[0] = bf16_to_f32(p[0]);
+      }
+    };
     for (int k = 0; k < top; ++k) {
-      const float os = out_scale ? out_scale[(long)n * top + k] : 1.f;
-      if (identity > 0 && chosen[k] >= E)
-        s += os * (pair_scale ? pair_scale[(long)n * top + k] : 1.f) * bf16_to_f32(h[(long)n * h_stride + o]);
-      else
-        s += os * rows[((long)n * top + k) * W + o];
+      float f = out_scale ? out_scale[(long)n * top + k] : 1.f;
+      if (identity > 0 && chosen[k] >= E) {
+        bf4(h + (long)n * h_stride + o);
+        if (pair_scale) f *= pair_scale[(long)n * top + k];
+      } else {
+        const float* p = rows + ((long)n * top + k) * W + o;
+        if (VEC) {
+          const float4 v = *reinterpret_cast<const float4*>(p);
+          x[0] = v.x, x[1] = v.y, x[2] = v.z, x[3] = v.w;
+        } else {
+          x[0] = p[0];
+        }
+      }
+#pragma unroll
+      for (int j = 0; j < V; ++j) s[j] += f * x[j];
     }
-    const float b = base ? bs * bf16_to_f32(base[(long)n * base_stride + o]) : 0.f;
-    out[(long)n * out_stride + o] = f32_to_bf16(b + weight * s);
+#pragma unroll
+    for (int j = 0; j < V; ++j) s[j] *= weight;
+    if (base) {
+      bf4(base + (long)n * base_stride + o);
+#pragma unroll
+      for (int j = 0; j < V; ++j) s[j] = bs * x[j] + s[j];
+    }
+    bf16_t* y = out + (long)n * out_stride + o;
+    if (VEC) *reinterpret_cast<uint2*>(y) = make_uint2(pack2_bf16(s[0], s[1]), pack2_bf16(s[2], s[3]));
+    else y[0] = f32_to_bf16(s[0]);
   }
 }
 
@@ -398,9 +429,14 @@ extern "C" int lmsf_table_moe_act(const void* h, int dtype, long h_stride, const
     hipLaunchKernelGGL((moe_tile_lds_kernel<0>), dim3(max_tiles, (W + 127) / 128), dim3(256), 0, stream,
                        (const bf16_t*)act, (long)F, top, (const bf16_t*)Wd, order, tiles, n_tiles, (void*)scratch_rows, W,
                        F, (const float*)nullptr, 0.f);
-    hipLaunchKernelGGL(moe_combine_kernel, dim3(n_tokens), dim3(256), 0, stream, scratch_rows, top, weight,
-                       (const bf16_t*)base, base_stride, (bf16_t*)out, out_stride, W, base_scale, out_scale, ids, table,
-                       vocab, E, identity, (const bf16_t*)h, h_stride, pair_scale);
+    const bool vec = W % 4 == 0 && out_stride % 4 == 0 && h_stride % 4 == 0 && (!base || base_stride % 4 == 0) &&
+                     ((uintptr_t)out) % 8 == 0 && ((uintptr_t)base) % 8 == 0 && lmsf_aligned16(scratch_rows);
+#define MOE_COMBINE(V)                                                                                                \
+  hipLaunchKernelGGL((moe_combine_kernel<V>), dim3(n_tokens), dim3(256), 0, stream, scratch_rows, top, weight,        \
+                     (const bf16_t*)base, base_stride, (bf16_t*)out, out_stride, W, base_scale, out_scale, ids, table, \
+                     vocab, E, identity, (const bf16_t*)h, h_stride, pair_scale)
+    if (vec) MOE_COMBINE(true); else MOE_COMBINE(false);
+#undef MOE_COMBINE
     LMSF_LAUNCH_CHECK("table_moe (grouped)");
     return 0;
   }
@@ -530,7 +566,7 @@ __global__ __launch_bounds__(256) void moe_route_groups_kernel(const float* __re
   for (int i = 0; i < 4; ++i) {
     const int g = lane + LMSF_WAVE * i;
     gbest[i] = -INFINITY;
-    if (g < groups)
+    if (g < groups && keep < groups)
       for (int e = g * per; e < (g + 1) * per; ++e) gbest[i] = fmaxf(gbest[i], key(e));
   }
   if (keep >= groups) kept = 0xFu;

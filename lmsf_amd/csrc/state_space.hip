@@ -25,6 +25,7 @@
 
 #define SS_L 64              // tokens of a chunk
 #define SS_MAX_STATE 1024    // N
+#define SS_PT (4 * 2 * 3 * 64 * 16)   // bytes of a chunk's decayed C . B in parts
 
 __device__ __forceinline__ float ss_softplus(float x) { return x > 20.f ? x : log1pf(expf(x)); }
 
@@ -40,6 +41,12 @@ __device__ __forceinline__ void ss_load4(const bf16_t* p, float* x) {
   const uint2 v = *reinterpret_cast<const uint2*>(p);
   x[0] = __uint_as_float(v.x << 16), x[1] = __uint_as_float(v.x & 0xffff0000u);
   x[2] = __uint_as_float(v.y << 16), x[3] = __uint_as_float(v.y & 0xffff0000u);
+}
+__device__ __forceinline__ void ss_store4(float* p, const float* x) {
+  *reinterpret_cast<float4*>(p) = make_float4(x[0], x[1], x[2], x[3]);
+}
+__device__ __forceinline__ void ss_store4(bf16_t* p, const float* x) {
+  *reinterpret_cast<uint2*>(p) = make_uint2(pack2_bf16(x[0], x[1]), pack2_bf16(x[2], x[3]));
 }
 // four neighbours from entry n of n_all on (VEC: whole groups at aligned places; else entries beyond the end are zeros)
 template <bool VEC, typename T>
@@ -355,9 +362,9 @@ __global__ __launch_bounds__(256) void state_space_outputs_kernel(
   const int Nk = (N + 31) / 32 * 32, dvp = (dv + 15) / 16 * 16, row_bytes = Nk * 2 + 16;
   unsigned char* Cs = lds;                              // [64][row_bytes]
   unsigned char* Bs = Cs + SS_L * row_bytes;            // [64][row_bytes]
-  unsigned char* XT = Bs + SS_L * row_bytes;            // [dvp][64] turned
-  unsigned char* PT = XT + dvp * 128;                   // 24 KB
-  float* sdt = reinterpret_cast<float*>(PT + 4 * 2 * 3 * 64 * 16);
+  unsigned char* XT = Bs + max(SS_L * row_bytes, SS_PT);   // [dvp][64] turned
+  unsigned char* PT = Bs;                               // (takes B's place once every wave has multiplied)
+  float* sdt = reinterpret_cast<float*>(XT + dvp * 128);
   float* shi = sdt + SS_L;
   float* slo = shi + SS_L;
   const int h = blockIdx.x, g = h / (H / G);
@@ -408,6 +415,7 @@ __global__ __launch_bounds__(256) void state_space_outputs_kernel(
       }
     }
     const float hi = shi[t], lo = slo[t];
+    __syncthreads();
 #pragma unroll
     for (int pair = 0; pair < 2; ++pair) {
       if (pair * 2 > wave) continue;
@@ -501,8 +509,8 @@ static size_t ss_sums_smem(int N, int dv) {
   return (size_t)((N + 15) / 16 * 16 + (dv + 15) / 16 * 16) * 128 + 4 * SS_L * sizeof(float);
 }
 static size_t ss_outputs_smem(int N, int dv) {
-  return (size_t)2 * SS_L * ((N + 31) / 32 * 64 + 16) + (size_t)(dv + 15) / 16 * 16 * 128 + 4 * 2 * 3 * 64 * 16 +
-         3 * SS_L * sizeof(float);
+  const int rows = SS_L * ((N + 31) / 32 * 64 + 16);
+  return (size_t)rows + (rows > SS_PT ? rows : SS_PT) + (size_t)(dv + 15) / 16 * 16 * 128 + 3 * SS_L * sizeof(float);
 }
 
 // tokens of a chunk of the chunked form; 0: its operands do not fit a workgroup's LDS (or the run is float32)
@@ -675,9 +683,7 @@ __global__ __launch_bounds__(1024) void gated_group_norm_kernel(const float* __r
       ss_load4(w + at + i, wv);
 #pragma unroll
       for (int j = 0; j < 4; ++j) wv[j] *= row[i + j] * inv;
-      T* o = out + n * out_stride + at + i;
-#pragma unroll
-      for (int j = 0; j < 4; ++j) o[j] = from_f32<T>(wv[j]);
+      ss_store4(out + n * out_stride + at + i, wv);
     }
   } else {
     for (int i = threadIdx.x; i < part; i += threads) out[n * out_stride + at + i] = from_f32<T>(w[at + i] * (row[i] * inv));

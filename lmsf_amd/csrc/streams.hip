@@ -210,6 +210,16 @@ __global__ __launch_bounds__(256) void stream_embedding_kernel(const int* __rest
   const int id = ids[n];
   const bool ok = id >= 0 && id < V;
   if (!ok && threadIdx.x == 0 && blockIdx.y == 0 && bad_flag) atomicOr(bad_flag, 1);
+  if (W % 4 == 0) {             // (X and the table begin at multiples of 16 bytes: every row at one of four entries)
+    for (int i = (blockIdx.y * 256 + threadIdx.x) * 4; i < W; i += gridDim.y * 1024) {
+      float v[4] = {0.f, 0.f, 0.f, 0.f};
+      if (ok) St4<T>::load(table + (long)id * W + i, v);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) v[j] *= scale;
+      for (int s = 0; s < ns; ++s) St4<float>::store(X + (n * ns + s) * W + i, v);
+    }
+    return;
+  }
   for (int i = blockIdx.y * 256 + threadIdx.x; i < W; i += gridDim.y * 256) {
     const float v = ok ? scale * to_f32<T>(table[(long)id * W + i]) : 0.f;
     for (int s = 0; s < ns; ++s) X[(n * ns + s) * W + i] = v;
@@ -221,8 +231,9 @@ extern "C" int lmsf_stream_embedding(const int* ids, const void* table, int dtyp
   LMSF_CHECK(ids && table && X, "stream_embedding: null pointer");
   LMSF_CHECK(dtype == LMSF_F32 || dtype == LMSF_BF16, "stream_embedding: unknown dtype code %d", dtype);
   LMSF_CHECK(ns > 0 && V > 0 && W > 0, "stream_embedding: bad sizes");
+  LMSF_CHECK(lmsf_aligned16(X) && lmsf_aligned16(table), "stream_embedding: operands must be 16-byte aligned");
   if (n_tokens <= 0) return 0;
-  const dim3 grid(n_tokens, min((W + 255) / 256, 64));
+  const dim3 grid(n_tokens, min((W + 1023) / 1024, 64));
   if (dtype == LMSF_F32)
     hipLaunchKernelGGL((stream_embedding_kernel<float>), grid, dim3(256), 0, stream, ids, (const float*)table, scale, X,
                        ns, V, W, bad_flag);
