@@ -165,66 +165,108 @@ __device__ __forceinline__ void ss_parts8(const float* x, SsFrag (&f)[3]) {
 __device__ __forceinline__ int ss_turned(int c, int piece) { return c * 128 + (((piece ^ c ^ (c >> 3)) & 7) << 4); }
 
 // Columns [0, cols) of 64 rows (``src`` at the chunk's first token, ``nt`` tokens, the others zeros) turned into ``dst``
-// [cols_padded][64]; ``vec``: whole groups of eight columns at aligned places.
+// [cols_padded][64]; ``vec``: whole groups of eight columns at aligned places. A thread takes two tokens of eight columns
+// a time, and asks for two such pieces before it stores one.
+__device__ __forceinline__ void ss_put_turned(const SsFrag& a, const SsFrag& b, int c0, int t, int cols_padded,
+                                              unsigned char* dst) {
+#pragma unroll
+  for (int j = 0; j < 8; ++j) {
+    const int c = c0 + j;
+    if (c >= cols_padded) break;
+    const uint32_t lo = (j & 1) ? a.w[j >> 1] >> 16 : a.w[j >> 1] & 0xffffu;
+    const uint32_t hi = (j & 1) ? b.w[j >> 1] >> 16 : b.w[j >> 1] & 0xffffu;
+    *reinterpret_cast<uint32_t*>(dst + ss_turned(c, t >> 3) + (t & 7) * 2) = lo | (hi << 16);
+  }
+}
 __device__ __forceinline__ void ss_stage_turned(const bf16_t* __restrict__ src, long stride, int nt, int cols,
                                                 int cols_padded, bool vec, unsigned char* dst) {
-  const int blocks = (cols_padded + 7) / 8;
-  // a thread: two tokens of eight columns
-  for (int i = threadIdx.x; i < blocks * (SS_L / 2); i += 256) {
-    const int cb = i % blocks, tp = i / blocks, t = 2 * tp, c0 = cb * 8;
+  const int blocks = (cols_padded + 7) / 8, items = blocks * (SS_L / 2);
+  if (vec) {
+    // (rows and columns outside are read from the last ones and dropped: no branch around a load)
+    for (int i0 = threadIdx.x; i0 < items; i0 += 512) {
+      SsFrag r[2][2];
+#pragma unroll
+      for (int k = 0; k < 2; ++k) {
+        const int i = min(i0 + k * 256, items - 1), c0 = min((i % blocks) * 8, cols - 8), t = 2 * (i / blocks);
+        r[k][0].q = *reinterpret_cast<const uint4*>(src + (long)min(t, nt - 1) * stride + c0);
+        r[k][1].q = *reinterpret_cast<const uint4*>(src + (long)min(t + 1, nt - 1) * stride + c0);
+      }
+#pragma unroll
+      for (int k = 0; k < 2; ++k) {
+        const int i = i0 + k * 256, c0 = (i % blocks) * 8, t = 2 * (i / blocks);
+        if (i >= items) break;
+        if (c0 >= cols || t >= nt) r[k][0].q = make_uint4(0, 0, 0, 0);
+        if (c0 >= cols || t + 1 >= nt) r[k][1].q = make_uint4(0, 0, 0, 0);
+        ss_put_turned(r[k][0], r[k][1], c0, t, cols_padded, dst);
+      }
+    }
+    return;
+  }
+  for (int i = threadIdx.x; i < items; i += 256) {
+    const int c0 = (i % blocks) * 8, t = 2 * (i / blocks);
     SsFrag a, b;
-    a.q = b.q = make_uint4(0, 0, 0, 0);
-    if (vec) {
-      if (c0 < cols) {
-        if (t < nt) a.q = *reinterpret_cast<const uint4*>(src + (long)t * stride + c0);
-        if (t + 1 < nt) b.q = *reinterpret_cast<const uint4*>(src + (long)(t + 1) * stride + c0);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      uint32_t x[4];
+#pragma unroll
+      for (int q = 0; q < 4; ++q) {
+        const int c = c0 + 2 * j + (q & 1), tt = t + (q >> 1);
+        x[q] = c < cols && tt < nt ? src[(long)tt * stride + c] : 0;
       }
-    } else {
-#pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        uint32_t x[4];
-#pragma unroll
-        for (int q = 0; q < 4; ++q) {
-          const int c = c0 + 2 * j + (q & 1), tt = t + (q >> 1);
-          x[q] = c < cols && tt < nt ? src[(long)tt * stride + c] : 0;
-        }
-        a.w[j] = x[0] | (x[1] << 16);
-        b.w[j] = x[2] | (x[3] << 16);
-      }
+      a.w[j] = x[0] | (x[1] << 16);
+      b.w[j] = x[2] | (x[3] << 16);
     }
-#pragma unroll
-    for (int j = 0; j < 8; ++j) {
-      const int c = c0 + j;
-      if (c >= cols_padded) break;
-      const uint32_t lo = (j & 1) ? a.w[j >> 1] >> 16 : a.w[j >> 1] & 0xffffu;
-      const uint32_t hi = (j & 1) ? b.w[j >> 1] >> 16 : b.w[j >> 1] & 0xffffu;
-      *reinterpret_cast<uint32_t*>(dst + ss_turned(c, t >> 3) + (t & 7) * 2) = lo | (hi << 16);
-    }
+    ss_put_turned(a, b, c0, t, cols_padded, dst);
   }
 }
 
-// The same columns as they lie, rows of ``row_bytes``.
-__device__ __forceinline__ void ss_stage(const bf16_t* __restrict__ src, long stride, int nt, int cols, int cols_padded,
-                                         bool vec, unsigned char* dst, int row_bytes) {
-  const int blocks = cols_padded / 8;
-  for (int i = threadIdx.x; i < blocks * SS_L; i += 256) {
-    const int cb = i % blocks, t = i / blocks, c0 = cb * 8;
+// Two matrices of the same columns as they lie (C and B), rows of ``row_bytes``, one behind the other from ``dst`` on
+// (``apart`` bytes).
+__device__ __forceinline__ void ss_stage_two(const bf16_t* __restrict__ src0, const bf16_t* __restrict__ src1, long stride,
+                                             int nt, int cols, int cols_padded, bool vec, unsigned char* dst, int apart,
+                                             int row_bytes) {
+  const int blocks = cols_padded / 8, items = 2 * SS_L * blocks;
+  if (vec) {
+    for (int i0 = threadIdx.x; i0 < items; i0 += 8 * 256) {
+      uint4 r[8];
+#pragma unroll
+      for (int k = 0; k < 8; ++k) {
+        const int i = min(i0 + k * 256, items - 1), row = i / blocks, c0 = min((i - row * blocks) * 8, cols - 8);
+        const bf16_t* src = row < SS_L ? src0 : src1;
+        r[k] = *reinterpret_cast<const uint4*>(src + (long)min(row & (SS_L - 1), nt - 1) * stride + c0);
+      }
+#pragma unroll
+      for (int k = 0; k < 8; ++k) {
+        const int i = i0 + k * 256, row = i / blocks, c0 = (i - row * blocks) * 8, t = row & (SS_L - 1);
+        if (i >= items) break;
+        if (c0 >= cols || t >= nt) r[k] = make_uint4(0, 0, 0, 0);
+        *reinterpret_cast<uint4*>(dst + (row < SS_L ? 0 : apart) + t * row_bytes + c0 * 2) = r[k];
+      }
+    }
+    return;
+  }
+  for (int i = threadIdx.x; i < items; i += 256) {
+    const int row = i / blocks, c0 = (i - row * blocks) * 8, t = row & (SS_L - 1);
+    const bf16_t* src = row < SS_L ? src0 : src1;
     SsFrag a;
     a.q = make_uint4(0, 0, 0, 0);
     if (t < nt) {
-      if (vec) {
-        if (c0 < cols) a.q = *reinterpret_cast<const uint4*>(src + (long)t * stride + c0);
-      } else {
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          const int c = c0 + 2 * j;
-          const uint32_t lo = c < cols ? src[(long)t * stride + c] : 0, hi = c + 1 < cols ? src[(long)t * stride + c + 1] : 0;
-          a.w[j] = lo | (hi << 16);
-        }
+      for (int j = 0; j < 4; ++j) {
+        const int c = c0 + 2 * j;
+        const uint32_t lo = c < cols ? src[(long)t * stride + c] : 0, hi = c + 1 < cols ? src[(long)t * stride + c + 1] : 0;
+        a.w[j] = lo | (hi << 16);
       }
     }
-    *reinterpret_cast<uint4*>(dst + t * row_bytes + c0 * 2) = a.q;
+    *reinterpret_cast<uint4*>(dst + (row < SS_L ? 0 : apart) + t * row_bytes + c0 * 2) = a.q;
   }
+}
+
+// The head of a workgroup: workgroups go to the eight dies in turn, and neighbouring heads (which share a group's B and C)
+// are given to one die.
+__device__ __forceinline__ int ss_head(int H) {
+  const int b = blockIdx.x;
+  return H % 8 == 0 ? (b % 8) * (H / 8) + b / 8 : b;
 }
 
 // The first wave works out a chunk's steps and sums of logarithms: dt [64] (0 behind the chunk's end), the sums as two
@@ -260,12 +302,12 @@ __global__ __launch_bounds__(256) void state_space_sums_kernel(
   float* shi = sdt + SS_L;
   float* slo = shi + SS_L;
   float* sw = slo + SS_L;                         // [64]: exp(c_L - c_u) dt_u
-  const int h = blockIdx.x, g = h / (H / G);
+  const int h = ss_head(H), g = h / (H / G);
   const long i = blockIdx.y;
   const int t0 = chunks[3 * i], nt = chunks[3 * i + 1];
-  ss_steps(dt_pre + (long)t0 * dt_stride, dt_stride, h, nt, dt_bias[h], rate[h], sdt, shi, slo);
   ss_stage_turned(xbc + (long)t0 * xbc_stride + b_at + g * N, xbc_stride, nt, N, Np, vec_b, BT);
   ss_stage_turned(xbc + (long)t0 * xbc_stride + x_at + h * dv, xbc_stride, nt, dv, dvp, vec_x, XT);
+  ss_steps(dt_pre + (long)t0 * dt_stride, dt_stride, h, nt, dt_bias[h], rate[h], sdt, shi, slo);
   __syncthreads();
   if (threadIdx.x < SS_L) {
     const int u = threadIdx.x;
@@ -353,7 +395,7 @@ __global__ __launch_bounds__(256) void state_space_fold_kernel(float* __restrict
 // rows u, columns t) and leaves its three bfloat16 parts in LDS as the second product takes them; then a wave takes 16
 // value entries at a time against all 64 tokens.
 // PT: [4 blocks of 16 t][2 pairs of u blocks][3 parts][64 lanes] of 16 bytes.
-__global__ __launch_bounds__(256) void state_space_outputs_kernel(
+__global__ __launch_bounds__(256, 3) void state_space_outputs_kernel(
     const bf16_t* __restrict__ xbc, long xbc_stride, int x_at, int b_at, int c_at, const float* __restrict__ dt_pre,
     long dt_stride, const float* __restrict__ dt_bias, const float* __restrict__ rate, const float* __restrict__ D,
     const int* __restrict__ chunks, const float* __restrict__ S0, float* __restrict__ y, long y_stride, int H, int G, int N,
@@ -367,7 +409,7 @@ __global__ __launch_bounds__(256) void state_space_outputs_kernel(
   float* sdt = reinterpret_cast<float*>(XT + dvp * 128);
   float* shi = sdt + SS_L;
   float* slo = shi + SS_L;
-  const int h = blockIdx.x, g = h / (H / G);
+  const int h = ss_head(H), g = h / (H / G);
   const long i = blockIdx.y;
   const int t0 = chunks[3 * i], nt = chunks[3 * i + 1];
   const int wave = threadIdx.x / LMSF_WAVE, lane = threadIdx.x % LMSF_WAVE, fr = lane % 16, fg = lane / 16;
@@ -393,10 +435,9 @@ __global__ __launch_bounds__(256) void state_space_outputs_kernel(
   for (int k = 0; k < 4; ++k)
     if (k < nk) load_state(wave, k, ahead[k]);
   const bf16_t* base = xbc + (long)t0 * xbc_stride;
-  ss_steps(dt_pre + (long)t0 * dt_stride, dt_stride, h, nt, dt_bias[h], rate[h], sdt, shi, slo);
-  ss_stage(base + c_at + g * N, xbc_stride, nt, N, Nk, vec_b, Cs, row_bytes);
-  ss_stage(base + b_at + g * N, xbc_stride, nt, N, Nk, vec_b, Bs, row_bytes);
+  ss_stage_two(base + c_at + g * N, base + b_at + g * N, xbc_stride, nt, N, Nk, vec_b, Cs, SS_L * row_bytes, row_bytes);
   ss_stage_turned(base + x_at + h * dv, xbc_stride, nt, dv, dvp, vec_x, XT);
+  ss_steps(dt_pre + (long)t0 * dt_stride, dt_stride, h, nt, dt_bias[h], rate[h], sdt, shi, slo);
   __syncthreads();
   {
     const int t = wave * 16 + fr;                        // this lane's token
@@ -450,6 +491,7 @@ __global__ __launch_bounds__(256) void state_space_outputs_kernel(
 #pragma unroll
         for (int q = 0; q < 3; ++q) acc[tb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(f[q].v, cf.v, acc[tb], 0, 0, 0);
       }
+      __builtin_amdgcn_sched_barrier(0);      // (else the scheduler asks for all blocks' operands at once and runs out of registers)
     };
     if (et != wave) {
 #pragma unroll
@@ -501,6 +543,7 @@ __global__ __launch_bounds__(256) void state_space_outputs_kernel(
             if (et * 16 + fg * 4 + r < dv) out[r] = o[r];
         }
       }
+      __builtin_amdgcn_sched_barrier(0);
     }
   }
 }
