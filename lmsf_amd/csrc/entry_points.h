@@ -81,6 +81,18 @@ int lmsf_state_space_chunked(const void* xbc, int dtype, long xbc_stride, int x_
 int lmsf_gated_group_norm(const float* y, long y_stride, const void* z, long z_stride, int dtype, const float* w, void*
     out, long out_stride, int n_rows, int inner, int parts, float eps, hipStream_t stream);
 
+// forms of the gated products and of the gated activation with a bound on both operands (act 6, kind 3)
+int lmsf_gated_act_limit(const void* in, void* out, int dtype, int n_tokens, int I, long in_stride, int kind, float limit,
+    hipStream_t stream);
+int lmsf_gemv_limit(const void* x, long ldx, const void* W, long ldw, const void* bias, void* y, int out_dtype, long ldy,
+    int M, int N, int K, int act, float limit, hipStream_t stream);
+int lmsf_gemm_skinny_limit(const void* x, long ldx, const void* W, long ldw, const void* bias, void* y, int out_dtype, long
+    ldy, int M, int N, int K, int variant, int act, float limit, hipStream_t stream);
+int lmsf_gemm_mid_limit(const void* x, long ldx, const void* W, long ldw, const void* bias, void* y, int out_dtype, long
+    ldy, int M, int N, int K, int act, float limit, int n_split, float* scratch, hipStream_t stream);
+int lmsf_gemm_large_limit(const void* x, long ldx, const void* W, long ldw, const void* bias, void* y, long ldy, int M, int
+    N, int K, int act, float limit, int plan, float* scratch, int reduce, hipStream_t stream);
+
 // latent.hip
 int lmsf_latent_cache_write(const void* x, int dtype, long x_stride, const float* w, float eps, const int* positions,
     const float* table, int rot, int max_pos, const int* slots, void* k_pages, void* v_pages, long num_pages,

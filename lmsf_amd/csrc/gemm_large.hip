@@ -62,10 +62,11 @@ __device__ __forceinline__ unsigned large_lds_address(const void* p) {
   return (unsigned)(size_t)(__attribute__((address_space(3))) const unsigned char*)p;
 }
 
-__device__ __forceinline__ float large_activation(float g, float u, int act) {
+__device__ __forceinline__ float large_activation(float g, float u, int act, float limit) {
   // the two products are rounded to the storage type before the activation, as the unfused path stores them
   g = bf16_to_f32(f32_to_bf16(g));
   u = bf16_to_f32(f32_to_bf16(u));
+  if (act == 6) return bounded_gate(g, u, limit);
   const float a = act == 1 ? g / (1.0f + expf(-g)) : 0.5f * g * (1.0f + erff(g * 0.70710678118654752f));
   return a * u;
 }
@@ -73,14 +74,15 @@ __device__ __forceinline__ float large_activation(float g, float u, int act) {
 #define LARGE_ROW 128         // bytes of a tile row: 64 k, two steps of the matrix instruction
 
 // BM: rows of x per workgroup (128 or 256). BN: rows of W per workgroup (128 or 256; with ACT half of them gate rows
-// and half the up rows of the same outputs). ACT: 0 none, 1 SiLU-gated, 2 GELU-gated. PARTIAL: float32 partial sums
+// and half the up rows of the same outputs). ACT: 0 none, 1 SiLU-gated, 2 GELU-gated, 6 gated with
+// both operands bounded by ``limit``. PARTIAL: float32 partial sums
 // of this workgroup's part of K instead of the result (not with ACT).
 template <int BM, int BN, int STAGES, int ACT, bool PARTIAL, int KG>
 __global__ __launch_bounds__(256 * KG) void gemm_large_kernel(const bf16_t* __restrict__ x, long ldx,
                                                          const bf16_t* __restrict__ W, long ldw,
                                                          const bf16_t* __restrict__ bias, bf16_t* __restrict__ y,
                                                          long ldy, float* __restrict__ part, int M, int N, int K,
-                                                         int n_split, int tiles_m, int tiles_n) {
+                                                         int n_split, int tiles_m, int tiles_n, float limit) {
   static_assert(!(ACT != 0 && PARTIAL), "the gated product is made in one piece");
   constexpr int MT = BM / 32;                      // accumulator tiles along x per wave
   constexpr int NT = BN / 32;                      // along W
@@ -248,7 +250,7 @@ __global__ __launch_bounds__(256 * KG) void gemm_large_kernel(const bf16_t* __re
         for (int i = 0; i < 4; ++i) {
           const float gg = acc[t][mt][i] + (bias ? bf16_to_f32(bias[n + i]) : 0.f);
           const float uu = acc[t + NT / 2][mt][i] + (bias ? bf16_to_f32(bias[N + n + i]) : 0.f);
-          o[i] = large_activation(gg, uu, ACT);
+          o[i] = large_activation(gg, uu, ACT, limit);
         }
         v.x = pack2_bf16(o[0], o[1]);
         v.y = pack2_bf16(o[2], o[3]);
@@ -277,7 +279,7 @@ __global__ __launch_bounds__(256 * KG) void gemm_large_kernel(const bf16_t* __re
 
 template <int BM, int BN, int STAGES, int ACT, bool PARTIAL, int KG = 1>
 static int launch_large(hipStream_t stream, const bf16_t* x, long ldx, const bf16_t* W, long ldw, const bf16_t* bias,
-                        bf16_t* y, long ldy, float* part, int M, int N, int K, int n_split) {
+                        bf16_t* y, long ldy, float* part, int M, int N, int K, int n_split, float limit) {
   const size_t smem = (size_t)STAGES * (BN + BM) * LARGE_ROW;
   auto kernel = gemm_large_kernel<BM, BN, STAGES, ACT, PARTIAL, KG>;
   static bool configured = false;   // per instantiation
@@ -294,7 +296,7 @@ static int launch_large(hipStream_t stream, const bf16_t* x, long ldx, const bf1
   const int tiles_m = (M + BM - 1) / BM, tiles_n = (N + n_out - 1) / n_out;
   const int groups = (tiles_n + 7) / 8;
   hipLaunchKernelGGL(kernel, dim3(groups * tiles_m * 8, n_split), dim3(256 * KG), smem, stream, x, ldx, W, ldw, bias, y, ldy,
-                     part, M, N, K, n_split, tiles_m, tiles_n);
+                     part, M, N, K, n_split, tiles_m, tiles_n, limit);
   return 0;
 }
 
@@ -305,15 +307,16 @@ static const int kLargeTiles[6][2] = {{128, 128}, {256, 128}, {192, 128}, {128, 
 
 template <int ACT, bool PARTIAL>
 static int launch_tiling(int tiling, hipStream_t stream, const bf16_t* x, long ldx, const bf16_t* W, long ldw,
-                         const bf16_t* bias, bf16_t* y, long ldy, float* part, int M, int N, int K, int n_split) {
+                         const bf16_t* bias, bf16_t* y, long ldy, float* part, int M, int N, int K, int n_split,
+                         float limit = 0.f) {
   switch (tiling) {
-    case 0: return launch_large<128, 128, 4, ACT, PARTIAL>(stream, x, ldx, W, ldw, bias, y, ldy, part, M, N, K, n_split);
-    case 1: return launch_large<256, 128, 3, ACT, PARTIAL>(stream, x, ldx, W, ldw, bias, y, ldy, part, M, N, K, n_split);
-    case 2: return launch_large<192, 128, 4, ACT, PARTIAL>(stream, x, ldx, W, ldw, bias, y, ldy, part, M, N, K, n_split);
+    case 0: return launch_large<128, 128, 4, ACT, PARTIAL>(stream, x, ldx, W, ldw, bias, y, ldy, part, M, N, K, n_split, limit);
+    case 1: return launch_large<256, 128, 3, ACT, PARTIAL>(stream, x, ldx, W, ldw, bias, y, ldy, part, M, N, K, n_split, limit);
+    case 2: return launch_large<192, 128, 4, ACT, PARTIAL>(stream, x, ldx, W, ldw, bias, y, ldy, part, M, N, K, n_split, limit);
     // the same tiles with two groups of four waves
-    case 3: return launch_large<128, 128, 4, ACT, PARTIAL, 2>(stream, x, ldx, W, ldw, bias, y, ldy, part, M, N, K, n_split);
-    case 4: return launch_large<256, 128, 3, ACT, PARTIAL, 2>(stream, x, ldx, W, ldw, bias, y, ldy, part, M, N, K, n_split);
-    default: return launch_large<192, 128, 4, ACT, PARTIAL, 2>(stream, x, ldx, W, ldw, bias, y, ldy, part, M, N, K, n_split);
+    case 3: return launch_large<128, 128, 4, ACT, PARTIAL, 2>(stream, x, ldx, W, ldw, bias, y, ldy, part, M, N, K, n_split, limit);
+    case 4: return launch_large<256, 128, 3, ACT, PARTIAL, 2>(stream, x, ldx, W, ldw, bias, y, ldy, part, M, N, K, n_split, limit);
+    default: return launch_large<192, 128, 4, ACT, PARTIAL, 2>(stream, x, ldx, W, ldw, bias, y, ldy, part, M, N, K, n_split, limit);
   }
 }
 
@@ -357,15 +360,13 @@ extern "C" long lmsf_gemm_large_scratch_floats(int M, int N, int n_split) {
 // lmsf_gemm_large_scratch_floats floats; with ``reduce`` 0 the sums stay there ([n_split, M, N], for a kernel that
 // adds them up itself, bias not yet added) and y is not written. ``plan``: tiling * 16 + n_split, as
 // lmsf_gemm_large_plan proposes. K a multiple of 64, N of 8, row strides of 8, 16-byte aligned bases.
-extern "C" int lmsf_gemm_large(const void* x, long ldx, const void* W, long ldw, const void* bias, void* y, long ldy,
-                               int M, int N, int K, int act, int plan, float* scratch, int reduce,
-                               hipStream_t stream);
+// act 6: the gated form with both operands bounded by ``limit`` (common.h: bounded_gate).
 extern "C" int lmsf_gemm_mid_reduce(const float* scratch, const void* bias, void* y, int out_dtype, long ldy, int M,
                                     int N, int n_split, hipStream_t stream);
 
-extern "C" int lmsf_gemm_large(const void* x, long ldx, const void* W, long ldw, const void* bias, void* y, long ldy,
-                               int M, int N, int K, int act, int plan, float* scratch, int reduce,
-                               hipStream_t stream) {
+extern "C" int lmsf_gemm_large_limit(const void* x, long ldx, const void* W, long ldw, const void* bias, void* y, long ldy,
+                                     int M, int N, int K, int act, float limit, int plan, float* scratch, int reduce,
+                                     hipStream_t stream) {
   const int tiling = plan / 16, n_split = plan % 16;
   LMSF_CHECK(tiling >= 0 && tiling < 6, "gemm_large: unknown tiling %d", tiling);
   LMSF_CHECK(x && W && (y || (n_split > 1 && !reduce)), "gemm_large: null pointer");
@@ -374,7 +375,7 @@ extern "C" int lmsf_gemm_large(const void* x, long ldx, const void* W, long ldw,
   LMSF_CHECK(ldx >= K && ldw >= K && ldx % 8 == 0 && ldw % 8 == 0 && (!y || (ldy >= N && ldy % 4 == 0)),
              "gemm_large: bad row strides");
   LMSF_CHECK(lmsf_aligned16(x) && lmsf_aligned16(W) && (!y || (((uintptr_t)y) & 7u) == 0), "gemm_large: operands must be 16-byte aligned");
-  LMSF_CHECK(act >= 0 && act <= 2, "gemm_large: unknown activation %d", act);
+  LMSF_CHECK((act >= 0 && act <= 2) || act == 6, "gemm_large: unknown activation %d", act);
   LMSF_CHECK(n_split >= 1 && n_split <= K / 64 && (n_split == 1 || act == 0), "gemm_large: bad split %d", n_split);
   LMSF_CHECK(n_split == 1 || (scratch && lmsf_aligned16(scratch)), "gemm_large: a split product needs scratch");
   const bf16_t* xp = (const bf16_t*)x;
@@ -388,10 +389,19 @@ extern "C" int lmsf_gemm_large(const void* x, long ldx, const void* W, long ldw,
     rc = launch_tiling<0, false>(tiling, stream, xp, ldx, wp, ldw, bp, yp, ldy, nullptr, M, N, K, 1);
   else if (act == 1)
     rc = launch_tiling<1, false>(tiling, stream, xp, ldx, wp, ldw, bp, yp, ldy, nullptr, M, N, K, 1);
-  else
+  else if (act == 2)
     rc = launch_tiling<2, false>(tiling, stream, xp, ldx, wp, ldw, bp, yp, ldy, nullptr, M, N, K, 1);
+  else
+    rc = launch_tiling<6, false>(tiling, stream, xp, ldx, wp, ldw, bp, yp, ldy, nullptr, M, N, K, 1, limit);
   if (rc != 0) return rc;
   LMSF_LAUNCH_CHECK("gemm_large");
   if (n_split > 1 && reduce) return lmsf_gemm_mid_reduce(scratch, bias, y, LMSF_BF16, ldy, M, N, n_split, stream);
   return 0;
+}
+
+extern "C" int lmsf_gemm_large(const void* x, long ldx, const void* W, long ldw, const void* bias, void* y, long ldy,
+                               int M, int N, int K, int act, int plan, float* scratch, int reduce,
+                               hipStream_t stream) {
+  LMSF_CHECK(act != 6, "gemm_large: the bounded form needs its limit");
+  return lmsf_gemm_large_limit(x, ldx, W, ldw, bias, y, ldy, M, N, K, act, 0.f, plan, scratch, reduce, stream);
 }

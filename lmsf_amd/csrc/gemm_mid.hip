@@ -40,10 +40,11 @@ __device__ __forceinline__ unsigned mid_lds_address(const void* p) {
   return (unsigned)(size_t)(__attribute__((address_space(3))) const unsigned char*)p;
 }
 
-__device__ __forceinline__ float mid_activation(float g, float u, int act) {
+__device__ __forceinline__ float mid_activation(float g, float u, int act, float limit) {
   // the two products are rounded to the storage type before the activation, as the unfused path stores them
   g = bf16_to_f32(f32_to_bf16(g));
   u = bf16_to_f32(f32_to_bf16(u));
+  if (act == 6) return bounded_gate(g, u, limit);
   const float a = act == 1 ? g / (1.0f + expf(-g)) : 0.5f * g * (1.0f + erff(g * 0.70710678118654752f));
   return a * u;
 }
@@ -62,8 +63,8 @@ __device__ __forceinline__ void mid_store4(float* p, const float* o) {
 #define MID_STAGES_OF(TW) ((TW) == 2 ? 4 : 5)   // stages of the ring: what fits into the 160 KB of LDS
 #define MID_TILE 2048
 
-// MT: tiles of 16 rows of x (2, 4, 6 or 8). ACT: 0 none, 1 silu-gated, 2 gelu-gated (W = [gate rows; up rows], N
-// outputs). PARTIAL: write float32 partial sums of this workgroup's part of K instead of the result. TW: tiles of 16
+// MT: tiles of 16 rows of x (2, 4, 6 or 8). ACT: 0 none, 1 silu-gated, 2 gelu-gated, 6 gated with both operands
+// bounded (W = [gate rows; up rows], N outputs). PARTIAL: write float32 partial sums of this workgroup's part of K instead of the result. TW: tiles of 16
 // outputs a wave owns (of each projection), so 64 TW outputs a workgroup.
 // (A form of the gated product with 32 outputs a workgroup, waves 0 and 1 on the gate rows and 2 and 3 on the up rows
 // of the same outputs, twice as many workgroups, two to a compute unit, was ahead at 17 to 48 rows while the
@@ -79,6 +80,7 @@ struct MidRowScale {
   int tiles;
   float eps;
   int H;
+  float limit;      // ACT 6 (no norm is meant): the bound of the gated activation's operands
 };
 #define MID_SCALE_HELD 32   // sums a thread holds: thread t has row t % 16 of the tiles t / 16, t / 16 + 16, ...
 
@@ -226,7 +228,7 @@ __global__ __launch_bounds__(256) void gemm_mid_kernel(const bf16_t* __restrict_
           } else {
             const float gg = acc[tw][mt][i] * inv + (bias ? bf16_to_f32(bias[n + i]) : 0.f);
             const float uu = acc[(WP - 1) * TW + tw][mt][i] * inv + (bias ? bf16_to_f32(bias[N + n + i]) : 0.f);
-            o[i] = mid_activation(gg, uu, ACT);
+            o[i] = mid_activation(gg, uu, ACT, rs.limit);
           }
         }
         mid_store4(y + (long)m * ldy + n, o);
@@ -239,7 +241,7 @@ __global__ __launch_bounds__(256) void gemm_mid_kernel(const bf16_t* __restrict_
 template <typename TOut>
 __global__ __launch_bounds__(256) void gemm_mid_reduce_kernel(const float* __restrict__ part,
                                                               const bf16_t* __restrict__ bias, TOut* __restrict__ y,
-                                                              long ldy, int M, int N, int n_split, int act) {
+                                                              long ldy, int M, int N, int n_split, int act, float limit) {
   const long idx = ((long)blockIdx.x * 256 + threadIdx.x) * 4;   // over M * N, four outputs of a row at a time
   if (idx >= (long)M * N) return;
   const int m = (int)(idx / N), n = (int)(idx - (long)m * N);
@@ -255,7 +257,7 @@ __global__ __launch_bounds__(256) void gemm_mid_reduce_kernel(const float* __res
     const float gg = sg[i] + (bias ? bf16_to_f32(bias[n + i]) : 0.f);
     if (act) {
       const float uu = su[i] + (bias ? bf16_to_f32(bias[N + n + i]) : 0.f);
-      o[i] = mid_activation(gg, uu, act);
+      o[i] = mid_activation(gg, uu, act, limit);
     } else {
       o[i] = gg;
     }
@@ -337,7 +339,7 @@ static int mid_check(const void* x, long ldx, const void* W, long ldw, int M, in
 // The product's kernel: the result into y (n_split == 1) or partial sums into scratch.
 static int mid_product(const bf16_t* xb, long ldx, const bf16_t* Wb, long ldw, const bf16_t* bb, void* y, int out_dtype,
                        long ldy, int M, int N, int K, int act, int n_split, float* scratch, hipStream_t stream,
-                       MidRowScale rs = MidRowScale{nullptr, 0, 0.f, 0}) {
+                       MidRowScale rs = MidRowScale{nullptr, 0, 0.f, 0, 0.f}) {
   dim3 grid((N + 63) / 64, n_split);
   int rc = 0;
 #define MID(MT_, ACT_, T_)                                                                                          \
@@ -347,9 +349,9 @@ static int mid_product(const bf16_t* xb, long ldx, const bf16_t* Wb, long ldw, c
   if (out_dtype == LMSF_F32) {
     if (M <= 32) MID(2, 0, float); else if (M <= 64) MID(4, 0, float); else if (M <= 96) MID(6, 0, float); else MID(8, 0, float);
   } else if (M <= 32) {
-    if (act == 0) MID(2, 0, bf16_t); else if (act == 1) MID(2, 1, bf16_t); else MID(2, 2, bf16_t);
+    if (act == 0) MID(2, 0, bf16_t); else if (act == 1) MID(2, 1, bf16_t); else if (act == 2) MID(2, 2, bf16_t); else MID(2, 6, bf16_t);
   } else if (M <= 64) {
-    if (act == 0) MID(4, 0, bf16_t); else if (act == 1) MID(4, 1, bf16_t); else MID(4, 2, bf16_t);
+    if (act == 0) MID(4, 0, bf16_t); else if (act == 1) MID(4, 1, bf16_t); else if (act == 2) MID(4, 2, bf16_t); else MID(4, 6, bf16_t);
   } else if (M <= 96) {
     MID(6, 0, bf16_t);
   } else {
@@ -362,23 +364,24 @@ static int mid_product(const bf16_t* xb, long ldx, const bf16_t* Wb, long ldw, c
 }
 
 static int mid_reduce(const float* scratch, const bf16_t* bb, void* y, int out_dtype, long ldy, int M, int N,
-                      int act, int n_split, hipStream_t stream) {
+                      int act, int n_split, hipStream_t stream, float limit = 0.f) {
   const long quads = ((long)M * N + 3) / 4;
   const dim3 rgrid((unsigned)((quads + 255) / 256));
   if (out_dtype == LMSF_F32)
     hipLaunchKernelGGL(gemm_mid_reduce_kernel<float>, rgrid, dim3(256), 0, stream, scratch, bb, (float*)y, ldy, M, N,
-                       n_split, act);
+                       n_split, act, limit);
   else
     hipLaunchKernelGGL(gemm_mid_reduce_kernel<bf16_t>, rgrid, dim3(256), 0, stream, scratch, bb, (bf16_t*)y, ldy, M,
-                       N, n_split, act);
+                       N, n_split, act, limit);
   LMSF_LAUNCH_CHECK("gemm_mid_reduce");
   return 0;
 }
 
-extern "C" int lmsf_gemm_mid(const void* x, long ldx, const void* W, long ldw, const void* bias, void* y,
-                             int out_dtype, long ldy, int M, int N, int K, int act, int n_split, float* scratch,
-                             hipStream_t stream) {
-  LMSF_CHECK(act >= 0 && act <= 2, "gemm_mid: unknown activation %d", act);
+// act 6: the gated form with both operands bounded by ``limit`` (common.h: bounded_gate).
+extern "C" int lmsf_gemm_mid_limit(const void* x, long ldx, const void* W, long ldw, const void* bias, void* y,
+                                   int out_dtype, long ldy, int M, int N, int K, int act, float limit, int n_split,
+                                   float* scratch, hipStream_t stream) {
+  LMSF_CHECK((act >= 0 && act <= 2) || act == 6, "gemm_mid: unknown activation %d", act);
   if (int rc = mid_check(x, ldx, W, ldw, M, N, K, M == 0 ? 1 : n_split, scratch, act)) return rc;
   LMSF_CHECK(y != nullptr && lmsf_aligned16(y) && ldy >= N && ldy % 4 == 0,
              "gemm_mid: y must be 16-byte aligned with a row stride that covers N and is a multiple of 4");
@@ -386,9 +389,17 @@ extern "C" int lmsf_gemm_mid(const void* x, long ldx, const void* W, long ldw, c
              "gemm_mid: output is bfloat16, or float32 without activation");
   if (M == 0) return 0;
   const bf16_t *xb = (const bf16_t*)x, *Wb = (const bf16_t*)W, *bb = (const bf16_t*)bias;
-  if (int rc = mid_product(xb, ldx, Wb, ldw, bb, y, out_dtype, ldy, M, N, K, act, n_split, scratch, stream)) return rc;
-  if (n_split > 1) return mid_reduce(scratch, bb, y, out_dtype, ldy, M, N, act, n_split, stream);
+  const MidRowScale rs = {nullptr, 0, 0.f, 0, limit};
+  if (int rc = mid_product(xb, ldx, Wb, ldw, bb, y, out_dtype, ldy, M, N, K, act, n_split, scratch, stream, rs)) return rc;
+  if (n_split > 1) return mid_reduce(scratch, bb, y, out_dtype, ldy, M, N, act, n_split, stream, limit);
   return 0;
+}
+
+extern "C" int lmsf_gemm_mid(const void* x, long ldx, const void* W, long ldw, const void* bias, void* y,
+                             int out_dtype, long ldy, int M, int N, int K, int act, int n_split, float* scratch,
+                             hipStream_t stream) {
+  LMSF_CHECK(act != 6, "gemm_mid: the bounded form needs its limit");
+  return lmsf_gemm_mid_limit(x, ldx, W, ldw, bias, y, out_dtype, ldy, M, N, K, act, 0.f, n_split, scratch, stream);
 }
 
 // The two halves of a product without activation whose K is split (n_split >= 2): the partial sums alone,
@@ -428,7 +439,7 @@ extern "C" int lmsf_gemm_mid_scaled(const void* x, long ldx, const void* W, long
   LMSF_CHECK(sumsq != nullptr && in_tiles > 0 && in_tiles == (K + 15) / 16 && in_tiles <= 16 * MID_SCALE_HELD,
              "gemm_mid_scaled: %d sums of squares must cover %d columns (at most %d)", in_tiles, K, 16 * 16 * MID_SCALE_HELD);
   if (M == 0) return 0;
-  const MidRowScale rs = {sumsq, in_tiles, eps, K};
+  const MidRowScale rs = {sumsq, in_tiles, eps, K, 0.f};
   if (mid_scaled_outputs(N) == 128) {
     const dim3 grid((N + 127) / 128, 1);
     const int rc = act == 1 ? launch_mid<2, 1, false, bf16_t, 2>(grid, stream, (const bf16_t*)x, ldx, (const bf16_t*)W, ldw,

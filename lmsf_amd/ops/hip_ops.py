@@ -1818,16 +1818,17 @@ class HipOps:
             return self.linear_gated(self.materialize(x), weight, bias, kind, limit)
         if (kind == "bounded") != (limit > 0):
             raise ValueError("a limit > 0 goes with the activation 'bounded'")
-        if rt.route == D.SEPARATE or (kind in ("gelu_tanh", "bounded") and rt.route not in (D.GEMV, D.SKINNY)):
-            # (these two are epilogues of the one-row and the few-rows product only)
+        if rt.route == D.SEPARATE or (kind == "gelu_tanh" and rt.route not in (D.GEMV, D.SKINNY)) \
+                or (kind == "bounded" and scaled):
+            # (the tanh form of GELU is an epilogue of the one-row and the few-rows product only)
             return self.gated_act(self.linear(self.materialize(x), weight, bias), kind, limit)
         self._dev(xt, weight, bias)
         if bias is not None and (bias.shape != (2 * I,) or bias.dtype != weight.dtype or not bias.is_contiguous()):
             raise ValueError("linear_gated: bias must be [%d] of the weight's dtype" % (2 * I))
         if rt.route == D.MID:
-            return self._linear_mid(x, weight, bias, kinds[kind], torch.bfloat16, rt)
+            return self._linear_mid(x, weight, bias, kinds[kind], torch.bfloat16, rt, limit=limit)
         if rt.route == D.LARGE:
-            return self._linear_large(x, weight, bias, kinds[kind], plan=rt.plan)
+            return self._linear_large(x, weight, bias, kinds[kind], plan=rt.plan, limit=limit)
         y = torch.empty((M, I), dtype=torch.bfloat16, device=x.device)
         head = (_ptr(xt), xt.stride(0), _ptr(weight), weight.stride(0), _ptr(bias), _ptr(y))
         if rt.route == D.MID_SCALED:
@@ -1848,7 +1849,7 @@ class HipOps:
         return y
 
     def _linear_mid(self, x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor], act: int,
-                    out_dtype: torch.dtype, rt: D.Route, out: Optional[torch.Tensor] = None):
+                    out_dtype: torch.dtype, rt: D.Route, out: Optional[torch.Tensor] = None, limit: float = 0.0):
         """The 17-and-more-rows product (csrc/gemm_mid.hip) as ``rt`` says."""
         self._dev(x, weight, bias)
         M, K = x.shape
@@ -1865,13 +1866,14 @@ class HipOps:
         floats = self.lib.lmsf_gemm_mid_scratch_floats(M, N, splits, act)
         scratch = torch.empty(floats, dtype=torch.float32, device=x.device) if floats else None
         y = out if out is not None else torch.empty((M, N), dtype=out_dtype, device=x.device)
-        self._check(self.lib.lmsf_gemm_mid(_ptr(x), x.stride(0), _ptr(weight), weight.stride(0), _ptr(bias), _ptr(y),
-                                           _code(out_dtype), y.stride(0), M, N, K, act, splits, _ptr(scratch),
-                                           self._stream()))
+        self._check(self.lib.lmsf_gemm_mid_limit(_ptr(x), x.stride(0), _ptr(weight), weight.stride(0), _ptr(bias), _ptr(y),
+                                                 _code(out_dtype), y.stride(0), M, N, K, act, float(limit), splits,
+                                                 _ptr(scratch), self._stream()))
         return y
 
     def _linear_large(self, x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor], act: int,
-                      pending_ok: bool = False, out: Optional[torch.Tensor] = None, plan: Optional[int] = None):
+                      pending_ok: bool = False, out: Optional[torch.Tensor] = None, plan: Optional[int] = None,
+                      limit: float = 0.0):
         """The many-rows product (csrc/gemm_large.hip); K a multiple of 64, W's rows of 8, row strides of 8,
         16-byte aligned bases. ``plan``: tiling and split (``lmsf_gemm_large_plan`` proposes one)."""
         self._dev(x, weight, bias)
@@ -1891,8 +1893,9 @@ class HipOps:
                                                      M, N, K, 0, plan, _ptr(scratch), 0, self._stream()))
                 return PendingProduct(scratch, bias, torch.bfloat16)
         y = out if out is not None else torch.empty((M, N), dtype=torch.bfloat16, device=x.device)
-        self._check(self.lib.lmsf_gemm_large(_ptr(x), x.stride(0), _ptr(weight), weight.stride(0), _ptr(bias), _ptr(y),
-                                             y.stride(0), M, N, K, act, plan, _ptr(scratch), 1, self._stream()))
+        self._check(self.lib.lmsf_gemm_large_limit(_ptr(x), x.stride(0), _ptr(weight), weight.stride(0), _ptr(bias), _ptr(y),
+                                                   y.stride(0), M, N, K, act, float(limit), plan, _ptr(scratch), 1,
+                                                   self._stream()))
         return y
 
     def tune_products(self, x: torch.Tensor, weights, bias: Optional[torch.Tensor] = None, candidates: int = 16,
